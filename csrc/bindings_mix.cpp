@@ -81,6 +81,13 @@ void gated_act(Tensor out, Tensor gu, int64_t kind, double limit, double alpha) 
                                (float)limit, (float)alpha, cur_stream()));
 }
 
+void gelu_act(Tensor out, Tensor z) {
+  const bool f = is_f32(z, "z");
+  TORCH_CHECK(is_f32(out, "out") == f && out.is_contiguous() && z.is_contiguous() && out.sizes() == z.sizes(),
+              "gelu_act: same dtype and shape, contiguous");
+  HIP_OK(die::launch_gelu_act(out.data_ptr(), z.data_ptr(), f, z.numel(), cur_stream()));
+}
+
 void route_sigmoid_topk(Tensor w, Tensor ids, Tensor x, Tensor wr) {
   check_rows(x, "x");
   const bool xf = is_f32(x, "x"), wf = is_f32(wr, "wr");
@@ -425,17 +432,20 @@ void moe_align(Tensor offsets, Tensor sorted, Tensor pos, Tensor ids, int64_t nu
 void register_seq_ops(pybind11::module& m);  // csrc/bindings_seq.cpp
 void register_lin_ops(pybind11::module& m);  // csrc/bindings_lin.cpp
 void register_rec_ops(pybind11::module& m);  // csrc/bindings_rec.cpp
+void register_conv_ops(pybind11::module& m);  // csrc/bindings_conv.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   register_seq_ops(m);
   register_lin_ops(m);
   register_rec_ops(m);
+  register_conv_ops(m);
   m.def("route_softmax_topk", &route_softmax_topk);
   m.def("topk_softmax_corrected", &topk_softmax_corrected);
   m.def("combine_weighted", &combine_weighted);
   m.def("rms_norm_ext", &rms_norm_ext);
   m.def("post_norm_residual", &post_norm_residual);
   m.def("gated_act", &gated_act);
+  m.def("gelu_act", &gelu_act);
   m.def("route_sigmoid_topk", &route_sigmoid_topk);
   m.def("topk_sigmoid", &topk_sigmoid);
   m.def("gather_scaled", &gather_scaled);

@@ -191,9 +191,10 @@ void exp_gate_scan(Tensor abe, Tensor x, int64_t ioff, int64_t foff, Tensor i_bi
                                    ragged(T, positions, cu_q, state_slots), cur_stream()));
 }
 
-void gated_linear_attn(Tensor out, OptTensor nq, Tensor x, int64_t qoff, int64_t koff, int64_t voff, Tensor ab,
+void gated_linear_attn(Tensor out, OptTensor nq, Tensor x, int64_t qoff, int64_t koff, int64_t voff, OptTensor ab,
                        Tensor state, OptTensor n_state, int64_t heads, int64_t groups, int64_t dim, int64_t vdim,
-                       double qscale, Tensor positions, OptTensor cu_q, Tensor state_slots) {
+                       double qscale, Tensor positions, OptTensor cu_q, Tensor state_slots, OptTensor z,
+                       OptTensor z_bias, double inv_tau) {
   check_rows(x, "x");
   const int64_t T = x.size(0);
   check_c(out, at::kFloat, "out");
@@ -203,8 +204,11 @@ void gated_linear_attn(Tensor out, OptTensor nq, Tensor x, int64_t qoff, int64_t
   TORCH_CHECK(qoff >= 0 && koff >= 0 && voff >= 0 && qoff + groups * dim <= x.size(1) &&
                   koff + groups * dim <= x.size(1) && voff + heads * vdim <= x.size(1),
               "q / k / v columns outside x");
-  check_c(ab, at::kFloat, "ab");
-  TORCH_CHECK(ab.dim() == 3 && ab.size(0) == T && ab.size(1) == heads && ab.size(2) >= 2, "ab [T, H, >= 2]");
+  TORCH_CHECK(ab.has_value() != z.has_value(), "ab (decay per head) or z (decay per row of the state)");
+  if (ab.has_value()) {
+    check_c(*ab, at::kFloat, "ab");
+    TORCH_CHECK(ab->dim() == 3 && ab->size(0) == T && ab->size(1) == heads && ab->size(2) >= 2, "ab [T, H, >= 2]");
+  }
   check_c(state, at::kFloat, "state");
   TORCH_CHECK(state.dim() == 4 && state.size(1) == heads && state.size(2) == dim && state.size(3) == vdim,
               "state [slots, H, dim, vdim]");
@@ -228,8 +232,21 @@ void gated_linear_attn(Tensor out, OptTensor nq, Tensor x, int64_t qoff, int64_t
   a.koff = (int)koff;
   a.voff = (int)voff;
   a.f32 = is_f32(x, "x");
-  a.ab = ab.data_ptr<float>();
-  a.abw = (int)ab.size(2);
+  a.ab = ab.has_value() ? ab->data_ptr<float>() : nullptr;
+  a.abw = ab.has_value() ? (int)ab->size(2) : 0;
+  a.z = nullptr;
+  a.zstride = 0;
+  a.z_bias = nullptr;
+  a.inv_tau = (float)inv_tau;
+  if (z.has_value()) {
+    check_rows(*z, "z");
+    TORCH_CHECK(is_f32(*z, "z") == a.f32 && z->size(0) == T && z->size(1) == heads * dim && z_bias.has_value() &&
+                    !n_state.has_value(),
+                "z [T, heads * dim] in x's dtype, with z_bias, without a normaliser");
+    a.z = z->data_ptr();
+    a.zstride = z->stride(0);
+    a.z_bias = f32_vec(z_bias, heads * dim, "z_bias");
+  }
   a.state = state.data_ptr<float>();
   a.heads = (int)heads;
   a.groups = (int)groups;
@@ -239,22 +256,38 @@ void gated_linear_attn(Tensor out, OptTensor nq, Tensor x, int64_t qoff, int64_t
   HIP_OK(die::launch_gated_linear_attn(a, ragged(T, positions, cu_q, state_slots), cur_stream()));
 }
 
-void head_norm_gate(Tensor out, Tensor o, Tensor nq, Tensor abe, Tensor g, Tensor w, int64_t heads, int64_t vdim,
-                    double eps) {
+void head_norm_gate(Tensor out, Tensor o, OptTensor nq, OptTensor abe, Tensor g, Tensor w, int64_t heads, int64_t vdim,
+                    double eps, bool gate_silu, double mult) {
+  die::HeadNormGateArgs a;
   check_c(o, at::kFloat, "o");
-  check_c(nq, at::kFloat, "nq");
-  check_c(abe, at::kFloat, "abe");
   TORCH_CHECK(o.dim() == 2 && o.size(1) == heads * vdim, "o [T, H * vdim]");
   const int64_t T = o.size(0);
-  TORCH_CHECK(nq.numel() == T * heads && abe.numel() == T * heads * 3, "nq [T, H], abe [T, H, 3]");
+  TORCH_CHECK(nq.has_value() == abe.has_value(), "nq and abe come together");
+  a.nq = a.abe = nullptr;
+  if (nq.has_value()) {
+    a.nq = f32_vec(nq, T * heads, "nq");
+    a.abe = f32_vec(abe, T * heads * 3, "abe");
+  }
   check_rows(g, "g");
-  const bool f = is_f32(g, "g");
+  a.f32 = is_f32(g, "g");
   TORCH_CHECK(g.size(0) == T && g.size(1) == heads * vdim, "g [T, H * vdim]");
-  TORCH_CHECK(is_f32(out, "out") == f && out.is_contiguous() && out.dim() == 2 && out.sizes() == o.sizes(),
-              "out [T, H * vdim] in g's dtype");
-  HIP_OK(die::launch_head_norm_gate(out.data_ptr(), o.data_ptr<float>(), nq.data_ptr<float>(), abe.data_ptr<float>(),
-                                    g.data_ptr(), g.stride(0), f, f32_vec(w, heads * vdim, "w"), (int)T, (int)heads,
-                                    (int)vdim, (float)eps, cur_stream()));
+  check_rows(out, "out");
+  TORCH_CHECK(is_f32(out, "out") == a.f32 && out.sizes() == o.sizes(), "out [T, H * vdim] in g's dtype");
+  TORCH_CHECK(w.numel() == vdim || w.numel() == heads * vdim, "w [vdim] or [H * vdim]");
+  a.w = f32_vec(w, w.numel(), "w");
+  a.w_shared = w.numel() != heads * vdim;
+  a.out = out.data_ptr();
+  a.ostride = out.stride(0);
+  a.o = o.data_ptr<float>();
+  a.g = g.data_ptr();
+  a.gstride = g.stride(0);
+  a.gate_silu = gate_silu;
+  a.T = (int)T;
+  a.heads = (int)heads;
+  a.vdim = (int)vdim;
+  a.eps = (float)eps;
+  a.mult = (float)mult;
+  HIP_OK(die::launch_head_norm_gate(a, cur_stream()));
 }
 
 void skip_gate_group_norm(Tensor out, Tensor o, Tensor x, Tensor D, Tensor z, Tensor w, int64_t heads, int64_t vdim,

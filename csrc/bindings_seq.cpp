@@ -159,29 +159,34 @@ die::DeltaShape delta_shape(int64_t heads, int64_t kv_heads, int64_t dim, int64_
 }
 
 // x [T, C], b [T, heads], a [T, heads]: column slices of ONE projection output (same row stride)
-void delta_prep(Tensor qkv32, Tensor bg, Tensor x, Tensor b, Tensor a, Tensor conv_w, OptTensor conv_wt,
-                Tensor conv_state, Tensor A_log, Tensor dt_bias, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, Tensor positions,
+void delta_prep(Tensor qkv32, Tensor bg, Tensor x, Tensor b, OptTensor a, Tensor conv_w, OptTensor conv_wt,
+                Tensor conv_state, OptTensor A_log, OptTensor dt_bias, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, Tensor positions,
                 OptTensor cu_q, Tensor state_slots) {
   TORCH_CHECK(conv_w.dim() == 2, "conv_w [C, taps]");
   auto sh = delta_shape(heads, kv_heads, dim, vdim, conv_w.size(1));
   const int64_t C = sh.channels(), T = x.size(0);
   check_rows(x, "x");
   check_rows(b, "b");
-  check_rows(a, "a");
   const bool f = is_f32(x, "x");
-  TORCH_CHECK(is_f32(b, "b") == f && is_f32(a, "a") == f, "one dtype");
-  TORCH_CHECK(x.size(1) == C && b.size(0) == T && a.size(0) == T && b.size(1) == heads && a.size(1) == heads &&
-                  b.stride(0) == x.stride(0) && a.stride(0) == x.stride(0),
-              "x [T, C], b / a [T, heads], slices of one projection");
+  TORCH_CHECK(is_f32(b, "b") == f, "one dtype");
+  TORCH_CHECK(x.size(1) == C && b.size(0) == T && b.size(1) == heads && b.stride(0) == x.stride(0),
+              "x [T, C], b [T, heads], slices of one projection");
+  if (a.has_value()) {
+    check_rows(*a, "a");
+    TORCH_CHECK(is_f32(*a, "a") == f && a->size(0) == T && a->size(1) == heads && a->stride(0) == x.stride(0) &&
+                    A_log.has_value() && dt_bias.has_value(),
+                "a [T, heads], a slice of the same projection, with A_log and dt_bias");
+  }
   check_c(qkv32, at::kFloat, "qkv32");
   check_c(bg, at::kFloat, "bg");
-  TORCH_CHECK(qkv32.numel() == T * C && bg.numel() == T * 2 * heads, "qkv32 [T, C], bg [T, 2 heads]");
+  TORCH_CHECK(qkv32.numel() == T * C && bg.numel() == T * (a.has_value() ? 2 : 1) * heads,
+              "qkv32 [T, C], bg [T, 2 heads] ([T, heads] without a)");
   check_c(conv_state, at::kFloat, "conv_state");
   TORCH_CHECK(conv_state.dim() == 3 && conv_state.size(1) == sh.taps - 1 && conv_state.size(2) == C,
               "conv_state [slots, taps - 1, C]");
   auto r = ragged(T, positions, cu_q, state_slots);
   HIP_OK(die::launch_delta_prep(qkv32.data_ptr<float>(), bg.data_ptr<float>(), x.data_ptr(), b.data_ptr(),
-                                a.data_ptr(), x.stride(0), f, f32_ptr(conv_w, C * sh.taps, "conv_w"),
+                                a.has_value() ? a->data_ptr() : nullptr, x.stride(0), f, f32_ptr(conv_w, C * sh.taps, "conv_w"),
                                 f32_ptr(conv_wt, C * sh.taps, "conv_wt"), conv_state.data_ptr<float>(), f32_ptr(A_log, heads, "A_log"),
                                 f32_ptr(dt_bias, heads, "dt_bias"), sh, r, cur_stream()));
 }
@@ -200,33 +205,58 @@ void conv_state_update(Tensor conv_state, Tensor x, int64_t heads, int64_t kv_he
 
 void gated_delta(Tensor out, Tensor qkv32, Tensor bg, Tensor gate, Tensor norm_w, double eps, Tensor state,
                  int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, Tensor positions, OptTensor cu_q,
-                 Tensor state_slots) {
-  auto sh = delta_shape(heads, kv_heads, dim, vdim, 1);
-  const int64_t C = sh.channels();
+                 Tensor state_slots, OptTensor z, OptTensor z_bias, OptTensor A_log, bool gate_sigmoid, double mult) {
+  die::GatedDeltaArgs a;
+  a.sh = delta_shape(heads, kv_heads, dim, vdim, 1);
+  const int64_t C = a.sh.channels();
   check_c(qkv32, at::kFloat, "qkv32");
   check_c(bg, at::kFloat, "bg");
   TORCH_CHECK(qkv32.dim() == 2 && qkv32.size(1) == C, "qkv32 [T, C]");
   const int64_t T = qkv32.size(0);
-  TORCH_CHECK(bg.numel() == T * 2 * heads, "bg [T, 2 heads]");
+  TORCH_CHECK(bg.numel() == T * (z.has_value() ? 1 : 2) * heads, "bg [T, 2 heads] ([T, heads] with z)");
   check_rows(gate, "gate");
-  const bool f = is_f32(gate, "gate");
+  a.f32 = is_f32(gate, "gate");
   TORCH_CHECK(gate.size(0) == T && gate.size(1) == heads * vdim, "gate [T, heads * vdim]");
-  TORCH_CHECK(is_f32(out, "out") == f && out.is_contiguous() && out.numel() == T * heads * vdim,
-              "out [T, heads * vdim] contiguous");
+  check_rows(out, "out");
+  TORCH_CHECK(is_f32(out, "out") == a.f32 && out.size(0) == T && out.size(1) == heads * vdim,
+              "out [T, heads * vdim] in gate's dtype");
   check_c(state, at::kFloat, "state");
   TORCH_CHECK(state.dim() == 4 && state.size(1) == heads && state.size(2) == dim && state.size(3) == vdim,
               "state [slots, heads, dim, vdim]");
-  auto r = ragged(T, positions, cu_q, state_slots);
-  HIP_OK(die::launch_gated_delta(out.data_ptr(), qkv32.data_ptr<float>(), bg.data_ptr<float>(), gate.data_ptr(),
-                                 gate.stride(0), f, f32_ptr(norm_w, vdim, "norm_w"), (float)eps,
-                                 state.data_ptr<float>(), sh, r, cur_stream()));
+  a.out = out.data_ptr();
+  a.ostride = out.stride(0);
+  a.qkv32 = qkv32.data_ptr<float>();
+  a.bg = bg.data_ptr<float>();
+  a.gate = gate.data_ptr();
+  a.gstride = gate.stride(0);
+  a.gate_sigmoid = gate_sigmoid;
+  a.z = nullptr;
+  a.zstride = 0;
+  a.z_bias = a.A_log = nullptr;
+  if (z.has_value()) {
+    check_rows(*z, "z");
+    TORCH_CHECK(is_f32(*z, "z") == a.f32 && z->size(0) == T && z->size(1) == heads * dim && z_bias.has_value() &&
+                    A_log.has_value(),
+                "z [T, heads * dim] in gate's dtype, with z_bias and A_log");
+    a.z = z->data_ptr();
+    a.zstride = z->stride(0);
+    a.z_bias = f32_ptr(z_bias, heads * dim, "z_bias");
+    a.A_log = f32_ptr(A_log, heads, "A_log");
+  }
+  a.norm_w = f32_ptr(norm_w, vdim, "norm_w");
+  a.eps = (float)eps;
+  a.mult = (float)mult;
+  a.state = state.data_ptr<float>();
+  HIP_OK(die::launch_gated_delta(a, ragged(T, positions, cu_q, state_slots), cur_stream()));
 }
 
 // q [T, H * dim], k [T, G * dim], v [T, G * vdim]: column slices of ONE projection output
 void qkv_prep(Tensor q_out, Tensor cache, Tensor q, Tensor k, OptTensor v, int64_t heads, int64_t kv_heads,
               int64_t dim, int64_t vdim, OptTensor q_norm, OptTensor k_norm, int64_t rot_dims, OptTensor inv_freq,
               bool v_unit, OptTensor v_lambda, OptTensor v_first, double eps, Tensor positions, Tensor slots,
-              bool head_norm, double q_temp_coef, int64_t q_temp_every, bool norm_after_rot) {
+              bool head_norm, double q_temp_coef, int64_t q_temp_every, bool norm_after_rot, OptTensor bias,
+              OptTensor conv_wt, OptTensor conv_state, OptTensor cu_q, OptTensor state_slots, double rot_gain,
+              OptTensor v_inv_freq) {
   check_rows(q, "q");
   check_rows(k, "k");
   die::QkvPrepArgs a;
@@ -274,6 +304,36 @@ void qkv_prep(Tensor q_out, Tensor cache, Tensor q, Tensor k, OptTensor v, int64
   a.rot_dims = (int)rot_dims;
   a.inv_freq = f32_ptr(inv_freq, rot_dims / 2, "inv_freq");
   a.v_unit = v_unit;
+  const int64_t C = heads * dim + kv_heads * (dim + vdim);
+  a.rot_gain = (float)rot_gain;
+  TORCH_CHECK(!v_inv_freq.has_value() || (vdim % 2 == 0 && v.has_value() && !v_unit), "rotated values: an even vdim");
+  a.v_inv_freq = f32_ptr(v_inv_freq, vdim / 2, "v_inv_freq");
+  a.bias = f32_ptr(bias, C, "bias");
+  a.conv_wt = nullptr;
+  a.conv_state = nullptr;
+  a.taps = 0;
+  a.r = die::RaggedRows{nullptr, nullptr, nullptr, 0, 0};
+  if (bias.has_value() || conv_wt.has_value()) {
+    const int64_t es = q.element_size();
+    const char* q0 = static_cast<const char*>(q.data_ptr());
+    TORCH_CHECK(v.has_value() && !v_lambda.has_value() && !(bias.has_value() && conv_wt.has_value()) &&
+                    static_cast<const char*>(k.data_ptr()) == q0 + heads * dim * es &&
+                    static_cast<const char*>(v->data_ptr()) == q0 + (heads + kv_heads) * dim * es,
+                "bias / conv: q, k and v in adjacent columns, one of the two, no value mixing");
+  }
+  if (conv_wt.has_value()) {
+    check_c(*conv_wt, at::kFloat, "conv_wt");
+    TORCH_CHECK(conv_wt->dim() == 2 && conv_wt->size(1) == C && conv_wt->size(0) >= 1 && conv_wt->size(0) <= 16,
+                "conv_wt [taps, C], taps <= 16");
+    TORCH_CHECK(conv_state.has_value() && state_slots.has_value(), "conv needs conv_state and state_slots");
+    check_c(*conv_state, at::kFloat, "conv_state");
+    a.taps = (int)conv_wt->size(0);
+    TORCH_CHECK(conv_state->dim() == 3 && conv_state->size(1) == a.taps - 1 && conv_state->size(2) == C,
+                "conv_state [slots, taps - 1, C]");
+    a.conv_wt = conv_wt->data_ptr<float>();
+    a.conv_state = conv_state->data_ptr<float>();
+    a.r = ragged(T, positions, cu_q, *state_slots);
+  }
   a.v_lambda = f32_ptr(v_lambda, 1, "v_lambda");
   a.v_first = nullptr;
   a.vfstride = 0;
@@ -296,7 +356,7 @@ void qkv_prep(Tensor q_out, Tensor cache, Tensor q, Tensor k, OptTensor v, int64
 void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTensor cu_q, Tensor ctx_lens,
                Tensor positions, OptTensor sink, OptTensor bias, int64_t max_q, int64_t heads, int64_t kv_heads,
                int64_t dim, int64_t vdim, int64_t window, double scale, int64_t impl, double softcap,
-               OptTensor slopes) {
+               OptTensor slopes, int64_t seg) {
   die::SinkAttnArgs a;
   a.f32 = is_f32(q, "q");
   TORCH_CHECK(is_f32(out, "out") == a.f32 && is_f32(cache, "cache") == a.f32, "one dtype");
@@ -347,7 +407,9 @@ void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTenso
   a.dim = (int)dim;
   a.vdim = (int)vdim;
   a.block_size = (int)cache.size(1);
+  TORCH_CHECK(window >= 0 && seg >= 0, "window, seg >= 0");
   a.window = (int)window;
+  a.seg = (int)seg;
   a.scale = (float)scale;
   a.impl = (int)impl;
   a.ws_o = a.ws_ml = nullptr;
@@ -358,6 +420,7 @@ void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTenso
   // length; splits beyond a sequence's keys exit at once)
   int64_t bound = block_tables.size(1) * cache.size(1);
   if (window > 0) bound = std::min<int64_t>(bound, window + max_q);
+  if (seg > 0) bound = std::min<int64_t>(bound, seg + max_q);
   int64_t ns = 1;
   if (die::sink_attn_uses_decode(a)) {
     // decode steps: a workgroup per (sequence, key/value head, split); trips of 128 keys, splits until about 2048

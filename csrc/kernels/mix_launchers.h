@@ -23,6 +23,9 @@ hipError_t launch_post_norm_residual(float* resid, void* act, const void* y, int
 hipError_t launch_gated_act(void* out, const void* gu, bool f32, int rows, int f, int kind, float limit, float alpha,
                             hipStream_t s);
 
+// out[i] = 0.5 z[i] (1 + erf(z[i] / sqrt 2)), n contiguous elements
+hipError_t launch_gelu_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s);
+
 // Router: z = x . Wr[e] in fp32, score = sigmoid(z), the K largest per token (lowest index on ties);
 // w [T, K] fp32 = the chosen scores (not renormalised), ids [T, K] int32
 hipError_t launch_route_sigmoid_topk(float* w, int* ids, const void* x, int64_t xstride, bool x_f32, const void* wr,

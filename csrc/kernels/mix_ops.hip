@@ -4,6 +4,7 @@
 //
 //   rms_norm_ext          y = x / sqrt(mean(x^2) + eps) * (w | 1 + w)
 //   post_norm_residual    resid(fp32) += rmsnorm(y) * (w | 1 + w); optional bf16 copy of the new residual
+//   gelu_act              0.5 z (1 + erf(z / sqrt 2))
 //   gated_act             silu(g) * u, or the clamped variant g' * sigmoid(alpha g') * (u' + 1)
 //   route_sigmoid_topk    router logits (fp32), sigmoid scores, top-K without renormalisation
 //   gather_scaled         expert input rows scaled by their routing weight
@@ -123,6 +124,25 @@ __global__ void __launch_bounds__(NT) gated_act_kernel(void* out, const void* gu
   }
   for (int c = threadIdx.x; c < f; c += NT)
     stv(out, r * f + c, f32, gate1(ldv(gu, r * 2 * f + c, f32), ldv(gu, r * 2 * f + f + c, f32), kind, limit, alpha));
+}
+
+// the exact (erf) GELU
+__device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
+// grid-stride over the flattened tensor; bf16 with a multiple of 8 elements: 16 bytes per access
+__global__ void __launch_bounds__(NT) gelu_act_kernel(void* out, const void* z, bool f32, int64_t n) {
+  const int64_t stride = (int64_t)gridDim.x * NT, i0 = (int64_t)blockIdx.x * NT + threadIdx.x;
+  if (!f32 && n % 8 == 0 && aligned16(z) && aligned16(out)) {
+    for (int64_t c = i0; c < n / 8; c += stride) {
+      float v[8];
+      unpack8(reinterpret_cast<const uint4*>(z)[c], v);
+#pragma unroll
+      for (int q = 0; q < 8; ++q) v[q] = gelu_erf(v[q]);
+      reinterpret_cast<uint4*>(out)[c] = pack8(v);
+    }
+    return;
+  }
+  for (int64_t c = i0; c < n; c += stride) stv(out, c, f32, gelu_erf(ldv(z, c, f32)));
 }
 
 constexpr int ROUTE_E_MAX = 256;
@@ -571,6 +591,13 @@ hipError_t launch_gated_act(void* out, const void* gu, bool f32, int rows, int f
   if (rows == 0) return hipSuccess;
   if (f <= 0 || kind < 0 || kind > 2) return hipErrorInvalidValue;
   hipLaunchKernelGGL(gated_act_kernel, dim3(rows), dim3(NT), 0, s, out, gu, f32, f, kind, limit, alpha);
+  return hipGetLastError();
+}
+
+hipError_t launch_gelu_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s) {
+  if (n == 0) return hipSuccess;
+  const int64_t blocks = (n / (f32 ? 1 : 8) + NT - 1) / NT + 1;
+  hipLaunchKernelGGL(gelu_act_kernel, dim3((unsigned)(blocks < 16384 ? blocks : 16384)), dim3(NT), 0, s, out, z, f32, n);
   return hipGetLastError();
 }
 

@@ -81,22 +81,40 @@ struct GatedLinearArgs {
   int64_t xstride;
   int qoff, koff, voff;
   bool f32;
-  const float* ab;         // [T, H, abw]: (a, b) = the first two entries
+  const float* ab;         // [T, H, abw]: (a, b) = the first two entries; not read with z
   int abw;
+  // z != nullptr: b = 1 and a decay per row of S, a = sigmoid(z + z_bias)^inv_tau
+  const void* z;           // [T, H * dim], row stride zstride, x's type
+  int64_t zstride;
+  const float* z_bias;     // [H * dim]
+  float inv_tau;
   float* state;            // [slots, H, dim, vdim]
   float* n_state;          // [slots, H, dim] or nullptr
   int heads, groups, dim, vdim;
   float qscale;
 };
-// Per (sequence, head), token by token: S <- a S + b k v^T; o = S^T (q * qscale); with n_state also
+// Per (sequence, head), token by token: S <- a S + b k v^T (with z: row i of S by its own a_i); o = S^T (q * qscale);
+// with n_state also
 // n <- a n + b k and nq = n . (q * qscale). Head h reads q and k of group h / (heads / groups).
 hipError_t launch_gated_linear_attn(const GatedLinearArgs& a, RaggedRows r, hipStream_t s);
 
-// out[t, h, :] = rms(o[t, h, :] / (max(|nq[t, h]|, abe[t, h, 2]) + 1e-6)) * w[h, :] * sigmoid(g[t, h, :]); o fp32,
-// g (row stride gstride) and out in the activation type
-hipError_t launch_head_norm_gate(void* out, const float* o, const float* nq, const float* abe, const void* g,
-                                 int64_t gstride, bool f32, const float* w, int T, int H, int vdim, float eps,
-                                 hipStream_t s);
+struct HeadNormGateArgs {
+  void* out;               // [T, H * vdim], row stride ostride, g's type
+  int64_t ostride;
+  const float* o;          // [T, H * vdim]
+  const float* nq;         // [T, H] with abe [T, H, 3], or nullptr: o / (max(|nq|, abe[.., 2]) + 1e-6) first
+  const float* abe;
+  const void* g;           // [T, H * vdim], row stride gstride
+  int64_t gstride;
+  bool f32;
+  bool gate_silu;          // SiLU(g), else sigmoid(g)
+  const float* w;          // [H * vdim], or [vdim] shared by the heads
+  bool w_shared;
+  int T, heads, vdim;
+  float eps, mult;
+};
+// out[t, h, :] = mult * rms(o[t, h, :]) * w * gate(g[t, h, :])
+hipError_t launch_head_norm_gate(const HeadNormGateArgs& a, hipStream_t s);
 
 // y = (o + D[h] * x) * silu(z); out = rms(y) over each of `parts` equal parts of the row * w; o fp32 [T, H * vdim];
 // x, z (row strides xstride / zstride) and out in the activation type

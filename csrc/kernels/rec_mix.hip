@@ -11,8 +11,9 @@
 //   exp_gate_scan             log-space input / forget gates under a running maximum: a wave-wide scan over tokens
 //   gated_linear_attn         S <- a S + b k v^T, o = S^T q: one workgroup per (sequence, head, block of columns), the
 //                             state in registers (a column per lane quad); the normaliser n <- a n + b k with its
-//                             read-out n . q rides on the first wave
-//   head_norm_gate            o / (max(|n . q|, floor) + 1e-6), per-head RMS norm, weight, sigmoid gate
+//                             read-out n . q rides on the first wave; optionally a decay per row of S,
+//                             sigmoid(z)^(1/tau), computed while a trip is staged
+//   head_norm_gate            (o / (max(|n . q|, floor) + 1e-6), optional,) per-head RMS norm, weight, sigmoid or SiLU gate
 //   skip_gate_group_norm      (o + D x) * silu(z), RMS norm in equal parts of the row, weight
 //   pair_post_norm_residual   resid += mult * rms((rms(y1) w1 + rms(y2) w2) / 2) * (1 + w)
 #include "common.h"
@@ -409,7 +410,8 @@ __global__ void __launch_bounds__(64) exp_gate_scan_kernel(float* abe, const voi
 // block 0, which runs a trip's tokens over the staged k and q once more after its columns and reduces the TB dot
 // products n . q over its lanes. (As a column of its own the normaliser would add a ninth wave to workgroups of 512
 // threads; measured, that ran 1.8x slower than the kernel without it, and a one-wave launch beside it 1.7x.)
-template <int DP, bool F32>
+// CD: a decay per row of the state instead of one per head.
+template <int DP, bool F32, bool CD>
 __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs a, RaggedRows r, int VC) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   constexpr int DPAD = 4 * DP;
@@ -417,7 +419,7 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
   float* qs = sm;                  // [TB][DPAD], zero beyond dim
   float* ks = qs + TB * DPAD;      // [TB][DPAD]
   float* vs = ks + TB * DPAD;      // [TB][VC]
-  float* as = vs + TB * VC;        // [TB][2]: a, b
+  float* as = vs + TB * VC;        // [TB][2]: a, b, or [TB][DPAD]: a per row of S
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x;
   const int v0 = blockIdx.z * VC;
   const int ncol = min(VC, dv - v0);
@@ -435,7 +437,7 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
     S[i] = (!fresh && row < d && j < ncol) ? st[(int64_t)row * dv] : 0.f;
   }
   constexpr int RP = DPAD > 64 ? DPAD / 64 : 1;
-  const bool norm = a.n_state != nullptr && blockIdx.z == 0 && tid < 64;   // wave-uniform
+  const bool norm = !CD && a.n_state != nullptr && blockIdx.z == 0 && tid < 64;   // wave-uniform
   float* nst = norm ? a.n_state + ((int64_t)r.state_slots[s] * H + h) * d : nullptr;
   float nv[RP];
 #pragma unroll
@@ -448,27 +450,36 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
       const int64_t base = (int64_t)(q0 + t0 + tt) * a.xstride + g * d + c;
       qs[e] = c < d ? ldt<F32>(a.x, base + a.qoff) * a.qscale : 0.f;
       ks[e] = c < d ? ldt<F32>(a.x, base + a.koff) : 0.f;
+      if (CD) {
+        // sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau)
+        const float z = c < d ? ldt<F32>(a.z, (int64_t)(q0 + t0 + tt) * a.zstride + h * d + c) + a.z_bias[h * d + c] : 0.f;
+        as[e] = c < d ? expf(-step_size<!F32>(-z) * a.inv_tau) : 0.f;
+      }
     }
     for (int e = tid; e < nb * VC; e += nthr) {
       const int tt = e / VC, c = e % VC;
       vs[e] = c < ncol ? ldt<F32>(a.x, (int64_t)(q0 + t0 + tt) * a.xstride + a.voff + h * dv + v0 + c) : 0.f;
     }
-    for (int e = tid; e < 2 * nb; e += nthr) as[e] = a.ab[((int64_t)(q0 + t0 + (e >> 1)) * H + h) * a.abw + (e & 1)];
+    for (int e = tid; !CD && e < 2 * nb; e += nthr) as[e] = a.ab[((int64_t)(q0 + t0 + (e >> 1)) * H + h) * a.abw + (e & 1)];
     __syncthreads();
     for (int tt = 0; tt < nb; ++tt) {
       const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD + part * DP);
       const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD + part * DP);
-      const float2 ab = *reinterpret_cast<const float2*>(as + 2 * tt);
-      const float vj = (j < ncol ? vs[tt * VC + j] : 0.f) * ab.y;
-      const float dec = ab.x;
+      const float4* at = reinterpret_cast<const float4*>(as + tt * DPAD + part * DP);
+      float vj = j < ncol ? vs[tt * VC + j] : 0.f, dec = 1.0f;
+      if (!CD) {
+        const float2 ab = *reinterpret_cast<const float2*>(as + 2 * tt);
+        vj *= ab.y;
+        dec = ab.x;
+      }
       float o0 = 0.f, o1 = 0.f;
 #pragma unroll
       for (int i = 0; i < DP / 4; ++i) {
-        const float4 k4 = kt[i], q4 = qt[i];
-        S[4 * i] = S[4 * i] * dec + k4.x * vj;
-        S[4 * i + 1] = S[4 * i + 1] * dec + k4.y * vj;
-        S[4 * i + 2] = S[4 * i + 2] * dec + k4.z * vj;
-        S[4 * i + 3] = S[4 * i + 3] * dec + k4.w * vj;
+        const float4 k4 = kt[i], q4 = qt[i], a4 = CD ? at[i] : make_float4(dec, dec, dec, dec);
+        S[4 * i] = S[4 * i] * a4.x + k4.x * vj;
+        S[4 * i + 1] = S[4 * i + 1] * a4.y + k4.y * vj;
+        S[4 * i + 2] = S[4 * i + 2] * a4.z + k4.z * vj;
+        S[4 * i + 3] = S[4 * i + 3] * a4.w + k4.w * vj;
         o0 += S[4 * i] * q4.x + S[4 * i + 2] * q4.z;
         o1 += S[4 * i + 1] * q4.y + S[4 * i + 3] * q4.w;
       }
@@ -518,17 +529,23 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
   }
 }
 
-template <int DP, bool F32> hipError_t launch_gla_dp(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
+template <int DP, bool F32, bool CD> hipError_t launch_gla_one(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
   const int VC = a.vdim < 128 ? a.vdim : 128;
   const int nvc = (a.vdim + VC - 1) / VC;
   const int threads = (4 * VC + 63) / 64 * 64;
-  const size_t smem = (size_t)(2 * TB * 4 * DP + TB * VC + 2 * TB) * sizeof(float);
-  hipLaunchKernelGGL((gated_linear_attn_kernel<DP, F32>), dim3(a.heads, r.num_seqs, nvc), dim3(threads), smem, s, a, r,
-                     VC);
+  const size_t smem = (size_t)((CD ? 3 : 2) * TB * 4 * DP + (TB * VC + 3) / 4 * 4 + 2 * TB) * sizeof(float);
+  if (smem > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gated_linear_attn_kernel<DP, F32, CD>),
+                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    if (e != hipSuccess) return e;
+  }
+  hipLaunchKernelGGL((gated_linear_attn_kernel<DP, F32, CD>), dim3(a.heads, r.num_seqs, nvc), dim3(threads), smem, s, a,
+                     r, VC);
   return hipGetLastError();
 }
 template <int DP> hipError_t launch_gla_dp(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
-  return a.f32 ? launch_gla_dp<DP, true>(a, r, s) : launch_gla_dp<DP, false>(a, r, s);
+  if (a.z != nullptr) return a.f32 ? launch_gla_one<DP, true, true>(a, r, s) : launch_gla_one<DP, false, true>(a, r, s);
+  return a.f32 ? launch_gla_one<DP, true, false>(a, r, s) : launch_gla_one<DP, false, false>(a, r, s);
 }
 
 // ------------------------------------------------------------------------------------------------ epilogues
@@ -553,15 +570,16 @@ __device__ __forceinline__ float4 f4(const float* p, int64_t i) { return *reinte
 
 // One workgroup per token; 16 lanes per head, 16 heads at a time. vec: head sizes and strides that are multiples of
 // 4 with aligned bases, 4 values per lane and trip.
-__global__ void __launch_bounds__(NT) head_norm_gate_kernel(void* out, const float* o, const float* nq,
-                                                           const float* abe, const void* g, int64_t gstride, bool f32,
-                                                           const float* w, int H, int dv, float eps, bool vec) {
+__global__ void __launch_bounds__(NT) head_norm_gate_kernel(HeadNormGateArgs a, bool vec) {
   const int64_t t = blockIdx.x;
   const int gl = threadIdx.x & 15, grp = threadIdx.x >> 4;
+  const int H = a.heads, dv = a.vdim;
+  const bool f32 = a.f32;
   for (int h = grp; h < H; h += NT / 16) {
-    const float den = fmaxf(fabsf(nq[t * H + h]), abe[(t * H + h) * 3 + 2]) + 1e-6f;
-    const float inv = 1.0f / den;
-    const float* oh = o + (t * H + h) * dv;
+    float inv = 1.0f;
+    if (a.nq != nullptr) inv = 1.0f / (fmaxf(fabsf(a.nq[t * H + h]), a.abe[(t * H + h) * 3 + 2]) + 1e-6f);
+    const float* oh = a.o + (t * H + h) * dv;
+    const float* w = a.w + (a.w_shared ? 0 : h * dv);
     float ss = 0.f;
     if (vec) {
       for (int c = 4 * gl; c < dv; c += 64) {
@@ -576,18 +594,19 @@ __global__ void __launch_bounds__(NT) head_norm_gate_kernel(void* out, const flo
     }
 #pragma unroll
     for (int off = 8; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
-    const float rsn = inv / sqrtf(ss / (float)dv + eps);
+    const float rsn = a.mult * inv / sqrtf(ss / (float)dv + a.eps);
+    auto gate = [&](float g) { return a.gate_silu ? siluf(g) : sigmoidf(g); };
     if (vec) {
       for (int c = 4 * gl; c < dv; c += 64) {
-        const float4 u = f4(oh, c), ww = f4(w, h * dv + c), gt = ld4(g, t * gstride + h * dv + c, f32);
-        st4(out, (t * H + h) * dv + c, f32,
-            make_float4(u.x * rsn * ww.x * sigmoidf(gt.x), u.y * rsn * ww.y * sigmoidf(gt.y),
-                        u.z * rsn * ww.z * sigmoidf(gt.z), u.w * rsn * ww.w * sigmoidf(gt.w)));
+        const float4 u = f4(oh, c), ww = f4(w, c), gt = ld4(a.g, t * a.gstride + h * dv + c, f32);
+        st4(a.out, t * a.ostride + h * dv + c, f32,
+            make_float4(u.x * rsn * ww.x * gate(gt.x), u.y * rsn * ww.y * gate(gt.y), u.z * rsn * ww.z * gate(gt.z),
+                        u.w * rsn * ww.w * gate(gt.w)));
       }
     } else {
       for (int c = gl; c < dv; c += 16) {
-        const float gt = ldv(g, t * gstride + h * dv + c, f32);
-        stv(out, (t * H + h) * dv + c, f32, oh[c] * rsn * w[h * dv + c] * sigmoidf(gt));
+        const float gt = ldv(a.g, t * a.gstride + h * dv + c, f32);
+        stv(a.out, t * a.ostride + h * dv + c, f32, oh[c] * rsn * w[c] * gate(gt));
       }
     }
   }
@@ -775,7 +794,8 @@ hipError_t launch_exp_gate_scan(float* abe, const void* x, int64_t xstride, int 
 hipError_t launch_gated_linear_attn(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
   if (r.num_seqs == 0 || r.total_rows == 0) return hipSuccess;
   if (!rows_ok(r) || a.heads < 1 || a.groups < 1 || a.heads % a.groups || a.dim < 1 || a.dim > 256 || a.vdim < 1 ||
-      a.abw < 2 || (a.n_state != nullptr) != (a.nq != nullptr))
+      (a.z == nullptr && (a.ab == nullptr || a.abw < 2)) || (a.n_state != nullptr) != (a.nq != nullptr) ||
+      (a.z != nullptr && (a.z_bias == nullptr || a.n_state != nullptr)))
     return hipErrorInvalidValue;
   if (a.dim <= 16) return launch_gla_dp<4>(a, r, s);
   if (a.dim <= 32) return launch_gla_dp<8>(a, r, s);
@@ -784,16 +804,13 @@ hipError_t launch_gated_linear_attn(const GatedLinearArgs& a, RaggedRows r, hipS
   return launch_gla_dp<64>(a, r, s);
 }
 
-hipError_t launch_head_norm_gate(void* out, const float* o, const float* nq, const float* abe, const void* g,
-                                 int64_t gstride, bool f32, const float* w, int T, int H, int vdim, float eps,
-                                 hipStream_t s) {
-  if (T == 0) return hipSuccess;
-  if (H < 1 || vdim < 1) return hipErrorInvalidValue;
-  const bool vec = vdim % 4 == 0 && gstride % 4 == 0 && (reinterpret_cast<uintptr_t>(g) & 15) == 0 &&
-                   (reinterpret_cast<uintptr_t>(o) & 15) == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0 &&
-                   (reinterpret_cast<uintptr_t>(out) & 15) == 0;
-  hipLaunchKernelGGL(head_norm_gate_kernel, dim3(T), dim3(NT), 0, s, out, o, nq, abe, g, gstride, f32, w, H, vdim, eps,
-                     vec);
+hipError_t launch_head_norm_gate(const HeadNormGateArgs& a, hipStream_t s) {
+  if (a.T == 0) return hipSuccess;
+  if (a.heads < 1 || a.vdim < 1 || (a.nq != nullptr && a.abe == nullptr)) return hipErrorInvalidValue;
+  auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = a.vdim % 4 == 0 && a.gstride % 4 == 0 && a.ostride % 4 == 0 && a16(a.g) && a16(a.o) && a16(a.w) &&
+                   a16(a.out);
+  hipLaunchKernelGGL(head_norm_gate_kernel, dim3(a.T), dim3(NT), 0, s, a, vec);
   return hipGetLastError();
 }
 

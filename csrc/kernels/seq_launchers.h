@@ -65,7 +65,7 @@ struct DeltaShape {
 // Per row: the short causal convolution (+ SiLU) of the C = [q | k | v] channels of x, with the taps - 1 inputs
 // before the step taken from conv_state [slots, taps - 1, C] (fp32, the most recent last); q and k heads made
 // unit vectors (q also times dim^-1/2); beta = sigmoid(b), g = exp(-exp(A_log) * softplus(a + dt_bias)).
-// Writes qkv32 [T, C] and bg [T, 2 * heads] = [beta | g], both fp32. A step with one row per sequence
+// Writes qkv32 [T, C] and bg [T, 2 * heads] = [beta | g], both fp32; a == nullptr: no per-head decay, bg [T, heads] = beta. A step with one row per sequence
 // (cu_q == nullptr) also moves the row's input into conv_state. conv_w is [C, taps]; conv_wt, optional, the same
 // weights tap-major ([taps, C]), which lets prompt-sized bf16 steps load them 16 bytes at a time.
 hipError_t launch_delta_prep(float* qkv32, float* bg, const void* x, const void* b, const void* a, int64_t xstride,
@@ -74,11 +74,28 @@ hipError_t launch_delta_prep(float* qkv32, float* bg, const void* x, const void*
 // conv_state[slot(s)] = the last taps - 1 inputs of sequence s after this step (nothing to do when cu_q == nullptr)
 hipError_t launch_conv_state_update(float* conv_state, const void* x, int64_t xstride, bool f32, DeltaShape sh,
                                     RaggedRows r, hipStream_t s);
-// Per (sequence, head), token by token: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, with
-// S [dim, vdim] fp32 kept in state [slots, heads, dim, vdim]. out[t, h, :] = o / rms(o) * norm_w * silu(gate[t, h, :]).
-hipError_t launch_gated_delta(void* out, const float* qkv32, const float* bg, const void* gate, int64_t gstride,
-                              bool f32, const float* norm_w, float eps, float* state, DeltaShape sh, RaggedRows r,
-                              hipStream_t s);
+struct GatedDeltaArgs {
+  void* out;              // [T, H * vdim], row stride ostride, gate's type
+  int64_t ostride;
+  const float* qkv32;     // [T, C]
+  const float* bg;        // [T, 2 H] = [beta | decay per head], or [T, H] = beta with a decay per key channel
+  const void* gate;       // [T, H * vdim], row stride gstride
+  int64_t gstride;
+  bool gate_sigmoid;      // output gate: sigmoid, else SiLU
+  // decay per key channel exp(-exp(A_log[h]) * softplus(z + z_bias)), or z == nullptr: the per-head decays in bg
+  const void* z;          // [T, H * dim], row stride zstride, gate's type
+  int64_t zstride;
+  const float* z_bias;    // [H * dim]
+  const float* A_log;     // [H]
+  bool f32;
+  const float* norm_w;    // [vdim]
+  float eps, mult;
+  float* state;           // [slots, heads, dim, vdim]
+  DeltaShape sh;
+};
+// Per (sequence, head), token by token: S <- g S (g per head, or per row of S); u = beta (v - S^T k); S <- S + k u^T;
+// o = S^T q, with S [dim, vdim] fp32. out[t, h, :] = mult * o / rms(o) * norm_w * gate function(gate[t, h, :]).
+hipError_t launch_gated_delta(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s);
 
 struct QkvPrepArgs {
   const void* q;          // [T, H * dim], [T, G * dim], [T, G * vdim]: slices of one projection, row stride xstride
@@ -91,6 +108,16 @@ struct QkvPrepArgs {
   const float* k_norm;
   bool head_norm;         // q_norm and k_norm are [dim], shared by all heads: RMS norm of every head by itself
   bool norm_after_rot;    // with head_norm: the rotation comes first and the norm acts on the rotated heads
+  // optional, for q, k and v in adjacent columns (C = H * dim + G * (dim + vdim) channels): a bias [C] of the projection,
+  // or a short causal convolution with tap-major weights [taps, C] over the sequence, whose inputs before the step come
+  // from conv_state [slots, taps - 1, C] (fp32); a step with one row per sequence also moves the row's input in
+  const float* bias;
+  const float* conv_wt;
+  float* conv_state;
+  int taps;
+  RaggedRows r;           // with conv_wt
+  float rot_gain;         // factor of the cosines and sines of q and k
+  const float* v_inv_freq;  // [vdim / 2]: values turned by position * v_inv_freq[i] over pairs (i, i + vdim / 2), or nullptr
   float q_temp_coef;      // != 0: q, after its norm, times 1 + coef * ln(floor((p + 1) / q_temp_every) + 1) at position p
   int q_temp_every;
   int rot_dims;           // rotated dims per head (pairs i, i + rot_dims / 2), 0: none
@@ -124,6 +151,7 @@ struct SinkAttnArgs {
   const float* slopes;    // [H] or nullptr: slopes[h] * n is taken off the score of a key at distance n
   int num_seqs, total_q, max_q, heads, kv_heads, dim, vdim, block_size;
   int window;             // keys j with 0 <= p - j < window (0: all j <= p)
+  int seg;                // > 0: and floor(j / seg) = floor(p / seg)
   float scale;
   bool f32;
   int impl;               // 0: the decode-step kernel or matrix cores where they apply, else FMA; 1: FMA;

@@ -6,11 +6,12 @@
 //   store_last_token    the step's last token of every sequence -> state (the next step's "previous token")
 //   stream_mix_norm     streams <- mix^T streams + out * y, and the next sublayer's input rmsnorm(in . streams) * g
 //   poly_norm_act       c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3
-//   delta_prep          short conv + SiLU of q/k/v, unit q/k, beta and decay of the gated delta rule
+//   delta_prep          short conv + SiLU of q/k/v, unit q/k, beta (and the per-head decay) of the gated delta rule
 //   conv_state_update   the convolution's trailing inputs -> state
 //   gated_delta         the recurrence itself, one workgroup per (sequence, head), the state in registers (a
 //                       column per lane quad)
-//   qkv_prep            q/k norm, rotate-half rotary, value norm / value mixing, paged cache write
+//   qkv_prep            projection bias or short conv, q/k norm, rotate-half rotary (optionally of the values too),
+//                       value norm / value mixing, paged cache write
 #include "common.h"
 #include "seq_launchers.h"
 
@@ -30,6 +31,8 @@ __device__ __forceinline__ void stv(void* p, int64_t i, bool f32, float v) {
 // the value as the activation dtype would hold it
 __device__ __forceinline__ float rnd(float v, bool f32) { return f32 ? v : bf2f(f2bf(v)); }
 __device__ __forceinline__ float siluf(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 constexpr int NT = 256;
 
@@ -313,6 +316,72 @@ __global__ void __launch_bounds__(NT) poly_norm_act_kernel(void* out, const void
 // ------------------------------------------------------------------------------------------ gated delta rule
 constexpr int TAPS_MAX = 16;
 
+// A row of a short causal convolution over the sequence: row `row` of x is row i of its sequence in this step, at
+// position p; inputs before the step come from st [taps - 1, C] (the most recent last), inputs before the sequence's
+// start are zero. 8 channels (bf16 rows, tap-major weights, 16-byte loads):
+__device__ __forceinline__ void conv8(float* acc, const bf16_t* x, int64_t row, int64_t xstride, int c8, const float* st,
+                                      const float* wt, int taps, int C, int i, int64_t p) {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+  for (int j = 0; j < taps; ++j) {
+    const int back = taps - 1 - j;
+    if (p - back < 0) continue;
+    const int src = i - back;
+    float xv[8];
+    if (src >= 0) {
+      unpack8(*reinterpret_cast<const uint4*>(x + (row - back) * xstride + 8 * c8), xv);
+    } else {
+      const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(taps - 1 + src) * C + 8 * c8);
+      const float4 s0 = sp[0], s1 = sp[1];
+      xv[0] = s0.x, xv[1] = s0.y, xv[2] = s0.z, xv[3] = s0.w, xv[4] = s1.x, xv[5] = s1.y, xv[6] = s1.z, xv[7] = s1.w;
+    }
+    const float4* wp = reinterpret_cast<const float4*>(wt + (int64_t)j * C + 8 * c8);
+    const float4 w0 = wp[0], w1 = wp[1];
+    acc[0] += w0.x * xv[0], acc[1] += w0.y * xv[1], acc[2] += w0.z * xv[2], acc[3] += w0.w * xv[3];
+    acc[4] += w1.x * xv[4], acc[5] += w1.y * xv[5], acc[6] += w1.z * xv[6], acc[7] += w1.w * xv[7];
+  }
+}
+// One row per sequence: the calling thread is the only reader of its channels' tail, so it shifts it: state row k takes
+// row k + 1 (zeros where that lies before the sequence's start), the last one the row's input.
+__device__ __forceinline__ void conv8_shift(const bf16_t* x, int64_t row, int64_t xstride, int c8, float* st, int taps,
+                                            int C, int64_t p) {
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  for (int k = 0; k + 1 < taps - 1; ++k) {
+    const bool live = p - (taps - 2 - k) >= 0;
+    float4* dp = reinterpret_cast<float4*>(st + (int64_t)k * C + 8 * c8);
+    const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(k + 1) * C + 8 * c8);
+    const float4 t0 = sp[0], t1 = sp[1];
+    dp[0] = live ? t0 : zero;
+    dp[1] = live ? t1 : zero;
+  }
+  if (taps > 1) {
+    float xv[8];
+    unpack8(*reinterpret_cast<const uint4*>(x + row * xstride + 8 * c8), xv);
+    float4* dp = reinterpret_cast<float4*>(st + (int64_t)(taps - 2) * C + 8 * c8);
+    dp[0] = make_float4(xv[0], xv[1], xv[2], xv[3]);
+    dp[1] = make_float4(xv[4], xv[5], xv[6], xv[7]);
+  }
+}
+// the same for one channel; wc / wj: strides of the weight's channel and tap
+__device__ __forceinline__ float conv1(const void* x, bool f32, int64_t row, int64_t xstride, int c, const float* st,
+                                       const float* w, int64_t wc, int64_t wj, int taps, int C, int i, int64_t p) {
+  float acc = 0.f;
+  for (int j = 0; j < taps; ++j) {
+    const int back = taps - 1 - j;
+    if (p - back < 0) continue;
+    const int src = i - back;
+    const float xv = src >= 0 ? ldv(x, (row - back) * xstride + c, f32) : st[(int64_t)(taps - 1 + src) * C + c];
+    acc += w[c * wc + j * wj] * xv;
+  }
+  return acc;
+}
+__device__ __forceinline__ void conv1_shift(const void* x, bool f32, int64_t row, int64_t xstride, int c, float* st,
+                                            int taps, int C, int64_t p) {
+  for (int k = 0; k + 1 < taps - 1; ++k)
+    st[(int64_t)k * C + c] = p - (taps - 2 - k) >= 0 ? st[(int64_t)(k + 1) * C + c] : 0.f;
+  if (taps > 1) st[(int64_t)(taps - 2) * C + c] = ldv(x, row * xstride + c, f32);
+}
+
 __global__ void __launch_bounds__(NT) delta_prep_kernel(float* qkv32, float* bg, const void* x, const void* b,
                                                        const void* a, int64_t xstride, bool f32, const float* conv_w,
                                                        const float* conv_wt, float* conv_state, const float* A_log,
@@ -328,65 +397,17 @@ __global__ void __launch_bounds__(NT) delta_prep_kernel(float* qkv32, float* bg,
   // bf16 steps with the weights also given tap-major ([taps, C]): 8 channels per thread and trip, 16-byte loads of
   // inputs, weights and state (a decode row is then two dependent trips per thread instead of C / 256)
   const bool wide = conv_wt != nullptr && !f32 && C % 8 == 0 && xstride % 8 == 0 && aligned16(x);
+  const bf16_t* xb = reinterpret_cast<const bf16_t*>(x);
   for (int c8 = threadIdx.x; wide && c8 < C / 8; c8 += NT) {
-    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    for (int j = 0; j < taps; ++j) {
-      const int back = taps - 1 - j;
-      if (p - back < 0) continue;
-      const int src = i - back;
-      float xv[8];
-      if (src >= 0) {
-        unpack8(*reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(x) + (int64_t)(row - back) * xstride + 8 * c8), xv);
-      } else {
-        const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(taps - 1 + src) * C + 8 * c8);
-        const float4 s0 = sp[0], s1 = sp[1];
-        xv[0] = s0.x, xv[1] = s0.y, xv[2] = s0.z, xv[3] = s0.w, xv[4] = s1.x, xv[5] = s1.y, xv[6] = s1.z, xv[7] = s1.w;
-      }
-
-      const float4* wp = reinterpret_cast<const float4*>(conv_wt + (int64_t)j * C + 8 * c8);
-      const float4 w0 = wp[0], w1 = wp[1];
-      acc[0] += w0.x * xv[0], acc[1] += w0.y * xv[1], acc[2] += w0.z * xv[2], acc[3] += w0.w * xv[3];
-      acc[4] += w1.x * xv[4], acc[5] += w1.y * xv[5], acc[6] += w1.z * xv[6], acc[7] += w1.w * xv[7];
-    }
+    float acc[8];
+    conv8(acc, xb, row, xstride, c8, st, conv_wt, taps, C, i, p);
 #pragma unroll
     for (int e = 0; e < 8; ++e) vals[8 * c8 + e] = rnd(siluf(rnd(acc[e], false)), false);
-    if (r.cu_q == nullptr) {
-      // one row per sequence: this thread is the only reader of its channels' tail, so it shifts it here: state
-      // row k takes row k + 1 (zeros where that lies before the sequence's start), the last one the row's input
-      const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
-      for (int k = 0; k + 1 < taps - 1; ++k) {
-        const bool live = p - (taps - 2 - k) >= 0;
-        float4* dp = reinterpret_cast<float4*>(st + (int64_t)k * C + 8 * c8);
-        const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(k + 1) * C + 8 * c8);
-        const float4 t0 = sp[0], t1 = sp[1];
-        dp[0] = live ? t0 : zero;
-        dp[1] = live ? t1 : zero;
-      }
-      if (taps > 1) {
-        float xv[8];
-        unpack8(*reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(x) + (int64_t)row * xstride + 8 * c8), xv);
-        float4* dp = reinterpret_cast<float4*>(st + (int64_t)(taps - 2) * C + 8 * c8);
-        dp[0] = make_float4(xv[0], xv[1], xv[2], xv[3]);
-        dp[1] = make_float4(xv[4], xv[5], xv[6], xv[7]);
-      }
-    }
+    if (r.cu_q == nullptr) conv8_shift(xb, row, xstride, c8, st, taps, C, p);
   }
   for (int c = threadIdx.x; !wide && c < C; c += NT) {
-    float acc = 0.f;
-    for (int j = 0; j < taps; ++j) {
-      const int back = taps - 1 - j;
-      if (p - back < 0) continue;
-      const int src = i - back;
-      const float xv = src >= 0 ? ldv(x, (int64_t)(row - back) * xstride + c, f32) : st[(int64_t)(taps - 1 + src) * C + c];
-      acc += conv_w[(int64_t)c * taps + j] * xv;
-    }
-    vals[c] = rnd(siluf(rnd(acc, f32)), f32);
-    if (r.cu_q == nullptr) {
-      // one row per sequence: this thread is the only reader of its channel's tail, so it shifts it here
-      for (int k = 0; k + 1 < taps - 1; ++k)
-        st[(int64_t)k * C + c] = p - (taps - 2 - k) >= 0 ? st[(int64_t)(k + 1) * C + c] : 0.f;
-      if (taps > 1) st[(int64_t)(taps - 2) * C + c] = ldv(x, (int64_t)row * xstride + c, f32);
-    }
+    vals[c] = rnd(siluf(rnd(conv1(x, f32, row, xstride, c, st, conv_w, taps, 1, taps, C, i, p), f32)), f32);
+    if (r.cu_q == nullptr) conv1_shift(x, f32, row, xstride, c, st, taps, C, p);
   }
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -408,6 +429,11 @@ __global__ void __launch_bounds__(NT) delta_prep_kernel(float* qkv32, float* bg,
     for (int c = threadIdx.x; c < C; c += NT) qkv32[(int64_t)row * C + c] = vals[c];
   }
   const int H = sh.heads;
+  if (a == nullptr) {   // the decay is the recurrence kernel's (per key channel)
+    for (int h = threadIdx.x; h < H; h += NT)
+      bg[(int64_t)row * H + h] = 1.0f / (1.0f + expf(-ldv(b, (int64_t)row * xstride + h, f32)));
+    return;
+  }
   for (int h = threadIdx.x; h < H; h += NT) {
     const float bv = ldv(b, (int64_t)row * xstride + h, f32);
     const float av = ldv(a, (int64_t)row * xstride + h, f32) + dt_bias[h];
@@ -452,12 +478,10 @@ constexpr int TB = 16;  // tokens staged per trip
 // split over the 4 lanes of a quad, lane `part` holding rows [part * DP, (part + 1) * DP) — so a token costs each
 // lane 3 * DP multiply-adds and two quad reductions (S^T k and S^T q), with q and k read from LDS as float4
 // broadcasts, and 4 * vdim lanes work on one head. Tokens are staged TB at a time; the read-outs of a trip are
-// normed and gated afterwards, one wave per token.
-template <int DP>
-__global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const float* qkv32, const float* bg,
-                                                          const void* gate, int64_t gstride, bool f32,
-                                                          const float* norm_w, float eps, float* state, DeltaShape sh,
-                                                          RaggedRows r) {
+// normed and gated afterwards, one wave per token. CD: a decay per key channel, computed while a trip is staged.
+template <int DP, bool CD>
+__global__ void __launch_bounds__(1024) gated_delta_kernel(GatedDeltaArgs a, RaggedRows r) {
+  const DeltaShape& sh = a.sh;
   extern __shared__ __attribute__((aligned(16))) float sm[];
   constexpr int DPAD = 4 * DP;
   const int d = sh.dim, dv = sh.vdim, H = sh.heads, G = sh.kv_heads, C = sh.channels();
@@ -466,7 +490,8 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const floa
   float* vs = ks + TB * DPAD;      // [TB][dv]
   float* os = vs + TB * dv;        // [TB][dv]
   float* bs = os + TB * dv;        // [TB] beta
-  float* gs = bs + TB;             // [TB] decay
+  float* gs = bs + TB;             // [TB] decay, or [TB][DPAD] with CD
+  const int bgw = CD ? H : 2 * H;
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x;
   const int j = tid >> 2, part = tid & 3;
   const int kh = h / (H / G);
@@ -474,7 +499,8 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const floa
   const int L = r.cu_q ? r.cu_q[s + 1] - q0 : 1;
   if (L <= 0) return;
   const bool fresh = r.positions[q0] <= 0;
-  float* st = state + ((int64_t)r.state_slots[s] * H + h) * d * dv;
+  float* st = a.state + ((int64_t)r.state_slots[s] * H + h) * d * dv;
+  const float expA = CD ? expf(a.A_log[h]) : 0.f;
   float S[DP];
 #pragma unroll
   for (int i = 0; i < DP; ++i) {
@@ -487,21 +513,30 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const floa
     __syncthreads();
     for (int e = tid; e < nb * DPAD; e += nthr) {
       const int tt = e / DPAD, c = e % DPAD;
-      const float* row = qkv32 + (int64_t)(q0 + t0 + tt) * C;
+      const float* row = a.qkv32 + (int64_t)(q0 + t0 + tt) * C;
       qs[e] = c < d ? row[kh * d + c] : 0.f;
       ks[e] = c < d ? row[G * d + kh * d + c] : 0.f;
+      if (CD) {
+        float g = 0.f;
+        if (c < d) {
+          const float z = ldv(a.z, (int64_t)(q0 + t0 + tt) * a.zstride + h * d + c, a.f32) + a.z_bias[h * d + c];
+          g = expf(-expA * softplusf(z));
+        }
+        gs[e] = g;
+      }
     }
     for (int e = tid; e < nb * dv; e += nthr) {
       const int tt = e / dv, c = e % dv;
-      vs[e] = qkv32[(int64_t)(q0 + t0 + tt) * C + 2 * G * d + h * dv + c];
+      vs[e] = a.qkv32[(int64_t)(q0 + t0 + tt) * C + 2 * G * d + h * dv + c];
     }
     if (tid < nb) {
-      bs[tid] = bg[(int64_t)(q0 + t0 + tid) * 2 * H + h];
-      gs[tid] = bg[(int64_t)(q0 + t0 + tid) * 2 * H + H + h];
+      bs[tid] = a.bg[(int64_t)(q0 + t0 + tid) * bgw + h];
+      if (!CD) gs[tid] = a.bg[(int64_t)(q0 + t0 + tid) * bgw + H + h];
     }
     __syncthreads();
     for (int tt = 0; tt < nb; ++tt) {
-      const float g = gs[tt], beta = bs[tt];
+      const float g = CD ? 1.0f : gs[tt], beta = bs[tt];
+      const float4* gt4 = reinterpret_cast<const float4*>(gs + tt * DPAD + part * DP);
       const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD + part * DP);
       const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD + part * DP);
       float kreg[DP];
@@ -513,10 +548,11 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const floa
         kreg[4 * i + 1] = k4.y;
         kreg[4 * i + 2] = k4.z;
         kreg[4 * i + 3] = k4.w;
-        S[4 * i] *= g;
-        S[4 * i + 1] *= g;
-        S[4 * i + 2] *= g;
-        S[4 * i + 3] *= g;
+        const float4 g4 = CD ? gt4[i] : make_float4(g, g, g, g);
+        S[4 * i] *= g4.x;
+        S[4 * i + 1] *= g4.y;
+        S[4 * i + 2] *= g4.z;
+        S[4 * i + 3] *= g4.w;
         d0 += S[4 * i] * k4.x + S[4 * i + 2] * k4.z;
         d1 += S[4 * i + 1] * k4.y + S[4 * i + 3] * k4.w;
       }
@@ -545,11 +581,12 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(void* out, const floa
       float ss = 0.f;
       for (int c = lane; c < dv; c += 64) ss += os[tt * dv + c] * os[tt * dv + c];
       ss = wave_sum(ss);
-      const float rs = 1.0f / sqrtf(ss / (float)dv + eps);
+      const float rs = a.mult / sqrtf(ss / (float)dv + a.eps);
       const int64_t row = q0 + t0 + tt;
       for (int c = lane; c < dv; c += 64) {
-        const float gt = ldv(gate, row * gstride + h * dv + c, f32);
-        stv(out, (row * H + h) * dv + c, f32, os[tt * dv + c] * rs * norm_w[c] * siluf(gt));
+        const float gt = ldv(a.gate, row * a.gstride + h * dv + c, a.f32);
+        stv(a.out, row * a.ostride + h * dv + c, a.f32,
+            os[tt * dv + c] * rs * a.norm_w[c] * (a.gate_sigmoid ? sigmoidf(gt) : siluf(gt)));
       }
     }
   }
@@ -571,8 +608,33 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
   float* qv = sm;
   float* kv = qv + nq;
   float* vv = kv + nk;
+  // cosine / sine of the row's rotation angles, shared by the heads: keys and queries, then values
+  const int half = a.rot_dims / 2, vhalf = a.v_inv_freq != nullptr ? dv / 2 : 0;
+  float* ct = vv + nv;
+  float* snt = ct + half + vhalf;
   const int64_t t = blockIdx.x;
   const bool f32 = a.f32;
+  {
+    const float p = (float)a.positions[t];
+    for (int e = threadIdx.x; e < half + vhalf; e += NT) {
+      const bool kq = e < half;
+      float sn, cs;
+      sincosf(p * (kq ? a.inv_freq[e] : a.v_inv_freq[e - half]), &sn, &cs);
+      const float gain = kq ? a.rot_gain : 1.0f;
+      ct[e] = cs * gain;
+      snt[e] = sn * gain;
+    }
+  }
+  // short convolution over the sequence of the channels q | k | v (adjacent columns)
+  const int C = nq + nk + nv;
+  const int taps = a.conv_wt != nullptr ? a.taps : 0;
+  int ci = 0;
+  float* cst = nullptr;
+  if (taps > 0) {
+    const int sq_ = seq_of_row(a.r.cu_q, a.r.num_seqs, (int)t);
+    ci = (int)t - (a.r.cu_q ? a.r.cu_q[sq_] : sq_);
+    cst = a.conv_state + (int64_t)a.r.state_slots[sq_] * (taps - 1) * C;
+  }
   float sq = 0.f, sk = 0.f;
   float lam = 0.f;
   if (a.v_lambda != nullptr) lam = a.v_lambda[0];
@@ -588,7 +650,24 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
     for (int c8 = threadIdx.x; c8 < (v_is_k ? nq + nk : nq + nk + nv) / 8; c8 += NT) {
       const int c = 8 * c8;
       float f[8];
-      if (c < nq) {
+      if (taps > 0 || a.bias != nullptr) {   // q, k and v are adjacent columns here
+        if (taps > 0) {
+          conv8(f, reinterpret_cast<const bf16_t*>(a.q), t, a.xstride, c8, cst, a.conv_wt, taps, C, ci, a.positions[t]);
+          if (a.r.cu_q == nullptr)
+            conv8_shift(reinterpret_cast<const bf16_t*>(a.q), t, a.xstride, c8, cst, taps, C, a.positions[t]);
+        } else {
+          unpack8(*reinterpret_cast<const uint4*>(qp + c), f);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) f[e] += a.bias[c + e];
+        }
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
+        if (c < nq)
+          sq += ss;
+        else if (c < nq + nk)
+          sk += ss;
+      } else if (c < nq) {
         unpack8(*reinterpret_cast<const uint4*>(qp + c), f);
 #pragma unroll
         for (int e = 0; e < 8; ++e) sq += f[e] * f[e];
@@ -609,17 +688,32 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
       for (int e = 0; e < 8; ++e) qv[c + e] = f[e];   // qv, kv and vv are adjacent
     }
   } else {
-    for (int c = threadIdx.x; c < nq; c += NT) {
+    const bool pre = taps > 0 || a.bias != nullptr;
+    for (int c = threadIdx.x; pre && c < C; c += NT) {   // q, k and v are adjacent columns here
+      float x;
+      if (taps > 0) {
+        x = conv1(a.q, f32, t, a.xstride, c, cst, a.conv_wt, 1, C, taps, C, ci, a.positions[t]);
+        if (a.r.cu_q == nullptr) conv1_shift(a.q, f32, t, a.xstride, c, cst, taps, C, a.positions[t]);
+      } else {
+        x = ldv(a.q, t * a.xstride + c, f32) + a.bias[c];
+      }
+      qv[c] = x;
+      if (c < nq)
+        sq += x * x;
+      else if (c < nq + nk)
+        sk += x * x;
+    }
+    for (int c = threadIdx.x; !pre && c < nq; c += NT) {
       const float x = ldv(a.q, t * a.xstride + c, f32);
       qv[c] = x;
       sq += x * x;
     }
-    for (int c = threadIdx.x; c < nk; c += NT) {
+    for (int c = threadIdx.x; !pre && c < nk; c += NT) {
       const float x = ldv(a.k, t * a.xstride + c, f32);
       kv[c] = x;
       sk += x * x;
     }
-    for (int c = threadIdx.x; c < (v_is_k ? 0 : nv); c += NT) {
+    for (int c = threadIdx.x; !pre && c < (v_is_k ? 0 : nv); c += NT) {
       float x = ldv(a.v, t * a.xstride + c, f32);
       if (a.v_lambda != nullptr) x = (1.0f - lam) * x + lam * ldv(a.v_first, t * a.vfstride + c, f32);
       vv[c] = x;
@@ -627,13 +721,10 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
   }
   const bool per_head = a.q_norm != nullptr && a.head_norm;
   auto rotate = [&]() {
-    const int half = a.rot_dims / 2;
-    const float p = (float)a.positions[t];
     for (int e = threadIdx.x; e < (H + G) * half; e += NT) {
       const int hd = e / half, i = e % half;
       float* base = hd < H ? qv + hd * d : kv + (hd - H) * d;
-      float sn, cs;
-      sincosf(p * a.inv_freq[i], &sn, &cs);
+      const float cs = ct[i], sn = snt[i];
       const float u = base[i], v = base[i + half];
       base[i] = u * cs - v * sn;
       base[i + half] = v * cs + u * sn;
@@ -687,6 +778,14 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
     __syncthreads();
   }
   if (a.rot_dims > 0 && !rot_first) rotate();
+  for (int e = threadIdx.x; e < G * vhalf; e += NT) {   // rotated values
+    const int g = e / vhalf, i = e % vhalf;
+    float* base = vv + g * dv;
+    const float cs = ct[half + i], sn = snt[half + i];
+    const float u = base[i], v = base[i + vhalf];
+    base[i] = u * cs - v * sn;
+    base[i + vhalf] = v * cs + u * sn;
+  }
   if (a.v_unit) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     for (int g = wave; g < G; g += NT / 64) {
@@ -791,32 +890,31 @@ hipError_t launch_conv_state_update(float* conv_state, const void* x, int64_t xs
   return hipGetLastError();
 }
 
-template <int DP>
-static hipError_t launch_gd(void* out, const float* qkv32, const float* bg, const void* gate, int64_t gstride, bool f32,
-                            const float* norm_w, float eps, float* state, DeltaShape sh, RaggedRows r, hipStream_t s) {
-  const int nthr = (4 * sh.vdim + 63) / 64 * 64;
-  const size_t lds = sizeof(float) * (TB * (2 * 4 * DP + 2 * sh.vdim) + 2 * TB);
+template <int DP, bool CD> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+  const int nthr = (4 * a.sh.vdim + 63) / 64 * 64;
+  const size_t lds = sizeof(float) * (TB * ((CD ? 3 : 2) * 4 * DP + 2 * a.sh.vdim) + 2 * TB);
   if (lds > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gated_delta_kernel<DP>),
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gated_delta_kernel<DP, CD>),
                                        hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
   }
-  hipLaunchKernelGGL(gated_delta_kernel<DP>, dim3(sh.heads, r.num_seqs), dim3(nthr), lds, s, out, qkv32, bg, gate,
-                     gstride, f32, norm_w, eps, state, sh, r);
+  hipLaunchKernelGGL((gated_delta_kernel<DP, CD>), dim3(a.sh.heads, r.num_seqs), dim3(nthr), lds, s, a, r);
   return hipGetLastError();
 }
+template <int DP> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+  return a.z != nullptr ? launch_gd<DP, true>(a, r, s) : launch_gd<DP, false>(a, r, s);
+}
 
-hipError_t launch_gated_delta(void* out, const float* qkv32, const float* bg, const void* gate, int64_t gstride,
-                              bool f32, const float* norm_w, float eps, float* state, DeltaShape sh, RaggedRows r,
-                              hipStream_t s) {
+hipError_t launch_gated_delta(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
   if (r.num_seqs == 0 || r.total_rows == 0) return hipSuccess;
-  if (!delta_ok(sh) || !rows_ok(r)) return hipErrorInvalidValue;
+  if (!delta_ok(a.sh) || !rows_ok(r) || (a.z != nullptr && (a.z_bias == nullptr || a.A_log == nullptr)))
+    return hipErrorInvalidValue;
   // rows of the state per lane of a quad: dim / 4, rounded up to a multiple of 4
-  if (sh.dim <= 16) return launch_gd<4>(out, qkv32, bg, gate, gstride, f32, norm_w, eps, state, sh, r, s);
-  if (sh.dim <= 32) return launch_gd<8>(out, qkv32, bg, gate, gstride, f32, norm_w, eps, state, sh, r, s);
-  if (sh.dim <= 64) return launch_gd<16>(out, qkv32, bg, gate, gstride, f32, norm_w, eps, state, sh, r, s);
-  if (sh.dim <= 128) return launch_gd<32>(out, qkv32, bg, gate, gstride, f32, norm_w, eps, state, sh, r, s);
-  return launch_gd<64>(out, qkv32, bg, gate, gstride, f32, norm_w, eps, state, sh, r, s);
+  if (a.sh.dim <= 16) return launch_gd<4>(a, r, s);
+  if (a.sh.dim <= 32) return launch_gd<8>(a, r, s);
+  if (a.sh.dim <= 64) return launch_gd<16>(a, r, s);
+  if (a.sh.dim <= 128) return launch_gd<32>(a, r, s);
+  return launch_gd<64>(a, r, s);
 }
 
 hipError_t launch_qkv_prep(const QkvPrepArgs& a, hipStream_t s) {
@@ -827,7 +925,13 @@ hipError_t launch_qkv_prep(const QkvPrepArgs& a, hipStream_t s) {
       (a.v == nullptr && (a.vdim != a.dim || a.v_lambda != nullptr)) || (a.head_norm && a.q_norm == nullptr) ||
       (a.q_temp_coef != 0.f && a.q_temp_every < 1))
     return hipErrorInvalidValue;
-  const size_t lds = sizeof(float) * ((size_t)a.heads * a.dim + (size_t)a.kv_heads * (a.dim + a.vdim));
+  if (a.v_inv_freq != nullptr && ((a.vdim & 1) || a.v_unit || a.v == nullptr)) return hipErrorInvalidValue;
+  if (a.conv_wt != nullptr && (a.bias != nullptr || a.v == nullptr || a.v_lambda != nullptr || a.taps < 1 ||
+                               a.taps > TAPS_MAX || !rows_ok(a.r) || (a.taps > 1 && a.conv_state == nullptr)))
+    return hipErrorInvalidValue;
+  if (a.bias != nullptr && (a.v == nullptr || a.v_lambda != nullptr)) return hipErrorInvalidValue;
+  const size_t lds = sizeof(float) * ((size_t)a.heads * a.dim + (size_t)a.kv_heads * (a.dim + a.vdim) + a.rot_dims +
+                                      (a.v_inv_freq != nullptr ? a.vdim : 0));
   if (lds > 150 * 1024) return hipErrorInvalidValue;
   if (lds > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(qkv_prep_kernel),

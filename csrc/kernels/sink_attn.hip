@@ -1,7 +1,8 @@
 // Grouped-query softmax attention over a paged cache, for prompt portions and single decode tokens alike. A cache
 // block holds block_size tokens head-major: [G][block_size][K: dim | V: vdim], so the keys and values that one
 // key/value head reads from a block are one contiguous piece of memory. A query at position p of its sequence sees the cached positions j <= p
-// with p - j < window (window 0: all of them); its score is (q . k_j) * scale + bias[min(p - j, bias_rows - 1), h]
+// with p - j < window (window 0: all of them) and, with seg > 0, floor(j / seg) = floor(p / seg) (positions attend
+// within fixed segments counted from position 0); its score is (q . k_j) * scale + bias[min(p - j, bias_rows - 1), h]
 // (bias optional); the softmax denominator holds one more per-head term exp(sink_h) that belongs to no position
 // (the running maximum starts at the sink, the running sum at 1). Query and value widths may differ.
 //
@@ -39,6 +40,13 @@ __device__ __forceinline__ float fast_tanh(float x) {
   return 1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f);
 }
 
+// the first key a query at position p sees
+__device__ __forceinline__ int first_key(const SinkAttnArgs& a, int p) {
+  int lo = a.window > 0 ? max(0, p - a.window + 1) : 0;
+  if (a.seg > 0) lo = max(lo, p - p % a.seg);
+  return lo;
+}
+
 template <int BK, int CC, int RPW, bool F32>
 __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, int KS, int VS) {
   constexpr int RW = RPW * WAVES;
@@ -57,7 +65,7 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
   const int ctx = a.ctx_lens[s];
   const int last_row = min(row0 + RW, nrows) - 1;
   const int p_first = (int)a.positions[q0 + row0 / QPG], p_last = (int)a.positions[q0 + last_row / QPG];
-  const int jlo = a.window > 0 ? max(0, p_first - a.window + 1) : 0;
+  const int jlo = first_key(a, p_first);
   const int jhi = min(p_last, ctx - 1);
 
   for (int r = wave; r < RW; r += WAVES) {
@@ -68,7 +76,7 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
     for (int d = lane; d < QS; d += 64) qs[r * QS + d] = (ok && d < D) ? ldt<F32>(a.q, (t * H + h) * D + d) : 0.f;
   }
 
-  int prow[RPW], hrow[RPW];
+  int prow[RPW], hrow[RPW], jrow[RPW];
   bool rok[RPW];
   float m[RPW], l[RPW], o[RPW][CC];
 #pragma unroll
@@ -76,6 +84,7 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
     const int row = row0 + wave * RPW + i;
     rok[i] = row < nrows;
     prow[i] = rok[i] ? (int)a.positions[q0 + row / QPG] : -1;
+    jrow[i] = first_key(a, max(prow[i], 0));
     hrow[i] = g * QPG + (rok[i] ? row % QPG : 0);
     const bool has_sink = a.sink != nullptr && rok[i];
     m[i] = has_sink ? a.sink[hrow[i]] : -1e30f;
@@ -116,7 +125,7 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
 #pragma unroll
       for (int off = BK; off < 64; off <<= 1) sc += __shfl_xor(sc, off, 64);
       const int n = prow[i] - j;
-      const bool valid = rok[i] && j <= jhi && n >= 0 && (a.window <= 0 || n < a.window);
+      const bool valid = rok[i] && j <= jhi && n >= 0 && j >= jrow[i];
       sc *= a.scale;
       if (a.softcap > 0.f) sc = a.softcap * tanhf(sc / a.softcap);
       if (valid && a.slopes != nullptr) sc -= a.slopes[hrow[i]] * (float)n;
@@ -198,7 +207,7 @@ template <bool F32> hipError_t launch_fma(const SinkAttnArgs& a, hipStream_t s) 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 128, vdim % 32 == 0, vdim <= 128.
+// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 256, vdim % 32 == 0, vdim <= 256.
 // Workgroup = NW waves x 32 rows of one (sequence, key/value head); NW = 1 for steps of few rows (decode). Per tile
 // of 32 keys, staged once in LDS as rows [K_g | V_g] (the next tile's global loads in flight meanwhile):
 //   S^T[key][q] = K Q^T        A = K rows from LDS, B = Q rows from LDS      (dim / 16 MFMAs)
@@ -247,7 +256,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
   const int ctx = a.ctx_lens[s];
   const int last_row = min(row0 + ROWS, nrows) - 1;
   const int p_first = (int)a.positions[q0 + row0 / QPG], p_last = (int)a.positions[q0 + last_row / QPG];
-  int jlo = a.window > 0 ? max(0, p_first - a.window + 1) : 0;
+  int jlo = first_key(a, p_first);
   int jhi = min(p_last, ctx - 1);
   if (nsplit > 1) {
     jlo += z * chunk;
@@ -282,6 +291,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
 
   const bool wave_live = row0 + wave * 32 < nrows;
   const int prow = rok ? (int)a.positions[q0 + myrow / QPG] : -1;
+  const int jrow = first_key(a, max(prow, 0));
   constexpr float LOG2E = 1.4426950408889634f;
   const float sl2 = a.scale * LOG2E;
   const bool shaped = a.softcap > 0.f || a.slopes != nullptr;
@@ -341,8 +351,9 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
   // a tile is interior for a wave when every one of its 32 x 32 (key, row) pairs is visible: no masking then
   const int wrow_first = row0 + wave * 32, wrow_last = wrow_first + 31;
   const bool wave_full = wrow_last < nrows;
-  const int pw_first = wave_full ? (int)a.positions[q0 + wrow_first / QPG] : 0;
-  const int pw_last = wave_full ? (int)a.positions[q0 + wrow_last / QPG] : 0;
+  const int pw_first = wave_live ? (int)a.positions[q0 + wrow_first / QPG] : 0;
+  const int pw_last = wave_live ? (int)a.positions[q0 + min(wrow_last, nrows - 1) / QPG] : 0;
+  const int jw_first = first_key(a, pw_first), jw_last = first_key(a, pw_last);
   for (int j0 = jlo; j0 <= jhi; j0 += MKT) {
     __syncthreads();  // every wave is done with the previous tile (first: the queries are being written)
     {
@@ -360,7 +371,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
     }
     __syncthreads();
     if (j0 + MKT <= jhi) fetch(j0 + MKT, bt_lds);  // in flight while this tile is computed
-    if (!wave_live) continue;
+    if (!wave_live || j0 > pw_last || j0 + MKT <= jw_first) continue;   // nothing of this tile is visible to the wave
     f32x16_t sc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) sc[r] = 0.f;
@@ -372,8 +383,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
       sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(af, bfr, sc, 0, 0, 0);
     }
     float mx = -INFINITY;
-    const bool interior = wave_full && j0 + MKT - 1 <= min(pw_first, jhi) &&
-                          (a.window <= 0 || pw_last - j0 < a.window);
+    const bool interior = wave_full && j0 + MKT - 1 <= min(pw_first, jhi) && j0 >= jw_last;
     if (shaped) {
       // capped scores and / or a linear distance penalty: cap * tanh(s * scale / cap) - slope * n, in log2 units.
       // tanh = 1 - 2 / (2^(2 x log2 e) + 1), so the capped score is one multiply-add of the reciprocal; the
@@ -397,7 +407,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
         for (int r = 0; r < 16; ++r) {
           const int j = j0 + (r & 3) + 8 * (r >> 2) + 4 * hh;
           const int n = prow - j;
-          const bool valid = interior || (rok && j <= jhi && n >= 0 && (a.window <= 0 || n < a.window));
+          const bool valid = interior || (rok && j <= jhi && n >= 0 && j >= jrow);
           float v = a.softcap > 0.f ? capl2 * fast_tanh(sc[r] * s_over_cap) : sc[r] * sl2;
           v -= slope2 * (float)n;
           if (bias != nullptr && valid) v += bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
@@ -429,7 +439,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
       for (int r = 0; r < 16; ++r) {
         const int j = j0 + (r & 3) + 8 * (r >> 2) + 4 * hh;
         const int n = prow - j;
-        const bool valid = rok && j <= jhi && n >= 0 && (a.window <= 0 || n < a.window);
+        const bool valid = rok && j <= jhi && n >= 0 && j >= jrow;
         float v = sc[r] * sl2;
         if (bias != nullptr && valid) v += bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
         v = valid ? v : -INFINITY;
@@ -507,32 +517,32 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
 
 
 // ---------------------------------------------------------------------------------------------------
-// Decode steps (one query token per sequence) in bf16, dim % 8 == 0 <= 128, vdim % 8 == 0 <= 128, at most 8 query
+// Decode steps (one query token per sequence) in bf16, dim % 8 == 0 <= 256, vdim % 8 == 0 <= 256, at most 8 query
 // heads per key/value head: no matrix cores and no staging of keys in LDS. A workgroup of 256 threads owns one
 // (sequence, key/value head, split of the keys) and walks its keys 128 at a time:
 //   scores   LK lanes share a key (16 bytes of it each, the query's matching 8 dims in registers), 256 / LK keys
 //            per pass, all passes' loads issued before the first is used; a shuffle reduction per row
 //   softmax  one wave per query row over the 128 scores in LDS (log2 units, running max and sum across trips,
 //            the sink seeds split 0)
-//   values   16 lanes share a value row, 16 keys per pass, loads issued before the softmax; each thread keeps
-//            R x 8 output columns and the 16 key groups are summed through LDS at the end
+//   values   VL lanes share a value row, 256 / VL keys per pass, loads issued before the softmax; each thread keeps
+//            R x 8 output columns and the 256 / VL key groups are summed through LDS at the end
 // Splits write unnormalised sums + (max, sum) to the workspace and sink_attn_merge_kernel combines them.
 constexpr int DCH = 128;   // keys per trip
 
-template <int R, int LK>
+template <int R, int LK, int VL>
 __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, float* ws_o, float* ws_ml, int nsplit,
                                                               int chunk) {
-  constexpr int NG = 256 / LK, NPK = DCH / NG, NPV = DCH / 16;
+  constexpr int NG = 256 / LK, NPK = DCH / NG, NV = 256 / VL, NPV = DCH / NV;
   extern __shared__ __attribute__((aligned(16))) float dsm[];
   float* sc = dsm;                       // [R][DCH] scores, then weights
   float* ml = sc + R * DCH;              // [R][3]: running max, running sum, this trip's rescale
-  float* red = ml + R * 4;               // [16][R][DV]
+  float* red = ml + R * 4;               // [NV][R][DV]
   __shared__ int btl[DCH / 1 + 2];       // block-table entries of the trip (at most one per key)
   const int z = blockIdx.x, s = blockIdx.y, g = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int H = a.heads, G = a.kv_heads, QPG = H / G, D = a.dim, DV = a.vdim, roww = D + DV;
   const int p = (int)a.positions[s];
   const int ctx = a.ctx_lens[s];
-  int jlo = a.window > 0 ? max(0, p - a.window + 1) : 0;
+  int jlo = first_key(a, p);
   int jhi = min(p, ctx - 1);
   if (nsplit > 1) {
     jlo += z * chunk;
@@ -552,7 +562,7 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
   const bf16_t* qg = reinterpret_cast<const bf16_t*>(a.q);
   const int* bt = a.block_tables + (int64_t)s * a.bt_stride;
   const int kl = tid % LK, kg = tid / LK;      // score phase: my 8 dims of the key, my key group
-  const int vl = tid & 15, vg = tid >> 4;      // value phase: my 8 columns, my key group
+  const int vl = tid % VL, vg = tid / VL;      // value phase: my 8 columns, my key group
   float qf[R][8];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
@@ -593,7 +603,7 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
     }
 #pragma unroll
     for (int u = 0; u < NPV; ++u) {
-      const int j = j0 + u * 16 + vg;
+      const int j = j0 + u * NV + vg;
       vq[u] = make_uint4(0, 0, 0, 0);
       if (j <= jhi && 8 * vl < DV) {
         const int jb = j / a.block_size;
@@ -650,7 +660,7 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
     for (int u = 0; u < NPV; ++u) {
       float f[8];
       unpack8(vq[u], f);
-      const int jj = u * 16 + vg;
+      const int jj = u * NV + vg;
 #pragma unroll
       for (int r = 0; r < R; ++r) {
         const float pw = sc[r * DCH + jj];
@@ -659,7 +669,7 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
       }
     }
   }
-  // sum the 16 key groups
+  // sum the NV key groups
   if (8 * vl < DV) {
 #pragma unroll
     for (int r = 0; r < R; ++r) {
@@ -673,7 +683,7 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
     const int r = idx / DV, c = idx % DV;
     float o = 0.f;
 #pragma unroll
-    for (int k = 0; k < 16; ++k) o += red[((int64_t)k * R + r) * DV + c];
+    for (int k = 0; k < NV; ++k) o += red[((int64_t)k * R + r) * DV + c];
     const int64_t orow = (int64_t)s * H + g * QPG + r;
     if (nsplit > 1) {
       ws_o[((int64_t)z * wrows + orow) * DV + c] = o;
@@ -756,16 +766,25 @@ template <int NW, int NKC> hipError_t launch_mfma_ndb(const SinkAttnArgs& a, hip
     case 3: return launch_mfma<3, NW, NKC>(a, s);
     case 4: return launch_mfma<4, NW, NKC>(a, s);
   }
+  if constexpr (NKC >= 16) {
+    switch (a.vdim / 32) {
+      case 5: return launch_mfma<5, NW, NKC>(a, s);
+      case 6: return launch_mfma<6, NW, NKC>(a, s);
+      case 7: return launch_mfma<7, NW, NKC>(a, s);
+      case 8: return launch_mfma<8, NW, NKC>(a, s);
+    }
+  }
   return hipErrorInvalidValue;
 }
 
 template <int NW> hipError_t launch_mfma_nw(const SinkAttnArgs& a, hipStream_t s) {
-  return a.dim <= 64 ? launch_mfma_ndb<NW, 8>(a, s) : launch_mfma_ndb<NW, 16>(a, s);
+  if (a.dim <= 64 && a.vdim <= 128) return launch_mfma_ndb<NW, 8>(a, s);
+  return a.dim <= 128 ? launch_mfma_ndb<NW, 16>(a, s) : launch_mfma_ndb<NW, 32>(a, s);
 }
 
-template <int R, int LK> hipError_t launch_decode_one(const SinkAttnArgs& a, hipStream_t s) {
-  auto* fn = sink_attn_decode_kernel<R, LK>;
-  const size_t lds = sizeof(float) * ((size_t)R * DCH + (size_t)R * 4 + (size_t)16 * R * a.vdim);
+template <int R, int LK, int VL> hipError_t launch_decode_one(const SinkAttnArgs& a, hipStream_t s) {
+  auto* fn = sink_attn_decode_kernel<R, LK, VL>;
+  const size_t lds = sizeof(float) * ((size_t)R * DCH + (size_t)R * 4 + (size_t)(256 / VL) * R * a.vdim);
   if (lds > 48 * 1024) {
     static size_t raised = 0;
     if (lds > raised) {
@@ -784,22 +803,26 @@ template <int R, int LK> hipError_t launch_decode_one(const SinkAttnArgs& a, hip
   return hipGetLastError();
 }
 
-template <int LK> hipError_t launch_decode_r(const SinkAttnArgs& a, hipStream_t s) {
+template <int LK, int VL> hipError_t launch_decode_r(const SinkAttnArgs& a, hipStream_t s) {
   const int qpg = a.heads / a.kv_heads;
-  if (qpg <= 1) return launch_decode_one<1, LK>(a, s);
-  if (qpg <= 2) return launch_decode_one<2, LK>(a, s);
-  if (qpg <= 4) return launch_decode_one<4, LK>(a, s);
-  return launch_decode_one<8, LK>(a, s);
+  if (qpg <= 1) return launch_decode_one<1, LK, VL>(a, s);
+  if (qpg <= 2) return launch_decode_one<2, LK, VL>(a, s);
+  if (qpg <= 4) return launch_decode_one<4, LK, VL>(a, s);
+  return launch_decode_one<8, LK, VL>(a, s);
+}
+
+template <int LK> hipError_t launch_decode_v(const SinkAttnArgs& a, hipStream_t s) {
+  return a.vdim <= 128 ? launch_decode_r<LK, 16>(a, s) : launch_decode_r<LK, 32>(a, s);
 }
 
 inline bool decode_ok(const SinkAttnArgs& a) {
-  return !a.f32 && a.cu_q == nullptr && a.max_q == 1 && a.heads / a.kv_heads <= 8 && a.dim % 8 == 0 && a.dim <= 128 &&
-         a.vdim % 8 == 0 && a.vdim <= 128 && (reinterpret_cast<uintptr_t>(a.q) & 15) == 0 &&
+  return !a.f32 && a.cu_q == nullptr && a.max_q == 1 && a.heads / a.kv_heads <= 8 && a.dim % 8 == 0 && a.dim <= 256 &&
+         a.vdim % 8 == 0 && a.vdim <= 256 && (reinterpret_cast<uintptr_t>(a.q) & 15) == 0 &&
          (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0 && (a.nsplit <= 1 || a.nsplit <= 128);
 }
 
 inline bool mfma_ok(const SinkAttnArgs& a) {
-  return !a.f32 && a.dim % 16 == 0 && a.dim <= 128 && a.vdim % 32 == 0 && a.vdim <= 128 &&
+  return !a.f32 && a.dim % 16 == 0 && a.dim <= 256 && a.vdim % 32 == 0 && a.vdim <= 256 &&
          (reinterpret_cast<uintptr_t>(a.q) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0 &&
          (reinterpret_cast<uintptr_t>(a.out) & 7) == 0;
 }
@@ -812,9 +835,12 @@ bool sink_attn_uses_decode(const SinkAttnArgs& a) { return a.impl == 0 && decode
 hipError_t launch_sink_attn(const SinkAttnArgs& a, hipStream_t s) {
   if (a.num_seqs == 0 || a.total_q == 0) return hipSuccess;
   if (a.heads < 1 || a.kv_heads < 1 || a.heads % a.kv_heads != 0 || a.dim < 1 || a.dim > 512 || a.vdim < 1 ||
-      a.vdim > 256 || a.block_size < 1 || a.max_q < 1 || (a.bias != nullptr && a.bias_rows < 1))
+      a.vdim > 256 || a.block_size < 1 || a.max_q < 1 || a.window < 0 || a.seg < 0 || (a.bias != nullptr && a.bias_rows < 1))
     return hipErrorInvalidValue;
-  if (sink_attn_uses_decode(a)) return a.dim <= 64 ? launch_decode_r<8>(a, s) : launch_decode_r<16>(a, s);
+  if (sink_attn_uses_decode(a)) {
+    if (a.dim <= 64) return launch_decode_v<8>(a, s);
+    return a.dim <= 128 ? launch_decode_v<16>(a, s) : launch_decode_v<32>(a, s);
+  }
   if (sink_attn_uses_mfma(a)) {
     const int qpg = a.heads / a.kv_heads;
     return a.max_q * qpg <= 32 ? launch_mfma_nw<1>(a, s) : launch_mfma_nw<4>(a, s);

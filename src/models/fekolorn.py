@@ -33,7 +33,7 @@ from typing import Any, Dict, List, Optional, Tuple
 import torch
 
 from src.models.datatar import MIXERS, LayerRowPool
-from src.ops import mix, seq
+from src.ops import mix, rec, seq
 from src.parallel.tp import TPContext
 
 
@@ -63,23 +63,42 @@ class SinkAttnSpec:
     #                            wavelengths of the rotary frequencies stretched (src.ops.mix.rope_inv_freq)
     norm_after_rot: bool = False   # with head_norm: the per-head norm follows the rotation instead of preceding it
     norm_weights: bool = True      # False: the q / k norms have no weights (and the checkpoint no such tensors)
+    seg: int = 0               # > 0: positions attend within fixed segments of this many, counted from position 0
+    qkv_bias: bool = False     # q, k and v projections have biases
+    conv: int = 0              # > 0: taps of a short causal convolution on the q, k and v channels
+    rot_yarn: Optional[Tuple[float, float, float, float]] = None   # (factor, original, fast, slow): YaRN scaling of the
+    #                            rotary frequencies (src.ops.mix.rope_inv_freq_yarn)
+    rot_values: bool = False   # values turned by their position over all vdim dims (pairs i, i + vdim / 2, rot_base),
+    #                            every head's output turned back by the query's position
+    unit_sink: bool = False    # one is added to the softmax denominator (a sink whose score is 0; no such tensor)
+    head_gate: bool = False    # every head's output times a sigmoid of its own projection of the input
 
     @property
     def cache_width(self) -> int:
         return self.kv_heads * (self.dim + self.vdim)
 
+    @property
+    def channels(self) -> int:
+        return self.heads * self.dim + self.cache_width
+
     def state_shapes(self) -> Dict[str, Tuple[tuple, torch.dtype]]:
+        if self.conv:
+            return {"qkv_conv": ((self.conv - 1, self.channels), torch.float32)}
         return {}
 
     def to_config(self) -> Dict[str, Any]:
         c: Dict[str, Any] = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim,
                              "scale": self.scale}
-        if self.window:
-            c["mask"] = {"size": self.window}
+        if self.window or self.seg:
+            c["mask"] = {"size": self.window or self.seg}
         if self.rot_dims:
             c["rot"] = {"base": self.rot_base, "dims": self.rot_dims}
             if self.rot_scaling is not None:
                 c["rot"]["scaling"] = dict(zip(("factor", "low", "high", "original"), self.rot_scaling))
+            if self.rot_yarn is not None:
+                c["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), self.rot_yarn))
+        if self.conv:
+            c["conv"] = self.conv
         if self.bias_max:
             c["bias_max"] = self.bias_max
         if self.v_mix:
@@ -266,6 +285,16 @@ class SinkAttentionMixer:
         self.o = rnd(hidden, s.heads * s.vdim)
         f32 = torch.float32
         self.sink = rnd(s.heads, scale=0.5, dt=f32) if s.has_sink else None
+        if s.unit_sink:
+            self.sink = torch.zeros(s.heads, dtype=f32, device=self.device)
+        if s.v_from_k and (s.qkv_bias or s.conv) or s.qkv_bias and s.conv:
+            raise ValueError("projection biases or a convolution, and not for values taken from the keys")
+        if s.rot_values and s.vdim % 2:
+            raise ValueError("rotated values need an even vdim")
+        self.qkv_b = rnd(s.channels, scale=0.3, dt=f32) if s.qkv_bias else None
+        self.conv_w = rnd(s.channels, s.conv, scale=0.5, dt=f32) if s.conv else None
+        self.conv_wt = None
+        self.gate = rnd(s.heads, hidden) if s.head_gate else None
         if s.norm_after_rot and not s.head_norm:
             raise ValueError("norm_after_rot is a form of head_norm")
         nscale = 0.1 if s.norm_weights else 0.0   # weightless norms: ones that no checkpoint tensor replaces
@@ -286,15 +315,27 @@ class SinkAttentionMixer:
         self.rel = rnd(self.rel_rows, s.heads, scale=0.5, dt=f32) if s.bias_max else None
         self.bias = None
         self.inv_freq = mix.rope_inv_freq(s.rot_base, s.rot_dims, self.device, s.rot_scaling) if s.rot_dims else None
+        self.rot_gain = 1.0
+        if s.rot_dims and s.rot_yarn is not None:
+            self.inv_freq, self.rot_gain = mix.rope_inv_freq_yarn(s.rot_base, s.rot_dims, self.device, *s.rot_yarn)
+        self.v_inv_freq = mix.rope_inv_freq(s.rot_base, s.vdim, self.device) if s.rot_values else None
         self.finalize()
 
     def finalize(self) -> None:
-        """Derived tensors, after the weights changed: the bias per distance from the bias per bucket."""
+        """Derived tensors, after the weights changed: the bias per distance from the bias per bucket, the convolution
+        weights tap-major."""
+        if self.conv_w is not None:
+            self.conv_wt = self.conv_w.t().contiguous()
         if self.rel is not None:
             self.bias = seq.distance_bias_table(self.rel, self.spec.bias_max, self.spec.window)
 
     def tensors(self) -> List[torch.Tensor]:
-        return [t for t in (self.qkv, self.o, self.sink, self.q_norm, self.k_norm, self.vmix, self.rel) if t is not None]
+        return [t for t in (self.qkv, self.o, self.sink, self.q_norm, self.k_norm, self.vmix, self.rel, self.qkv_b,
+                            self.conv_w, self.gate) if t is not None]
+
+    def _channels(self) -> Dict[str, Tuple[int, int]]:
+        """Channel range of each projection in q | k | v order (a bias's and a convolution's, too)."""
+        return {"q": (0, self.nq), "k": (self.nq, self.nq + self.nk), "v": (self.nq + self.nk, self.nq + self.nk + self.nv)}
 
     def in_rows(self) -> int:
         return self.qkv.shape[0]
@@ -308,8 +349,16 @@ class SinkAttentionMixer:
             return _put(self.qkv[self.nq + self.nk:], t)
         if name == "o":
             return _put(self.o, t)
-        if name == "sink" and self.sink is not None:
+        if name == "sink" and self.sink is not None and not self.spec.unit_sink:
             return _put(self.sink, t)
+        if name == "g" and self.gate is not None:
+            return _put(self.gate, t)
+        if name in ("q.b", "k.b", "v.b") and self.qkv_b is not None:
+            a, b = self._channels()[name[0]]
+            return _put(self.qkv_b[a:b], t)
+        if name in ("q.conv", "k.conv", "v.conv") and self.conv_w is not None:
+            a, b = self._channels()[name[0]]
+            return _put(self.conv_w[a:b], t)
         if name == "q.norm" and self.q_norm is not None and self.spec.norm_weights:
             return _put(self.q_norm, t)
         if name == "k.norm" and self.k_norm is not None and self.spec.norm_weights:
@@ -326,8 +375,15 @@ class SinkAttentionMixer:
         out = {"q": self.qkv[: self.nq], "k": self.qkv[self.nq: self.nq + self.nk], "o": self.o}
         if self.nv:
             out["v"] = self.qkv[self.nq + self.nk:]
-        if self.sink is not None:
+        if self.sink is not None and not self.spec.unit_sink:
             out["sink"] = self.sink
+        if self.gate is not None:
+            out["g"] = self.gate
+        for k, (a, b) in self._channels().items():
+            if self.qkv_b is not None:
+                out[k + ".b"] = self.qkv_b[a:b]
+            if self.conv_w is not None:
+                out[k + ".conv"] = self.conv_w[a:b]
         if self.q_norm is not None and self.spec.norm_weights:
             out["q.norm"], out["k.norm"] = self.q_norm, self.k_norm
         if self.vmix is not None:
@@ -339,6 +395,13 @@ class SinkAttentionMixer:
     def attend(self, p: torch.Tensor, positions: torch.Tensor, meta, cache: torch.Tensor, eps: float,
                shared: Dict[str, Any]) -> torch.Tensor:
         """p [T, >= nq + nk + nv]: this mixer's q | k | v columns of a projection output. Returns W_o attn."""
+        return mix.linear(self.heads_out(p, positions, meta, cache, eps, shared), self.o)
+
+    def heads_out(self, p: torch.Tensor, positions: torch.Tensor, meta, cache: torch.Tensor, eps: float,
+                  shared: Dict[str, Any], state: Optional[Dict[str, torch.Tensor]] = None,
+                  rag: Optional[seq.Ragged] = None) -> torch.Tensor:
+        """The heads' outputs [T, H * vdim] before gate and output projection, for the same p. ``state`` / ``rag``: the
+        layer's state slots and the step's rows, for a mixer with a convolution."""
         s = self.spec
         q, k = p[:, : self.nq], p[:, self.nq: self.nq + self.nk]
         v = p[:, self.nq + self.nk: self.nq + self.nk + self.nv] if self.nv else None
@@ -351,11 +414,14 @@ class SinkAttentionMixer:
         qr = seq.qkv_prep(q, k, v, cache, s.heads, s.kv_heads, s.dim, s.vdim, positions, meta.slot_mapping, eps,
                           q_norm=self.q_norm, k_norm=self.k_norm, rot_dims=s.rot_dims, inv_freq=self.inv_freq,
                           v_unit=s.v_unit, v_lambda=lam, v_first=v_first, head_norm=s.head_norm,
-                          q_temp_coef=s.q_temp_coef, q_temp_every=s.q_temp_every, norm_after_rot=s.norm_after_rot)
-        o = seq.sink_attn(qr, cache, meta.block_tables, meta.cu_q if meta.is_prefill else None, meta.ctx_lens,
-                          positions, self.sink, self.bias, meta.max_q_len if meta.is_prefill else 1, s.heads,
-                          s.kv_heads, s.dim, s.vdim, s.window, s.scale, softcap=s.softcap, slopes=self.slopes)
-        return mix.linear(o, self.o)
+                          q_temp_coef=s.q_temp_coef, q_temp_every=s.q_temp_every, norm_after_rot=s.norm_after_rot,
+                          bias=self.qkv_b, conv_wt=self.conv_wt, conv_state=state["qkv_conv"] if s.conv else None,
+                          rag=rag if s.conv else None, rot_gain=self.rot_gain, v_inv_freq=self.v_inv_freq)
+        if s.conv:
+            rec.conv_tail_update(state["qkv_conv"], p[:, : s.channels], rag)
+        return seq.sink_attn(qr, cache, meta.block_tables, meta.cu_q if meta.is_prefill else None, meta.ctx_lens,
+                             positions, self.sink, self.bias, meta.max_q_len if meta.is_prefill else 1, s.heads,
+                             s.kv_heads, s.dim, s.vdim, s.window, s.scale, softcap=s.softcap, slopes=self.slopes, seg=s.seg)
 
     def forward_streams(self, h, positions, meta, cache, eps, state, shared, rag):
         """(y1, y2, a1, a2): the mixer's output is a1 * y1 (+ a2 * y2)."""

@@ -3,7 +3,8 @@ Dtype-generic ops (bf16 or fp32 storage, fp32 arithmetic) on the ``src/_Cmix`` H
 
 * :func:`rms_norm_ext`, :func:`post_norm_residual` — RMS norms with a plain weight or a `1 + w` gain,
   the second one applied to a sublayer's OUTPUT and added into an fp32 residual stream;
-* :func:`gated_act` — SiLU-gated, clamped sigmoid-gated and GELU-gated feed-forward activations;
+* :func:`gated_act`, :func:`gelu_act` — SiLU-gated, clamped sigmoid-gated and GELU-gated feed-forward activations, and
+  the plain exact GELU;
 * :func:`route_sigmoid_topk`, :func:`moe_input_scaled` — sigmoid-scored top-k routing whose weight scales
   the expert's input, with an optional always-on shared expert;
 * :func:`route_softmax_topk`, :func:`moe_output_weighted` — softmax-scored top-k routing with a correction that
@@ -95,6 +96,16 @@ def gated_act(gu: torch.Tensor, kind: int = ACT_SILU, limit: float = 0.0, alpha:
     gu = gu.contiguous()
     out = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
     _kern().gated_act(out, gu, kind, limit, alpha)
+    return out
+
+
+def gelu_act(z: torch.Tensor) -> torch.Tensor:
+    """0.5 z (1 + erf(z / sqrt 2)), z's shape and dtype."""
+    if not z.is_cuda:
+        return F.gelu(z.float()).to(z.dtype)
+    z = z.contiguous()
+    out = torch.empty_like(z)
+    _kern().gelu_act(out, z)
     return out
 
 
@@ -332,6 +343,23 @@ def rope_inv_freq(base: float, dims: int, device, scaling: Optional[Tuple[float,
         mid = (1.0 - s) * f / factor + s * f
         f = torch.where(wl < orig / high, f, torch.where(wl > orig / low, f / factor, mid))
     return f.float().to(device)
+
+
+def rope_inv_freq_yarn(base: float, dims: int, device, factor: float, original: float, fast: float,
+                       slow: float) -> Tuple[torch.Tensor, float]:
+    """YaRN: (fp32 [dims / 2] frequencies, factor of the cosines and sines). With the pair index that makes t full turns
+    over ``original`` positions, d(t) = dims ln(original / (2 pi t)) / (2 ln base), the frequency base^(-2 i / dims) is kept
+    below floor(d(fast)), divided by ``factor`` above ceil(d(slow)) and blended linearly in i between; computed in
+    float64 and rounded once."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / dims)
+
+    def d(turns: float) -> float:
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(d(fast)), 0), min(math.ceil(d(slow)), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (f / factor * ramp + f * (1.0 - ramp)).float().to(device), 0.1 * math.log(factor) + 1.0
 
 
 def latent_kv_write(cache: torch.Tensor, kv: torch.Tensor, w: torch.Tensor, positions: torch.Tensor,

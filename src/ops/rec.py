@@ -11,9 +11,10 @@ Ops for recurrent mixers whose state is a vector or matrix per channel or head, 
 * :func:`exp_gate_scan` — exponential input gate and sigmoid forget gate in log space with a running maximum:
   the per-token decay, input weight and normaliser floor of a matrix-memory LSTM;
 * :func:`gated_linear_attn` — the matrix recurrence S <- a_t S + b_t k_t v_t^T, o_t = S^T q_t with one (a_t, b_t) per
-  token and head, grouped q / k, and an optional normaliser vector n <- a_t n + b_t k_t read out as n . q;
-* :func:`head_norm_gate` — the read-out divided by max(|n . q|, floor) + 1e-6, every head RMS-normed, weight,
-  sigmoid gate;
+  token and head, grouped q / k, and an optional normaliser vector n <- a_t n + b_t k_t read out as n . q; or with a
+  decay per key channel (row of S), sigmoid(z)^(1/tau);
+* :func:`head_norm_gate` — (optional: the read-out divided by max(|n . q|, floor) + 1e-6,) every head RMS-normed, weight,
+  sigmoid or SiLU gate;
 * :func:`skip_gate_group_norm` — (o + D_h x) * SiLU(z), RMS norm in equal parts of the row, weight;
 * :func:`pair_post_norm_residual` — two sublayer outputs, each RMS-normed over the row with its own weight,
   averaged, then the layer's norm on the result, times a constant, added into the fp32 residual: one launch.
@@ -39,11 +40,13 @@ def _rms(x: torch.Tensor, eps: float) -> torch.Tensor:
     return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
 
 
-def embed_scaled(ids: torch.Tensor, embed: torch.Tensor, scale: float) -> Tuple[torch.Tensor, torch.Tensor]:
-    """(resid fp32 [T, W] = embed[ids] * scale, act = resid in embed's dtype; the same tensor for an fp32 table)."""
+def embed_scaled(ids: torch.Tensor, embed: torch.Tensor, scale: float,
+                 copy: bool = True) -> Tuple[torch.Tensor, torch.Tensor]:
+    """(resid fp32 [T, W] = embed[ids] * scale, act = resid in embed's dtype; the same tensor for an fp32 table, or
+    with ``copy`` off)."""
     T, W = ids.shape[0], embed.shape[1]
     resid = torch.empty(T, W, dtype=torch.float32, device=ids.device)
-    act = resid if embed.dtype == torch.float32 else torch.empty(T, W, dtype=embed.dtype, device=ids.device)
+    act = resid if not copy or embed.dtype == torch.float32 else torch.empty(T, W, dtype=embed.dtype, device=ids.device)
     if ids.is_cuda:
         _kern().embed_scaled(resid, None if act is resid else act, embed, ids, float(scale))
         return resid, act
@@ -161,26 +164,33 @@ def exp_gate_scan(x: torch.Tensor, ioff: int, foff: int, i_bias: torch.Tensor, f
     return abe
 
 
-def gated_linear_attn(x: torch.Tensor, qoff: int, koff: int, voff: int, ab: torch.Tensor, state: torch.Tensor,
+def gated_linear_attn(x: torch.Tensor, qoff: int, koff: int, voff: int, ab: Optional[torch.Tensor], state: torch.Tensor,
                       n_state: Optional[torch.Tensor], heads: int, groups: int, dim: int, vdim: int, qscale: float,
-                      rag: Ragged) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+                      rag: Ragged, z: Optional[torch.Tensor] = None, z_bias: Optional[torch.Tensor] = None,
+                      tau: float = 1.0) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
     """x [T, *]: q | k (groups * dim each; head h reads group h // (heads / groups)) and v (heads * vdim) at column
     offsets qoff / koff / voff. Per (sequence, head), token by token, with (a, b) = ab[t, h, :2]:
     S <- a S + b k v^T;  o = S^T (q * qscale), S [dim, vdim] fp32 in ``state`` [slots, H, dim, vdim]. With ``n_state``
-    [slots, H, dim] also n <- a n + b k and nq = n . (q * qscale). Returns (o [T, H * vdim] fp32, nq [T, H] fp32 or
-    None)."""
+    [slots, H, dim] also n <- a n + b k and nq = n . (q * qscale). With ``z`` [T, H * dim] (any row stride) instead of
+    ``ab``: b = 1 and row i of S decays by its own a_i = sigmoid(z_i + z_bias_i)^(1 / tau). Returns (o [T, H * vdim] fp32,
+    nq [T, H] fp32 or None)."""
     T = x.shape[0]
     o = torch.empty(T, heads * vdim, dtype=torch.float32, device=x.device)
     nq = torch.empty(T, heads, dtype=torch.float32, device=x.device) if n_state is not None else None
     if x.is_cuda:
         _kern().gated_linear_attn(o, nq, x, qoff, koff, voff, ab, state, n_state, heads, groups, dim, vdim,
-                                  float(qscale), rag.positions, rag.cu_q, rag.state_slots)
+                                  float(qscale), rag.positions, rag.cu_q, rag.state_slots, z, z_bias, 1.0 / float(tau))
         return o, nq
     rep = heads // groups
     q = x[:, qoff: qoff + groups * dim].float().view(T, groups, dim).repeat_interleave(rep, 1) * qscale
     k = x[:, koff: koff + groups * dim].float().view(T, groups, dim).repeat_interleave(rep, 1)
     v = x[:, voff: voff + heads * vdim].float().view(T, heads, vdim)
     ov = o.view(T, heads, vdim)
+    if z is not None:
+        dec = torch.exp(F.logsigmoid(z.float() + z_bias) / tau).view(T, heads, dim, 1)
+        bs = torch.ones(T, heads)
+    else:
+        dec, bs = ab[:, :, 0, None, None], ab[:, :, 1]
     pos = rag.positions.tolist()
     for q0, n, slot in rag.spans(T):
         fresh = pos[q0] <= 0
@@ -189,11 +199,11 @@ def gated_linear_attn(x: torch.Tensor, qoff: int, koff: int, voff: int, ab: torc
         if n_state is not None:
             nv = torch.zeros_like(n_state[slot]) if fresh else n_state[slot].clone()
         for t in range(q0, q0 + n):
-            a, b = ab[t, :, 0], ab[t, :, 1]
-            S = a[:, None, None] * S + (b[:, None] * k[t])[:, :, None] * v[t][:, None, :]
+            a, b = dec[t], bs[t]
+            S = a * S + (b[:, None] * k[t])[:, :, None] * v[t][:, None, :]
             ov[t] = torch.einsum("hdv,hd->hv", S, q[t])
             if nv is not None:
-                nv = a[:, None] * nv + b[:, None] * k[t]
+                nv = a[:, 0] * nv + b[:, None] * k[t]
                 nq[t] = (nv * q[t]).sum(-1)
         state[slot] = S
         if nv is not None:
@@ -201,18 +211,26 @@ def gated_linear_attn(x: torch.Tensor, qoff: int, koff: int, voff: int, ab: torc
     return o, nq
 
 
-def head_norm_gate(o: torch.Tensor, nq: torch.Tensor, abe: torch.Tensor, g: torch.Tensor, w: torch.Tensor, heads: int,
-                   vdim: int, eps: float) -> torch.Tensor:
-    """o [T, H * vdim] fp32, nq [T, H], abe [T, H, 3] (its last entry the floor), g [T, H * vdim] (any row stride):
-    u = o_h / (max(|nq_h|, floor_h) + 1e-6); out = rms(u) over each head * w * sigmoid(g), in g's dtype."""
+def head_norm_gate(o: torch.Tensor, nq: Optional[torch.Tensor], abe: Optional[torch.Tensor], g: torch.Tensor,
+                   w: torch.Tensor, heads: int, vdim: int, eps: float, gate_silu: bool = False, mult: float = 1.0,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """o [T, H * vdim] fp32, g [T, H * vdim] (any row stride), w [H * vdim] or [vdim] (shared by the heads):
+    mult * rms(u) over each head * w * gate(g) in g's dtype, gate = SiLU or sigmoid; u = o, or with nq [T, H] and
+    abe [T, H, 3] (its last entry the floor) u = o_h / (max(|nq_h|, floor_h) + 1e-6). ``out``: where to write ([T, H * vdim],
+    any row stride)."""
     T = o.shape[0]
-    out = torch.empty(T, heads * vdim, dtype=g.dtype, device=o.device)
+    if out is None:
+        out = torch.empty(T, heads * vdim, dtype=g.dtype, device=o.device)
     if o.is_cuda:
-        _kern().head_norm_gate(out, o, nq, abe, g, w, heads, vdim, float(eps))
+        _kern().head_norm_gate(out, o, nq, abe, g, w, heads, vdim, float(eps), bool(gate_silu), float(mult))
         return out
-    den = torch.maximum(nq.abs(), abe[..., 2]) + 1e-6
-    u = _rms(o.view(T, heads, vdim) / den[..., None], eps).reshape(T, heads * vdim)
-    return (u * w * torch.sigmoid(g.float())).to(g.dtype)
+    u = o.view(T, heads, vdim)
+    if nq is not None:
+        u = u / (torch.maximum(nq.abs(), abe[..., 2]) + 1e-6)[..., None]
+    gf = g.float()
+    gate = F.silu(gf) if gate_silu else torch.sigmoid(gf)
+    out.copy_(mult * (_rms(u, eps) * w.view(-1, vdim)).reshape(T, heads * vdim) * gate)
+    return out
 
 
 def skip_gate_group_norm(o: torch.Tensor, x: torch.Tensor, D: torch.Tensor, z: torch.Tensor, w: torch.Tensor,

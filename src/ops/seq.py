@@ -10,7 +10,7 @@ Ops for models that carry per-sequence state besides the paged KV cache, on the 
 * :func:`delta_prep`, :func:`conv_state_update`, :func:`gated_delta` — short causal convolutions and the gated
   delta rule with its fp32 matrix state per head;
 * :func:`qkv_prep`, :func:`sink_attn` — grouped-query attention over a paged cache with a softmax sink, an
-  optional sliding window, rotate-half rotary positions, whole-projection q/k norms, value norms or cross-layer
+  optional sliding window or fixed segments, rotate-half rotary positions, whole-projection q/k norms, value norms or cross-layer
   value mixing, and a learned bias per (distance, head).
 
 A step is a ragged batch (:class:`Ragged`): sequence s owns rows ``cu_q[s] .. cu_q[s + 1] - 1`` (``cu_q`` None: one
@@ -147,19 +147,19 @@ def poly_norm_act(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tens
 
 
 # ---------------------------------------------------------------------------------------------- gated delta rule
-def delta_prep(x: torch.Tensor, b: torch.Tensor, a: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor,
-               A_log: torch.Tensor, dt_bias: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int,
+def delta_prep(x: torch.Tensor, b: torch.Tensor, a: Optional[torch.Tensor], conv_w: torch.Tensor,
+               conv_state: torch.Tensor, A_log: Optional[torch.Tensor], dt_bias: Optional[torch.Tensor], heads: int, kv_heads: int, dim: int, vdim: int,
                rag: Ragged, conv_wt: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, torch.Tensor]:
     """x [T, C = 2 G dim + H vdim] = [q | k | v] channels: causal convolution over the sequence's last ``taps``
     inputs (those before the step from conv_state [slots, taps - 1, C]) + SiLU; q and k heads to unit length
     (q also times dim^-1/2). Returns (qkv32 [T, C] fp32, bg [T, 2 H] fp32 = [sigmoid(b) | exp(-exp(A_log) *
-    softplus(a + dt_bias))]). On the GPU a step with one row per sequence also moves the row's input into
+    softplus(a + dt_bias))]; without ``a`` bg [T, H] = sigmoid(b)). On the GPU a step with one row per sequence also moves the row's input into
     conv_state (:func:`conv_state_update` then has nothing left to do). ``conv_wt``: the same weights tap-major,
     [taps, C] contiguous, which lets the kernel load them 16 bytes at a time in prompt-sized bf16 steps."""
     T, C = x.shape
     taps = conv_w.shape[1]
     qkv32 = torch.empty(T, C, dtype=torch.float32, device=x.device)
-    bg = torch.empty(T, 2 * heads, dtype=torch.float32, device=x.device)
+    bg = torch.empty(T, heads if a is None else 2 * heads, dtype=torch.float32, device=x.device)
     if x.is_cuda:
         _kern().delta_prep(qkv32, bg, x, b, a, conv_w, conv_wt, conv_state, A_log, dt_bias, heads, kv_heads, dim, vdim,
                            rag.positions, rag.cu_q, rag.state_slots)
@@ -179,7 +179,8 @@ def delta_prep(x: torch.Tensor, b: torch.Tensor, a: torch.Tensor, conv_w: torch.
     qk[:, :G] *= dim ** -0.5
     qkv32[:, : 2 * G * dim] = qk.reshape(T, 2 * G * dim)
     bg[:, :heads] = torch.sigmoid(b.float())
-    bg[:, heads:] = torch.exp(-torch.exp(A_log) * F.softplus(a.float() + dt_bias))
+    if a is not None:
+        bg[:, heads:] = torch.exp(-torch.exp(A_log) * F.softplus(a.float() + dt_bias))
     return qkv32, bg
 
 
@@ -201,32 +202,44 @@ def conv_state_update(conv_state: torch.Tensor, x: torch.Tensor, heads: int, kv_
 
 
 def gated_delta(qkv32: torch.Tensor, bg: torch.Tensor, gate: torch.Tensor, norm_w: torch.Tensor, eps: float,
-                state: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, rag: Ragged) -> torch.Tensor:
+                state: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, rag: Ragged,
+                z: Optional[torch.Tensor] = None, z_bias: Optional[torch.Tensor] = None,
+                A_log: Optional[torch.Tensor] = None, gate_sigmoid: bool = False, mult: float = 1.0,
+                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per (sequence, head), token by token: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q; the state S
-    [dim, vdim] fp32 lives in ``state`` [slots, H, dim, vdim]. Returns o / rms(o) * norm_w * silu(gate),
-    [T, H * vdim] in gate's dtype."""
+    [dim, vdim] fp32 lives in ``state`` [slots, H, dim, vdim]. Returns mult * o / rms(o) * norm_w * silu(gate) (sigmoid with
+    ``gate_sigmoid``), [T, H * vdim] in gate's dtype, written to ``out`` (any row stride) if given. With ``z`` [T, H * dim]
+    (any row stride) g is a decay per row of S, exp(-exp(A_log[h]) * softplus(z + z_bias)), and bg [T, H] holds beta only."""
     T = qkv32.shape[0]
-    out = torch.empty(T, heads * vdim, dtype=gate.dtype, device=gate.device)
+    if out is None:
+        out = torch.empty(T, heads * vdim, dtype=gate.dtype, device=gate.device)
     if gate.is_cuda:
         _kern().gated_delta(out, qkv32, bg, gate, norm_w, eps, state, heads, kv_heads, dim, vdim, rag.positions,
-                            rag.cu_q, rag.state_slots)
+                            rag.cu_q, rag.state_slots, z, z_bias, A_log, bool(gate_sigmoid), float(mult))
         return out
     G, rep = kv_heads, heads // kv_heads
     q = qkv32[:, : G * dim].view(T, G, dim).repeat_interleave(rep, 1)
     k = qkv32[:, G * dim: 2 * G * dim].view(T, G, dim).repeat_interleave(rep, 1)
     v = qkv32[:, 2 * G * dim:].view(T, heads, vdim)
+    if z is not None:
+        dec = F.softplus(z.float() + z_bias).view(T, heads, dim)
+        dec = torch.exp(-torch.exp(A_log)[None, :, None] * dec)[..., None]
+    else:
+        dec = bg[:, heads:, None, None]
     o = torch.empty(T, heads, vdim)
     pos = rag.positions.tolist()
     for q0, n, slot in rag.spans(T):
         S = state[slot].clone() if pos[q0] > 0 else torch.zeros_like(state[slot])      # [H, dim, vdim]
         for t in range(q0, q0 + n):
-            S = S * bg[t, heads:, None, None]
+            S = S * dec[t]
             u = bg[t, :heads, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
             S = S + k[t][:, :, None] * u[:, None, :]
             o[t] = torch.einsum("hdv,hd->hv", S, q[t])
         state[slot] = S
-    o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * norm_w * F.silu(gate.float().view(T, heads, vdim))
-    return o.reshape(T, heads * vdim).to(gate.dtype)
+    gf = gate.float().view(T, heads, vdim)
+    o = mult * o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps) * norm_w * (torch.sigmoid(gf) if gate_sigmoid else F.silu(gf))
+    out.copy_(o.reshape(T, heads * vdim))
+    return out
 
 
 # ---------------------------------------------------------------------------------------------------- attention
@@ -256,43 +269,69 @@ def qkv_prep(q: torch.Tensor, k: torch.Tensor, v: Optional[torch.Tensor], cache:
              q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None, rot_dims: int = 0,
              inv_freq: Optional[torch.Tensor] = None, v_unit: bool = False, v_lambda: Optional[torch.Tensor] = None,
              v_first: Optional[torch.Tensor] = None, head_norm: bool = False, q_temp_coef: float = 0.0,
-             q_temp_every: int = 1, norm_after_rot: bool = False) -> torch.Tensor:
+             q_temp_every: int = 1, norm_after_rot: bool = False, bias: Optional[torch.Tensor] = None,
+             conv_wt: Optional[torch.Tensor] = None, conv_state: Optional[torch.Tensor] = None,
+             rag: Optional[Ragged] = None, rot_gain: float = 1.0,
+             v_inv_freq: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The step between the q/k/v projection and the attention, one launch: optional RMS norm of q and of k (plain
     weights) over the whole projection or, with ``head_norm``, of every head by itself with weights [dim] shared by
     the heads; optional query temperature, q times 1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1) after its
     norm; optional rotate-half rotary on the first ``rot_dims`` dims of every head (pair i, i + rot_dims / 2, angle
     position * inv_freq[i]) — with ``norm_after_rot`` (and ``head_norm``) the rotation comes first and the per-head
     norm acts on the rotated heads; values either divided by their per-head root mean square or blended as
-    (1 - l) v + l v_first; ``v`` None: the values are the keys as projected, before norm and rotation. Writes the
-    token's keys and values into the cache at slots[t] (< 0: skipped; a block's interior is head-major,
+    (1 - l) v + l v_first; ``v`` None: the values are the keys as projected, before norm and rotation. With q, k and v in
+    adjacent columns (C channels) the step starts with ``bias`` [C] fp32, or with a short causal convolution of each
+    channel over the sequence (``conv_wt`` [taps, C] fp32, the current row's weights last; inputs before the step from
+    conv_state [slots, taps - 1, C], moved on in the same launch when the step has one row per sequence, else by
+    :func:`src.ops.rec.conv_tail_update`). ``rot_gain`` multiplies the cosines and sines of q and k; ``v_inv_freq``
+    [vdim / 2]: the values are turned too, pair (i, i + vdim / 2) by position * v_inv_freq[i]. Writes the token's keys and values into the cache at slots[t] (< 0: skipped; a block's interior is head-major,
     [G][block_size][k | v]) and returns q [T, H * dim]."""
     T = q.shape[0]
     if q.is_cuda:
         q_out = torch.empty(T, heads * dim, dtype=q.dtype, device=q.device)
         _kern().qkv_prep(q_out, cache, q, k, v, heads, kv_heads, dim, vdim, q_norm, k_norm, rot_dims, inv_freq, v_unit,
                          v_lambda, v_first, eps, positions, slots, head_norm, float(q_temp_coef), int(q_temp_every),
-                         bool(norm_after_rot))
+                         bool(norm_after_rot), bias, conv_wt, conv_state, None if rag is None else rag.cu_q,
+                         None if rag is None else rag.state_slots, float(rot_gain), v_inv_freq)
         return q_out
     if v is None:
         v = k
     qf, kf, vf = q.float(), k.float(), v.float()
+    if bias is not None or conv_wt is not None:
+        nq, nk = heads * dim, kv_heads * dim
+        u = torch.cat([qf, kf, vf], 1)
+        if bias is not None:
+            y = u + bias
+        else:
+            taps, y = conv_wt.shape[0], torch.empty_like(u)
+            p_ = rag.positions.tolist()
+            for q0, n_, slot in rag.spans(T):
+                hist = conv_state[slot].clone() if p_[q0] > 0 else torch.zeros(taps - 1, u.shape[1])
+                if 0 < p_[q0] < taps - 1:
+                    hist[: taps - 1 - p_[q0]] = 0
+                s_ = torch.cat([hist, u[q0:q0 + n_]], 0)
+                y[q0:q0 + n_] = (s_.unfold(0, taps, 1) * conv_wt.t()[None]).sum(-1)
+        qf, kf, vf = y[:, :nq], y[:, nq: nq + nk], y[:, nq + nk:]
     if v_lambda is not None:
         vf = (1.0 - v_lambda) * vf + v_lambda * v_first.float()
 
-    def rot(x, n):
-        half = rot_dims // 2
-        ang = positions.float()[:, None] * inv_freq[None, :]
-        c, s = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
-        x = x.view(T, n, dim).clone()
-        u, w = x[..., :half].clone(), x[..., half:rot_dims].clone()
+    def turn(x, n, size, dims, freq, gain):
+        half = dims // 2
+        ang = positions.float()[:, None] * freq[None, :]
+        c, s = (torch.cos(ang) * gain)[:, None, :], (torch.sin(ang) * gain)[:, None, :]
+        x = x.reshape(T, n, size).clone()
+        u, w = x[..., :half].clone(), x[..., half:dims].clone()
         x[..., :half] = u * c - w * s
-        x[..., half:rot_dims] = w * c + u * s
-        return x.reshape(T, n * dim)
+        x[..., half:dims] = w * c + u * s
+        return x.reshape(T, n * size)
+
+    def rot(x, n):
+        return turn(x, n, dim, rot_dims, inv_freq, rot_gain)
 
     if rot_dims and norm_after_rot:
         qf, kf = rot(qf, heads), rot(kf, kv_heads)
     if q_norm is not None and head_norm:
-        qh, kh = qf.view(T, heads, dim), kf.view(T, kv_heads, dim)
+        qh, kh = qf.reshape(T, heads, dim), kf.reshape(T, kv_heads, dim)
         qf = (qh / torch.sqrt((qh * qh).mean(-1, keepdim=True) + eps) * q_norm).reshape(T, heads * dim)
         kf = (kh / torch.sqrt((kh * kh).mean(-1, keepdim=True) + eps) * k_norm).reshape(T, kv_heads * dim)
     elif q_norm is not None:
@@ -303,21 +342,25 @@ def qkv_prep(q: torch.Tensor, k: torch.Tensor, v: Optional[torch.Tensor], cache:
         qf = qf * (1.0 + q_temp_coef * torch.log(steps + 1.0))[:, None]
     if rot_dims and not norm_after_rot:
         qf, kf = rot(qf, heads), rot(kf, kv_heads)
+    if v_inv_freq is not None:
+        vf = turn(vf, kv_heads, vdim, vdim, v_inv_freq, 1.0)
     if v_unit:
         vh = vf.view(T, kv_heads, vdim)
         vf = (vh / torch.sqrt((vh * vh).mean(-1, keepdim=True) + eps)).reshape(T, kv_heads * vdim)
     ok = slots >= 0
     _head_major(cache, kv_heads)[slots[ok]] = torch.cat(
-        [kf.view(T, kv_heads, dim), vf.view(T, kv_heads, vdim)], 2)[ok].to(cache.dtype)
+        [kf.reshape(T, kv_heads, dim), vf.reshape(T, kv_heads, vdim)], 2)[ok].to(cache.dtype)
     return qf.to(q.dtype)
 
 
 def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, cu_q: Optional[torch.Tensor],
               ctx_lens: torch.Tensor, positions: torch.Tensor, sink: Optional[torch.Tensor],
               bias: Optional[torch.Tensor], max_q: int, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
-              scale: float, impl: int = 0, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
+              scale: float, impl: int = 0, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
+              seg: int = 0) -> torch.Tensor:
     """Grouped-query attention over the cache that :func:`qkv_prep` writes. The query at position p sees the cached
-    positions j <= p with p - j < window (0: all). Score: s = (q . k_j) * scale; with ``softcap`` > 0,
+    positions j <= p with p - j < window (0: all) and, with ``seg`` > 0, of its own segment: floor(j / seg) =
+    floor(p / seg). Score: s = (q . k_j) * scale; with ``softcap`` > 0,
     s <- softcap * tanh(s / softcap); then - slopes[h] * (p - j) (``slopes`` [H] fp32, a linear distance penalty)
     and + bias[min(p - j, rows - 1), h]. The softmax denominator has one more term exp(sink[h]) when ``sink`` is
     given. Returns [T, H * vdim]. ``impl``: 0 = the matrix-core kernel where it applies, 1 = the FMA kernel, 2 = the
@@ -326,7 +369,7 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
     if q.is_cuda:
         out = torch.empty(T, heads * vdim, dtype=q.dtype, device=q.device)
         _kern().sink_attn(out, q, cache, block_tables, cu_q, ctx_lens, positions, sink, bias, max_q, heads, kv_heads,
-                          dim, vdim, window, scale, impl, float(softcap), slopes)
+                          dim, vdim, window, scale, impl, float(softcap), slopes, int(seg))
         return out
     bs = cache.shape[1]
     hm = _head_major(cache, kv_heads)
@@ -347,6 +390,8 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
         for t in range(cu[s], cu[s + 1]):
             n = pos[t] - j
             ok = (n >= 0) & ((n < window) if window > 0 else torch.ones_like(n, dtype=torch.bool))
+            if seg > 0:
+                ok &= j // seg == pos[t] // seg
             sc = torch.einsum("hd,jhd->hj", qh[t], kk) * scale
             if softcap:
                 sc = softcap * torch.tanh(sc / softcap)
