@@ -139,6 +139,10 @@ def parse(argv=None):
                    help="instead of the default workload: Kogerax beside Fekolorn (recurrent state next to attention) at "
                         "equal sizes, prefill / decode throughput and its kernels alone (bench/kogerax_compare.py)")
     p.add_argument("--kogerax-args", default="", help="arguments passed on to bench/kogerax_compare.py")
+    p.add_argument("--rerozen-compare", action="store_true",
+                   help="instead of the default workload: Rerozen beside Fekolorn (attention next to a linear recurrence) at "
+                        "equal sizes, prefill / decode throughput and its kernels alone (bench/rerozen_compare.py)")
+    p.add_argument("--rerozen-args", default="", help="arguments passed on to bench/rerozen_compare.py")
     return p.parse_args(argv)
 
 
@@ -505,6 +509,15 @@ def main(argv=None) -> int:
         mod = importlib.util.module_from_spec(spec)
         spec.loader.exec_module(mod)
         return mod.main(shlex.split(args.kogerax_args))
+    if args.rerozen_compare:  # likewise a separate measurement
+        import importlib.util
+        import shlex
+
+        spec = importlib.util.spec_from_file_location("rerozen_compare",
+                                                      os.path.join(ROOT, "bench", "rerozen_compare.py"))
+        mod = importlib.util.module_from_spec(spec)
+        spec.loader.exec_module(mod)
+        return mod.main(shlex.split(args.rerozen_args))
     if needs_launcher(args):
         return self_launch(args, argv)
     world = int(os.environ.get("WORLD_SIZE", "1"))
