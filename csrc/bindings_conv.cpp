@@ -52,14 +52,25 @@ void conv_norm(Tensor h, Tensor resid_in, OptTensor resid_out, OptTensor y, Tens
   a.y = nullptr;
   a.ystride = 0;
   a.y_f32 = false;
+  a.yslabs = 1;
+  a.yslab = 0;
   if (y.has_value()) {
-    check_rows(*y, "y");
     a.y_f32 = is_f32(*y, "y");
-    TORCH_CHECK(y->size(0) == T && y->size(1) == W && resid_out.has_value(), "y [T, W], with resid_out");
+    if (y->dim() == 3) {
+      TORCH_CHECK(a.y_f32 && y->is_contiguous() && y->size(0) >= 1 && y->size(1) == T && y->size(2) == W,
+                  "y as partial sums: fp32 [n, T, W] contiguous");
+      a.yslabs = (int)y->size(0);
+      a.yslab = T * W;
+      a.ystride = W;
+    } else {
+      check_rows(*y, "y");
+      TORCH_CHECK(y->size(0) == T && y->size(1) == W, "y [T, W]");
+      a.ystride = y->stride(0);
+    }
+    TORCH_CHECK(resid_out.has_value(), "y needs resid_out");
     check_c(*resid_out, at::kFloat, "resid_out");
     TORCH_CHECK(resid_out->sizes() == resid_in.sizes(), "resid_out like resid_in");
     a.y = y->data_ptr();
-    a.ystride = y->stride(0);
     a.resid_out = resid_out->data_ptr<float>();
   }
   a.w = f32_vec(w, W, "w");

@@ -19,6 +19,8 @@ struct ConvNormArgs {
   const void* y;           // [T, W], row stride ystride, or nullptr
   int64_t ystride;
   bool y_f32;
+  int yslabs;              // fp32 y as the sum of this many partial sums, yslab elements apart (else 1)
+  int64_t yslab;
   const float* w;          // [W]
   float eps;
   const float* conv_wt;    // [taps, W], tap-major, the current row's weights last; nullptr: no convolution

@@ -10,13 +10,14 @@
 //                             channel's states in the registers of 1 - 4 lanes for the whole step
 //   exp_gate_scan             log-space input / forget gates under a running maximum: a wave-wide scan over tokens
 //   gated_linear_attn         S <- a S + b k v^T, o = S^T q: one workgroup per (sequence, head, block of columns), the
-//                             state in registers (a column per lane quad); the normaliser n <- a n + b k with its
+//                             state in registers (four columns per group of 4 - 16 lanes); the normaliser n <- a n + b k with its
 //                             read-out n . q rides on the first wave; optionally a decay per row of S,
 //                             sigmoid(z)^(1/tau), computed while a trip is staged
 //   head_norm_gate            (o / (max(|n . q|, floor) + 1e-6), optional,) per-head RMS norm, weight, sigmoid or SiLU gate
 //   skip_gate_group_norm      (o + D x) * silu(z), RMS norm in equal parts of the row, weight
 //   pair_post_norm_residual   resid += mult * rms((rms(y1) w1 + rms(y2) w2) / 2) * (1 + w)
 #include "common.h"
+#include "lane_reduce.h"
 #include "rec_launchers.h"
 
 namespace die {
@@ -211,16 +212,6 @@ __global__ void __launch_bounds__(NT) conv_tail_update_kernel(float* conv_state,
 constexpr int TB = 16;   // tokens staged per trip
 constexpr int SCH = 256; // threads per workgroup of the scan
 
-// softplus in bf16 steps: hardware exponential and logarithm (v_exp_f32 / v_log_f32), a series where 1 + e^z rounds
-template <bool FAST> __device__ __forceinline__ float step_size(float z) {
-  if constexpr (FAST) {
-    const float e = __expf(-fabsf(z));
-    const float l = e < 9.765625e-4f ? e - 0.5f * e * e : __logf(1.0f + e);
-    return fmaxf(z, 0.f) + l;
-  } else {
-    return softplusf(z);
-  }
-}
 // silu(z): bf16 steps use the hardware's exponential and reciprocal
 template <bool FAST> __device__ __forceinline__ float gate_of(float z) {
   if constexpr (FAST)
@@ -307,7 +298,7 @@ __global__ void __launch_bounds__(SCH) selective_scan_kernel(SelectiveScanArgs a
 #pragma unroll
     for (int tt = 0; tt < TB; ++tt) {
       if (tt < nb) {
-        const float x = xr[tt], d = step_size<FAST>(dr[tt] + dtb);
+        const float x = xr[tt], d = softplus_of<FAST>(dr[tt] + dtb);
         const float dx = d * x;
         const float4* Bt = reinterpret_cast<const float4*>(Bs + tt * NPAD + part * NP);
         const float4* Ct = reinterpret_cast<const float4*>(Cs + tt * NPAD + part * NP);
@@ -403,90 +394,173 @@ __global__ void __launch_bounds__(64) exp_gate_scan_kernel(float* abe, const voi
 }
 
 // ---------------------------------------------------------------------------------------- matrix recurrence
-// One workgroup per (head, sequence, block of VC columns). The state lives in registers for the whole step: column j
-// is split over the 4 lanes of a quad, lane `part` holding rows [part * DP, (part + 1) * DP). A token costs each lane
-// 2 * DP multiply-adds and one quad reduction; q (scaled) and k come from LDS as float4 broadcasts, b scales the
-// value. The normaliser n <- a n + b k (a vector of `dim` rows, RP per lane) is carried by the first wave of column
-// block 0, which runs a trip's tokens over the staged k and q once more after its columns and reduces the TB dot
-// products n . q over its lanes. (As a column of its own the normaliser would add a ninth wave to workgroups of 512
-// threads; measured, that ran 1.8x slower than the kernel without it, and a one-wave launch beside it 1.7x.)
-// CD: a decay per row of the state instead of one per head.
-template <int DP, bool F32, bool CD>
-__global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs a, RaggedRows r, int VC) {
+// 4 consecutive values at p[i + c] of a row piece of n values (c a multiple of 4), zeros beyond it. VEC (n and the row's
+// start multiples of 4, the base aligned): one 8- / 16-byte load without a branch around it, so that a run of these stays
+// in flight together.
+template <bool F32, bool VEC> __device__ __forceinline__ float4 ld4z(const void* p, int64_t i, int c, int n) {
+  if constexpr (VEC) {
+    const int64_t at = i + (c < n ? c : 0);
+    float4 v;
+    if constexpr (F32) {
+      v = *reinterpret_cast<const float4*>(reinterpret_cast<const float*>(p) + at);
+    } else {
+      const uint2 w = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(p) + at);
+      v = make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
+                      __uint_as_float(w.y & 0xffff0000u));
+    }
+    return c < n ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+  } else {
+    float f[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f[e] = c + e < n ? ldt<F32>(p, i + c + e) : 0.f;
+    return make_float4(f[0], f[1], f[2], f[3]);
+  }
+}
+
+// One workgroup per (head, sequence, block of VC columns). The state lives in registers for the whole step: a group of LN
+// lanes holds 4 columns, lane l of it the rows 4 LN m + 4 l + i (m < M, i < 4). A token costs a lane 3 multiply-adds per
+// value and one sum over its group (on DPP adds); q (scaled), k and with CD the decays come from LDS as consecutive
+// float4s, b scales the value. Up to TB tokens are staged per trip, the next trip's rows are already in flight. The
+// normaliser n <- a n + b k (a vector of `dim` rows, RP per lane) is carried by the first wave of column block 0, which
+// runs a trip's tokens over the staged k and q once more after its columns and reduces the TB dot products n . q over its
+// lanes. (As a column of its own the normaliser would add a ninth wave to workgroups of 512 threads; measured, that ran
+// 1.8x slower than the kernel without it, and a one-wave launch beside it 1.7x.) CD: a decay per row of the state instead
+// of one per head. VEC: dim, vdim, the column offsets and the row strides are multiples of 4.
+template <int LN, int M, bool F32, bool CD, bool VEC>
+__global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs a, RaggedRows r, int VC, int TT) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  constexpr int DPAD = 4 * DP;
+  constexpr int DPAD = 4 * LN * M, NE = 2, NV = 4;
   const int d = a.dim, dv = a.vdim, H = a.heads;
+  const int vcp = (VC + 3) & ~3;
   float* qs = sm;                  // [TB][DPAD], zero beyond dim
   float* ks = qs + TB * DPAD;      // [TB][DPAD]
-  float* vs = ks + TB * DPAD;      // [TB][VC]
-  float* as = vs + TB * VC;        // [TB][2]: a, b, or [TB][DPAD]: a per row of S
+  float* vs = ks + TB * DPAD;      // [TB][vcp]
+  float* as = vs + TB * vcp;       // [TB][2]: a, b, or [TB][DPAD]: a per row of S
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x;
   const int v0 = blockIdx.z * VC;
   const int ncol = min(VC, dv - v0);
-  const int j = tid >> 2, part = tid & 3;
+  const int l = tid % LN, j0 = 4 * (tid / LN);
   const int g = h / (H / a.groups);
   const int q0 = r.cu_q ? r.cu_q[s] : s;
   const int L = r.cu_q ? r.cu_q[s + 1] - q0 : 1;
   if (L <= 0) return;
   const bool fresh = r.positions[q0] <= 0;
-  float* st = a.state + ((int64_t)r.state_slots[s] * H + h) * (int64_t)d * dv + v0 + j;
-  float S[DP];
-#pragma unroll
-  for (int i = 0; i < DP; ++i) {
-    const int row = part * DP + i;
-    S[i] = (!fresh && row < d && j < ncol) ? st[(int64_t)row * dv] : 0.f;
-  }
+  const bool live = j0 < ncol;
+  float* st = a.state + ((int64_t)r.state_slots[s] * H + h) * (int64_t)d * dv + v0;
   constexpr int RP = DPAD > 64 ? DPAD / 64 : 1;
   const bool norm = !CD && a.n_state != nullptr && blockIdx.z == 0 && tid < 64;   // wave-uniform
   float* nst = norm ? a.n_state + ((int64_t)r.state_slots[s] * H + h) * d : nullptr;
   float nv[RP];
 #pragma unroll
   for (int i = 0; i < RP; ++i) nv[i] = (norm && !fresh && tid + 64 * i < d) ? nst[tid + 64 * i] : 0.f;
-  for (int t0 = 0; t0 < L; t0 += TB) {
-    const int nb = min(TB, L - t0);
-    __syncthreads();
-    for (int e = tid; e < nb * DPAD; e += nthr) {
-      const int tt = e / DPAD, c = e % DPAD;
-      const int64_t base = (int64_t)(q0 + t0 + tt) * a.xstride + g * d + c;
-      qs[e] = c < d ? ldt<F32>(a.x, base + a.qoff) * a.qscale : 0.f;
-      ks[e] = c < d ? ldt<F32>(a.x, base + a.koff) : 0.f;
-      if (CD) {
-        // sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau)
-        const float z = c < d ? ldt<F32>(a.z, (int64_t)(q0 + t0 + tt) * a.zstride + h * d + c) + a.z_bias[h * d + c] : 0.f;
-        as[e] = c < d ? expf(-step_size<!F32>(-z) * a.inv_tau) : 0.f;
+
+  // a trip's rows in registers on their way to LDS
+  float4 rq[NE], rk[NE], rz[NE], rv[NV];
+  float2 rab;
+  // (a thread without a row of its own loads the trip's last one and does not store it)
+  auto fetch = [&](int t0) {
+    const int nb = min(TT, L - t0);
+#pragma unroll
+    for (int u = 0; u < NE; ++u) {
+      const int e = tid + u * nthr, tt = e / (DPAD / 4), c = 4 * (e % (DPAD / 4));
+      const int64_t row = q0 + t0 + min(tt, nb - 1), base = row * a.xstride + g * d;
+      rq[u] = ld4z<F32, VEC>(a.x, base + a.qoff, c, d);
+      rk[u] = ld4z<F32, VEC>(a.x, base + a.koff, c, d);
+      if (CD) rz[u] = ld4z<F32, VEC>(a.z, row * a.zstride + h * d, c, d);
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      if (u * LN >= TB) break;   // a trip's values fill at most TB / LN float4s per thread
+      const int e = tid + u * nthr, tt = e / (vcp / 4), c = 4 * (e % (vcp / 4));
+      rv[u] = ld4z<F32, VEC>(a.x, (int64_t)(q0 + t0 + min(tt, nb - 1)) * a.xstride + a.voff + h * dv + v0, c, ncol);
+    }
+    if (!CD) {
+      const float* p = a.ab + ((int64_t)(q0 + t0 + min(tid, nb - 1)) * H + h) * a.abw;
+      rab = make_float2(p[0], p[1]);
+    }
+  };
+  // sigmoid(z)^(1/tau) = exp(-softplus(-z) / tau)
+  float4 zb[NE];
+#pragma unroll
+  for (int u = 0; u < NE; ++u)
+    if (CD) zb[u] = ld4z<true, VEC>(a.z_bias, h * d, 4 * ((tid + u * nthr) % (DPAD / 4)), d);
+  auto decay1 = [&](float z, int c) { return c < d ? exp_of<!F32>(-softplus_of<!F32>(-z) * a.inv_tau) : 0.f; };
+  auto stage = [&](int nb) {
+#pragma unroll
+    for (int u = 0; u < NE; ++u) {
+      const int e = tid + u * nthr, tt = e / (DPAD / 4), c = 4 * (e % (DPAD / 4));
+      if (tt < nb) {
+        *reinterpret_cast<float4*>(qs + tt * DPAD + c) =
+            make_float4(rq[u].x * a.qscale, rq[u].y * a.qscale, rq[u].z * a.qscale, rq[u].w * a.qscale);
+        *reinterpret_cast<float4*>(ks + tt * DPAD + c) = rk[u];
+        if (CD)
+          *reinterpret_cast<float4*>(as + tt * DPAD + c) =
+              make_float4(decay1(rz[u].x + zb[u].x, c), decay1(rz[u].y + zb[u].y, c + 1), decay1(rz[u].z + zb[u].z, c + 2),
+                          decay1(rz[u].w + zb[u].w, c + 3));
       }
     }
-    for (int e = tid; e < nb * VC; e += nthr) {
-      const int tt = e / VC, c = e % VC;
-      vs[e] = c < ncol ? ldt<F32>(a.x, (int64_t)(q0 + t0 + tt) * a.xstride + a.voff + h * dv + v0 + c) : 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      if (u * LN >= TB) break;
+      const int e = tid + u * nthr, tt = e / (vcp / 4), c = 4 * (e % (vcp / 4));
+      if (tt < nb) *reinterpret_cast<float4*>(vs + tt * vcp + c) = rv[u];
     }
-    for (int e = tid; !CD && e < 2 * nb; e += nthr) as[e] = a.ab[((int64_t)(q0 + t0 + (e >> 1)) * H + h) * a.abw + (e & 1)];
+    if (!CD && tid < nb) *reinterpret_cast<float2*>(as + 2 * tid) = rab;
+  };
+
+  fetch(0);
+  float S[M][4][4];   // [m][i][column]
+#pragma unroll
+  for (int m = 0; m < M; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int row = 4 * LN * m + 4 * l + i;
+      float4 v = ld4z<true, VEC>(st, (int64_t)min(row, d - 1) * dv, j0, ncol);
+      if (fresh || row >= d) v = make_float4(0.f, 0.f, 0.f, 0.f);   // (a new sequence reads its slot but not its content)
+      S[m][i][0] = v.x, S[m][i][1] = v.y, S[m][i][2] = v.z, S[m][i][3] = v.w;
+    }
+  for (int t0 = 0; t0 < L; t0 += TT) {
+    const int nb = min(TT, L - t0);
+    if (t0 > 0) __syncthreads();   // every wave is done with the previous trip
+    stage(nb);
     __syncthreads();
+    if (t0 + TT < L) fetch(t0 + TT);
     for (int tt = 0; tt < nb; ++tt) {
-      const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD + part * DP);
-      const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD + part * DP);
-      const float4* at = reinterpret_cast<const float4*>(as + tt * DPAD + part * DP);
-      float vj = j < ncol ? vs[tt * VC + j] : 0.f, dec = 1.0f;
+      const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD) + l;
+      const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD) + l;
+      const float4* at = reinterpret_cast<const float4*>(as + tt * DPAD) + l;
+      const float4 v4 = live ? *reinterpret_cast<const float4*>(vs + tt * vcp + j0) : make_float4(0.f, 0.f, 0.f, 0.f);
+      float vj[4] = {v4.x, v4.y, v4.z, v4.w}, dec = 1.0f, o[4] = {0.f, 0.f, 0.f, 0.f};
       if (!CD) {
         const float2 ab = *reinterpret_cast<const float2*>(as + 2 * tt);
-        vj *= ab.y;
+#pragma unroll
+        for (int c = 0; c < 4; ++c) vj[c] *= ab.y;
         dec = ab.x;
       }
-      float o0 = 0.f, o1 = 0.f;
 #pragma unroll
-      for (int i = 0; i < DP / 4; ++i) {
-        const float4 k4 = kt[i], q4 = qt[i], a4 = CD ? at[i] : make_float4(dec, dec, dec, dec);
-        S[4 * i] = S[4 * i] * a4.x + k4.x * vj;
-        S[4 * i + 1] = S[4 * i + 1] * a4.y + k4.y * vj;
-        S[4 * i + 2] = S[4 * i + 2] * a4.z + k4.z * vj;
-        S[4 * i + 3] = S[4 * i + 3] * a4.w + k4.w * vj;
-        o0 += S[4 * i] * q4.x + S[4 * i + 2] * q4.z;
-        o1 += S[4 * i + 1] * q4.y + S[4 * i + 3] * q4.w;
+      for (int m = 0; m < M; ++m) {
+        const float4 k4 = kt[LN * m], q4 = qt[LN * m], a4 = CD ? at[LN * m] : make_float4(dec, dec, dec, dec);
+        const float kk[4] = {k4.x, k4.y, k4.z, k4.w}, qq[4] = {q4.x, q4.y, q4.z, q4.w}, aa[4] = {a4.x, a4.y, a4.z, a4.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) {
+            S[m][i][c] = S[m][i][c] * aa[i] + kk[i] * vj[c];
+            o[c] += S[m][i][c] * qq[i];
+          }
       }
-      float o = o0 + o1;
-      o += __shfl_xor(o, 1, 64);
-      o += __shfl_xor(o, 2, 64);
-      if (part == 0 && j < ncol) a.out[((int64_t)(q0 + t0 + tt) * H + h) * dv + v0 + j] = o;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) o[c] = group_sum<LN>(o[c]);
+      if (l == 0 && live) {
+        float* op = a.out + ((int64_t)(q0 + t0 + tt) * H + h) * dv + v0 + j0;
+        if constexpr (VEC) {
+          *reinterpret_cast<float4*>(op) = make_float4(o[0], o[1], o[2], o[3]);
+        } else {
+#pragma unroll
+          for (int c = 0; c < 4; ++c)
+            if (j0 + c < ncol) op[c] = o[c];
+        }
+      }
     }
     if (norm) {
       float p[TB];
@@ -515,12 +589,22 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
       }
     }
   }
-  if (j < ncol) {
+  if (live) {
 #pragma unroll
-    for (int i = 0; i < DP; ++i) {
-      const int row = part * DP + i;
-      if (row < d) st[(int64_t)row * dv] = S[i];
-    }
+    for (int m = 0; m < M; ++m)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int row = 4 * LN * m + 4 * l + i;
+        if (row >= d) continue;
+        float* p = st + (int64_t)row * dv + j0;
+        if constexpr (VEC) {
+          *reinterpret_cast<float4*>(p) = make_float4(S[m][i][0], S[m][i][1], S[m][i][2], S[m][i][3]);
+        } else {
+#pragma unroll
+          for (int c = 0; c < 4; ++c)
+            if (j0 + c < ncol) p[c] = S[m][i][c];
+        }
+      }
   }
   if (norm) {
 #pragma unroll
@@ -529,23 +613,35 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
   }
 }
 
-template <int DP, bool F32, bool CD> hipError_t launch_gla_one(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
+template <int LN, int M, bool F32, bool CD, bool VEC> hipError_t launch_gla_one(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
   const int VC = a.vdim < 128 ? a.vdim : 128;
-  const int nvc = (a.vdim + VC - 1) / VC;
-  const int threads = (4 * VC + 63) / 64 * 64;
-  const size_t smem = (size_t)((CD ? 3 : 2) * TB * 4 * DP + (TB * VC + 3) / 4 * 4 + 2 * TB) * sizeof(float);
+  const int nvc = (a.vdim + VC - 1) / VC, groups = (VC + 3) / 4;
+  const int threads = (LN * groups + 63) / 64 * 64;
+  // tokens per trip: what two float4s of q and k per thread can hold
+  int tt = 2 * threads / (LN * M);
+  tt = tt > TB ? TB : tt;
+  const size_t smem = (size_t)((CD ? 3 : 2) * TB * 4 * LN * M + TB * 4 * groups + 2 * TB) * sizeof(float);
+  auto* fn = gated_linear_attn_kernel<LN, M, F32, CD, VEC>;
   if (smem > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gated_linear_attn_kernel<DP, F32, CD>),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     if (e != hipSuccess) return e;
   }
-  hipLaunchKernelGGL((gated_linear_attn_kernel<DP, F32, CD>), dim3(a.heads, r.num_seqs, nvc), dim3(threads), smem, s, a,
-                     r, VC);
+  hipLaunchKernelGGL(fn, dim3(a.heads, r.num_seqs, nvc), dim3(threads), smem, s, a, r, VC, tt);
   return hipGetLastError();
 }
-template <int DP> hipError_t launch_gla_dp(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
-  if (a.z != nullptr) return a.f32 ? launch_gla_one<DP, true, true>(a, r, s) : launch_gla_one<DP, false, true>(a, r, s);
-  return a.f32 ? launch_gla_one<DP, true, false>(a, r, s) : launch_gla_one<DP, false, false>(a, r, s);
+template <int LN, int M> hipError_t launch_gla_dp(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
+  auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = a.dim % 4 == 0 && a.vdim % 4 == 0 && a.xstride % 4 == 0 && a.qoff % 4 == 0 && a.koff % 4 == 0 &&
+                   a.voff % 4 == 0 && a16(a.x) && a16(a.state) && a16(a.out) && a16(a.z_bias) &&
+                   (a.z == nullptr || (a.zstride % 4 == 0 && a16(a.z)));
+  if (a.f32) {
+    if (a.z != nullptr)
+      return vec ? launch_gla_one<LN, M, true, true, true>(a, r, s) : launch_gla_one<LN, M, true, true, false>(a, r, s);
+    return vec ? launch_gla_one<LN, M, true, false, true>(a, r, s) : launch_gla_one<LN, M, true, false, false>(a, r, s);
+  }
+  if (a.z != nullptr)
+    return vec ? launch_gla_one<LN, M, false, true, true>(a, r, s) : launch_gla_one<LN, M, false, true, false>(a, r, s);
+  return vec ? launch_gla_one<LN, M, false, false, true>(a, r, s) : launch_gla_one<LN, M, false, false, false>(a, r, s);
 }
 
 // ------------------------------------------------------------------------------------------------ epilogues
@@ -797,11 +893,12 @@ hipError_t launch_gated_linear_attn(const GatedLinearArgs& a, RaggedRows r, hipS
       (a.z == nullptr && (a.ab == nullptr || a.abw < 2)) || (a.n_state != nullptr) != (a.nq != nullptr) ||
       (a.z != nullptr && (a.z_bias == nullptr || a.n_state != nullptr)))
     return hipErrorInvalidValue;
-  if (a.dim <= 16) return launch_gla_dp<4>(a, r, s);
-  if (a.dim <= 32) return launch_gla_dp<8>(a, r, s);
-  if (a.dim <= 64) return launch_gla_dp<16>(a, r, s);
-  if (a.dim <= 128) return launch_gla_dp<32>(a, r, s);
-  return launch_gla_dp<64>(a, r, s);
+  if (a.dim <= 16) return launch_gla_dp<4, 1>(a, r, s);
+  if (a.dim <= 32) return launch_gla_dp<8, 1>(a, r, s);
+  if (a.dim <= 64) return launch_gla_dp<16, 1>(a, r, s);
+  if (a.dim <= 128) return launch_gla_dp<16, 2>(a, r, s);
+  if (a.dim <= 192) return launch_gla_dp<16, 3>(a, r, s);
+  return launch_gla_dp<16, 4>(a, r, s);
 }
 
 hipError_t launch_head_norm_gate(const HeadNormGateArgs& a, hipStream_t s) {

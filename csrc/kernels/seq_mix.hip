@@ -8,11 +8,12 @@
 //   poly_norm_act       c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3
 //   delta_prep          short conv + SiLU of q/k/v, unit q/k, beta (and the per-head decay) of the gated delta rule
 //   conv_state_update   the convolution's trailing inputs -> state
-//   gated_delta         the recurrence itself, one workgroup per (sequence, head), the state in registers (a
-//                       column per lane quad)
+//   gated_delta         the recurrence itself, one workgroup per (sequence, head), the state in registers (four
+//                       columns per group of 4 - 16 lanes)
 //   qkv_prep            projection bias or short conv, q/k norm, rotate-half rotary (optionally of the values too),
 //                       value norm / value mixing, paged cache write
 #include "common.h"
+#include "lane_reduce.h"
 #include "seq_launchers.h"
 
 namespace die {
@@ -32,7 +33,6 @@ __device__ __forceinline__ void stv(void* p, int64_t i, bool f32, float v) {
 __device__ __forceinline__ float rnd(float v, bool f32) { return f32 ? v : bf2f(f2bf(v)); }
 __device__ __forceinline__ float siluf(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 constexpr int NT = 256;
 
@@ -472,131 +472,191 @@ __global__ void __launch_bounds__(NT) conv_state_update_kernel(float* conv_state
   }
 }
 
-constexpr int TB = 16;  // tokens staged per trip
+constexpr int TB = 16;  // tokens staged per trip, at most
 
-// One workgroup per (sequence, head). The state S [dim, vdim] lives in registers for the whole step: column j is
-// split over the 4 lanes of a quad, lane `part` holding rows [part * DP, (part + 1) * DP) — so a token costs each
-// lane 3 * DP multiply-adds and two quad reductions (S^T k and S^T q), with q and k read from LDS as float4
-// broadcasts, and 4 * vdim lanes work on one head. Tokens are staged TB at a time; the read-outs of a trip are
-// normed and gated afterwards, one wave per token. CD: a decay per key channel, computed while a trip is staged.
-template <int DP, bool CD>
-__global__ void __launch_bounds__(1024) gated_delta_kernel(GatedDeltaArgs a, RaggedRows r) {
+// 4 consecutive values at p[i + c] of a row piece of n values (c a multiple of 4), zeros beyond it. VEC (n and the row's
+// start multiples of 4, the base aligned): one 8- / 16-byte load without a branch around it, so that a run of these stays
+// in flight together.
+template <bool F32, bool VEC> __device__ __forceinline__ float4 ld4z(const void* p, int64_t i, int c, int n) {
+  if constexpr (VEC) {
+    const float4 v = ld4(p, i + (c < n ? c : 0), F32);
+    return c < n ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+  } else {
+    float f[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f[e] = c + e < n ? ldv(p, i + c + e, F32) : 0.f;
+    return make_float4(f[0], f[1], f[2], f[3]);
+  }
+}
+
+// One workgroup per (sequence, head). The state S [dim, vdim] lives in registers for the whole step: a group of LN lanes
+// holds 4 columns, lane l of it the rows 4 LN m + 4 l + i (m < M, i < 4) — 16 M values per lane, LN M 4 >= dim. A token
+// costs a lane 4 multiply-adds per value and two sums over its group (S^T k and S^T q, on DPP adds); k, q (and with CD
+// the decays) are read from LDS as consecutive float4s, one read per 16 values of the state. Up to TB tokens are staged
+// per trip, the next trip's rows are already in flight; the read-outs of a trip are normed and gated afterwards, one wave
+// per token. CD: a decay per key channel, computed while a trip is staged. VEC: dim, vdim and the row strides are multiples
+// of 4.
+template <int LN, int M, bool F32, bool CD, bool VEC>
+__global__ void __launch_bounds__(1024) gated_delta_kernel(GatedDeltaArgs a, RaggedRows r, int TT) {
   const DeltaShape& sh = a.sh;
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  constexpr int DPAD = 4 * DP;
+  constexpr int DPAD = 4 * LN * M, NE = 2, NV = 4;
   const int d = sh.dim, dv = sh.vdim, H = sh.heads, G = sh.kv_heads, C = sh.channels();
+  const int dvp = (dv + 3) & ~3;
   float* qs = sm;                  // [TB][DPAD], zero beyond dim
   float* ks = qs + TB * DPAD;      // [TB][DPAD]
-  float* vs = ks + TB * DPAD;      // [TB][dv]
-  float* os = vs + TB * dv;        // [TB][dv]
-  float* bs = os + TB * dv;        // [TB] beta
-  float* gs = bs + TB;             // [TB] decay, or [TB][DPAD] with CD
-  const int bgw = CD ? H : 2 * H;
+  float* gs = ks + TB * DPAD;      // [TB][DPAD] with CD: decays
+  float* vs = gs + (CD ? TB * DPAD : 0);   // [TB][dvp]
+  float* os = vs + TB * dvp;       // [TB][dvp]
+  float* bs = os + TB * dvp;       // [TB][2]: beta, decay per head
   const int h = blockIdx.x, s = blockIdx.y, tid = threadIdx.x, nthr = blockDim.x;
-  const int j = tid >> 2, part = tid & 3;
+  const int l = tid % LN, j0 = 4 * (tid / LN);
   const int kh = h / (H / G);
   const int q0 = r.cu_q ? r.cu_q[s] : s;
   const int L = r.cu_q ? r.cu_q[s + 1] - q0 : 1;
   if (L <= 0) return;
   const bool fresh = r.positions[q0] <= 0;
+  const bool live = j0 < dv;
   float* st = a.state + ((int64_t)r.state_slots[s] * H + h) * d * dv;
   const float expA = CD ? expf(a.A_log[h]) : 0.f;
-  float S[DP];
+  const int bgw = CD ? H : 2 * H;
+
+  // a trip's rows in registers on their way to LDS
+  float4 rq[NE], rk[NE], rz[NE], rv[NV];
+  float2 rb;
+  // (a thread without a row of its own loads the trip's last one and does not store it)
+  auto fetch = [&](int t0) {
+    const int nb = min(TT, L - t0);
 #pragma unroll
-  for (int i = 0; i < DP; ++i) {
-    const int row = part * DP + i;
-    S[i] = (!fresh && row < d && j < dv) ? st[(int64_t)row * dv + j] : 0.f;
-  }
+    for (int u = 0; u < NE; ++u) {
+      const int e = tid + u * nthr, tt = e / (DPAD / 4), c = 4 * (e % (DPAD / 4));
+      const int64_t row = q0 + t0 + min(tt, nb - 1);
+      rq[u] = ld4z<true, VEC>(a.qkv32, row * C + kh * d, c, d);
+      rk[u] = ld4z<true, VEC>(a.qkv32, row * C + G * d + kh * d, c, d);
+      if (CD) rz[u] = ld4z<F32, VEC>(a.z, row * a.zstride + h * d, c, d);
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      if (u * LN >= TB) break;   // a trip's values fill at most TB / LN float4s per thread
+      const int e = tid + u * nthr, tt = e / (dvp / 4), c = 4 * (e % (dvp / 4));
+      rv[u] = ld4z<true, VEC>(a.qkv32, (int64_t)(q0 + t0 + min(tt, nb - 1)) * C + 2 * G * d + h * dv, c, dv);
+    }
+    const float* b = a.bg + (int64_t)(q0 + t0 + min(tid, nb - 1)) * bgw + h;
+    rb = make_float2(b[0], CD ? 0.f : b[H]);
+  };
+  float4 zb[NE];
+#pragma unroll
+  for (int u = 0; u < NE; ++u)
+    if (CD) zb[u] = ld4z<true, VEC>(a.z_bias, h * d, 4 * ((tid + u * nthr) % (DPAD / 4)), d);
+  auto decay1 = [&](float z, int c) { return c < d ? exp_of<!F32>(-expA * softplus_of<!F32>(z)) : 0.f; };
+  auto stage = [&](int nb) {
+#pragma unroll
+    for (int u = 0; u < NE; ++u) {
+      const int e = tid + u * nthr, tt = e / (DPAD / 4), c = 4 * (e % (DPAD / 4));
+      if (tt < nb) {
+        *reinterpret_cast<float4*>(qs + tt * DPAD + c) = rq[u];
+        *reinterpret_cast<float4*>(ks + tt * DPAD + c) = rk[u];
+        if (CD)
+          *reinterpret_cast<float4*>(gs + tt * DPAD + c) =
+              make_float4(decay1(rz[u].x + zb[u].x, c), decay1(rz[u].y + zb[u].y, c + 1), decay1(rz[u].z + zb[u].z, c + 2),
+                          decay1(rz[u].w + zb[u].w, c + 3));
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      if (u * LN >= TB) break;
+      const int e = tid + u * nthr, tt = e / (dvp / 4), c = 4 * (e % (dvp / 4));
+      if (tt < nb) *reinterpret_cast<float4*>(vs + tt * dvp + c) = rv[u];
+    }
+    if (tid < nb) *reinterpret_cast<float2*>(bs + 2 * tid) = rb;
+  };
+
+  fetch(0);
+  float S[M][4][4];   // [m][i][column]
+#pragma unroll
+  for (int m = 0; m < M; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int row = 4 * LN * m + 4 * l + i;
+      float4 v = ld4z<true, VEC>(st, (int64_t)min(row, d - 1) * dv, j0, dv);
+      if (fresh || row >= d) v = make_float4(0.f, 0.f, 0.f, 0.f);   // (a new sequence reads its slot but not its content)
+      S[m][i][0] = v.x, S[m][i][1] = v.y, S[m][i][2] = v.z, S[m][i][3] = v.w;
+    }
   const int lane = tid & 63, wave = tid >> 6, nwaves = nthr >> 6;
-  for (int t0 = 0; t0 < L; t0 += TB) {
-    const int nb = min(TB, L - t0);
+  for (int t0 = 0; t0 < L; t0 += TT) {
+    const int nb = min(TT, L - t0);
+    stage(nb);
     __syncthreads();
-    for (int e = tid; e < nb * DPAD; e += nthr) {
-      const int tt = e / DPAD, c = e % DPAD;
-      const float* row = a.qkv32 + (int64_t)(q0 + t0 + tt) * C;
-      qs[e] = c < d ? row[kh * d + c] : 0.f;
-      ks[e] = c < d ? row[G * d + kh * d + c] : 0.f;
-      if (CD) {
-        float g = 0.f;
-        if (c < d) {
-          const float z = ldv(a.z, (int64_t)(q0 + t0 + tt) * a.zstride + h * d + c, a.f32) + a.z_bias[h * d + c];
-          g = expf(-expA * softplusf(z));
-        }
-        gs[e] = g;
-      }
-    }
-    for (int e = tid; e < nb * dv; e += nthr) {
-      const int tt = e / dv, c = e % dv;
-      vs[e] = a.qkv32[(int64_t)(q0 + t0 + tt) * C + 2 * G * d + h * dv + c];
-    }
-    if (tid < nb) {
-      bs[tid] = a.bg[(int64_t)(q0 + t0 + tid) * bgw + h];
-      if (!CD) gs[tid] = a.bg[(int64_t)(q0 + t0 + tid) * bgw + H + h];
-    }
-    __syncthreads();
+    if (t0 + TT < L) fetch(t0 + TT);
     for (int tt = 0; tt < nb; ++tt) {
-      const float g = CD ? 1.0f : gs[tt], beta = bs[tt];
-      const float4* gt4 = reinterpret_cast<const float4*>(gs + tt * DPAD + part * DP);
-      const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD + part * DP);
-      const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD + part * DP);
-      float kreg[DP];
-      float d0 = 0.f, d1 = 0.f;
+      const float2 bg = *reinterpret_cast<const float2*>(bs + 2 * tt);
+      const float4 v4 = live ? *reinterpret_cast<const float4*>(vs + tt * dvp + j0) : make_float4(0.f, 0.f, 0.f, 0.f);
+      const float4* kt = reinterpret_cast<const float4*>(ks + tt * DPAD) + l;
+      const float4* qt = reinterpret_cast<const float4*>(qs + tt * DPAD) + l;
+      const float4* gt = reinterpret_cast<const float4*>(gs + tt * DPAD) + l;
+      float kk[M][4], dot[4] = {0.f, 0.f, 0.f, 0.f}, o[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < DP / 4; ++i) {
-        const float4 k4 = kt[i];
-        kreg[4 * i] = k4.x;
-        kreg[4 * i + 1] = k4.y;
-        kreg[4 * i + 2] = k4.z;
-        kreg[4 * i + 3] = k4.w;
-        const float4 g4 = CD ? gt4[i] : make_float4(g, g, g, g);
-        S[4 * i] *= g4.x;
-        S[4 * i + 1] *= g4.y;
-        S[4 * i + 2] *= g4.z;
-        S[4 * i + 3] *= g4.w;
-        d0 += S[4 * i] * k4.x + S[4 * i + 2] * k4.z;
-        d1 += S[4 * i + 1] * k4.y + S[4 * i + 3] * k4.w;
-      }
-      float dot = d0 + d1;
-      dot += __shfl_xor(dot, 1, 64);
-      dot += __shfl_xor(dot, 2, 64);
-      const float u = beta * ((j < dv ? vs[tt * dv + j] : 0.f) - dot);
-      float o0 = 0.f, o1 = 0.f;
+      for (int m = 0; m < M; ++m) {
+        const float4 k4 = kt[LN * m], g4 = CD ? gt[LN * m] : make_float4(bg.y, bg.y, bg.y, bg.y);
+        const float gg[4] = {g4.x, g4.y, g4.z, g4.w};
+        kk[m][0] = k4.x, kk[m][1] = k4.y, kk[m][2] = k4.z, kk[m][3] = k4.w;
 #pragma unroll
-      for (int i = 0; i < DP / 4; ++i) {
-        const float4 q4 = qt[i];
-        S[4 * i] += kreg[4 * i] * u;
-        S[4 * i + 1] += kreg[4 * i + 1] * u;
-        S[4 * i + 2] += kreg[4 * i + 2] * u;
-        S[4 * i + 3] += kreg[4 * i + 3] * u;
-        o0 += S[4 * i] * q4.x + S[4 * i + 2] * q4.z;
-        o1 += S[4 * i + 1] * q4.y + S[4 * i + 3] * q4.w;
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) {
+            S[m][i][c] *= gg[i];
+            dot[c] += S[m][i][c] * kk[m][i];
+          }
       }
-      float o = o0 + o1;
-      o += __shfl_xor(o, 1, 64);
-      o += __shfl_xor(o, 2, 64);
-      if (part == 0 && j < dv) os[tt * dv + j] = o;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) dot[c] = group_sum<LN>(dot[c]);
+      const float u[4] = {bg.x * (v4.x - dot[0]), bg.x * (v4.y - dot[1]), bg.x * (v4.z - dot[2]), bg.x * (v4.w - dot[3])};
+#pragma unroll
+      for (int m = 0; m < M; ++m) {
+        const float4 q4 = qt[LN * m];
+        const float qq[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) {
+            S[m][i][c] += kk[m][i] * u[c];
+            o[c] += S[m][i][c] * qq[i];
+          }
+      }
+#pragma unroll
+      for (int c = 0; c < 4; ++c) o[c] = group_sum<LN>(o[c]);
+      if (l == 0 && live) *reinterpret_cast<float4*>(os + tt * dvp + j0) = make_float4(o[0], o[1], o[2], o[3]);
     }
     __syncthreads();
     for (int tt = wave; tt < nb; tt += nwaves) {
       float ss = 0.f;
-      for (int c = lane; c < dv; c += 64) ss += os[tt * dv + c] * os[tt * dv + c];
+      for (int c = lane; c < dv; c += 64) ss += os[tt * dvp + c] * os[tt * dvp + c];
       ss = wave_sum(ss);
       const float rs = a.mult / sqrtf(ss / (float)dv + a.eps);
       const int64_t row = q0 + t0 + tt;
       for (int c = lane; c < dv; c += 64) {
-        const float gt = ldv(a.gate, row * a.gstride + h * dv + c, a.f32);
-        stv(a.out, row * a.ostride + h * dv + c, a.f32,
-            os[tt * dv + c] * rs * a.norm_w[c] * (a.gate_sigmoid ? sigmoidf(gt) : siluf(gt)));
+        const float gt = ldv(a.gate, row * a.gstride + h * dv + c, F32);
+        stv(a.out, row * a.ostride + h * dv + c, F32,
+            os[tt * dvp + c] * rs * a.norm_w[c] * (a.gate_sigmoid ? sigmoidf(gt) : siluf(gt)));
       }
     }
   }
-  if (j < dv) {
+  if (!live) return;
 #pragma unroll
-    for (int i = 0; i < DP; ++i) {
-      const int row = part * DP + i;
-      if (row < d) st[(int64_t)row * dv + j] = S[i];
+  for (int m = 0; m < M; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int row = 4 * LN * m + 4 * l + i;
+      if (row >= d) continue;
+      float* p = st + (int64_t)row * dv + j0;
+      if constexpr (VEC) {
+        *reinterpret_cast<float4*>(p) = make_float4(S[m][i][0], S[m][i][1], S[m][i][2], S[m][i][3]);
+      } else {
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+          if (j0 + c < dv) p[c] = S[m][i][c];
+      }
     }
-  }
 }
 
 // --------------------------------------------------------------------------------------------------- qkv prep
@@ -890,31 +950,45 @@ hipError_t launch_conv_state_update(float* conv_state, const void* x, int64_t xs
   return hipGetLastError();
 }
 
-template <int DP, bool CD> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
-  const int nthr = (4 * a.sh.vdim + 63) / 64 * 64;
-  const size_t lds = sizeof(float) * (TB * ((CD ? 3 : 2) * 4 * DP + 2 * a.sh.vdim) + 2 * TB);
+template <int LN, int M, bool F32, bool CD, bool VEC> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+  const int groups = (a.sh.vdim + 3) / 4;
+  const int nthr = (LN * groups + 63) / 64 * 64;
+  // tokens per trip: what two float4s of q and k per thread can hold
+  int tt = 2 * nthr / (LN * M);
+  tt = tt > TB ? TB : tt;
+  const size_t lds = sizeof(float) * (TB * ((CD ? 3 : 2) * 4 * LN * M + 2 * 4 * groups) + 2 * TB);
+  auto* fn = gated_delta_kernel<LN, M, F32, CD, VEC>;
   if (lds > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gated_delta_kernel<DP, CD>),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
   }
-  hipLaunchKernelGGL((gated_delta_kernel<DP, CD>), dim3(a.sh.heads, r.num_seqs), dim3(nthr), lds, s, a, r);
+  hipLaunchKernelGGL(fn, dim3(a.sh.heads, r.num_seqs), dim3(nthr), lds, s, a, r, tt);
   return hipGetLastError();
 }
-template <int DP> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
-  return a.z != nullptr ? launch_gd<DP, true>(a, r, s) : launch_gd<DP, false>(a, r, s);
+template <int LN, int M> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+  auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = a.sh.dim % 4 == 0 && a.sh.vdim % 4 == 0 && a16(a.qkv32) && a16(a.state) && a16(a.z_bias) &&
+                   (a.z == nullptr || (a.zstride % 4 == 0 && a16(a.z)));
+  if (a.f32) {
+    if (a.z != nullptr)
+      return vec ? launch_gd<LN, M, true, true, true>(a, r, s) : launch_gd<LN, M, true, true, false>(a, r, s);
+    return vec ? launch_gd<LN, M, true, false, true>(a, r, s) : launch_gd<LN, M, true, false, false>(a, r, s);
+  }
+  if (a.z != nullptr)
+    return vec ? launch_gd<LN, M, false, true, true>(a, r, s) : launch_gd<LN, M, false, true, false>(a, r, s);
+  return vec ? launch_gd<LN, M, false, false, true>(a, r, s) : launch_gd<LN, M, false, false, false>(a, r, s);
 }
 
 hipError_t launch_gated_delta(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
   if (r.num_seqs == 0 || r.total_rows == 0) return hipSuccess;
   if (!delta_ok(a.sh) || !rows_ok(r) || (a.z != nullptr && (a.z_bias == nullptr || a.A_log == nullptr)))
     return hipErrorInvalidValue;
-  // rows of the state per lane of a quad: dim / 4, rounded up to a multiple of 4
-  if (a.sh.dim <= 16) return launch_gd<4>(a, r, s);
-  if (a.sh.dim <= 32) return launch_gd<8>(a, r, s);
-  if (a.sh.dim <= 64) return launch_gd<16>(a, r, s);
-  if (a.sh.dim <= 128) return launch_gd<32>(a, r, s);
-  return launch_gd<64>(a, r, s);
+  if (a.sh.dim <= 16) return launch_gd<4, 1>(a, r, s);
+  if (a.sh.dim <= 32) return launch_gd<8, 1>(a, r, s);
+  if (a.sh.dim <= 64) return launch_gd<16, 1>(a, r, s);
+  if (a.sh.dim <= 128) return launch_gd<16, 2>(a, r, s);
+  if (a.sh.dim <= 192) return launch_gd<16, 3>(a, r, s);
+  return launch_gd<16, 4>(a, r, s);
 }
 
 hipError_t launch_qkv_prep(const QkvPrepArgs& a, hipStream_t s) {

@@ -410,7 +410,7 @@ class ScaledPairMixer:
         conv.rot_head_gate(o, p[:, self.gate_at: self.gate_at + s.left.heads], s.left.heads, s.left.vdim, s.left_scale,
                            positions, l.v_inv_freq, out=u[:, :nl])
         self.right.recur(p, self.at, low, eps, state, rag, s.right_scale, u[:, nl:])
-        return mix.linear(u, self.w_o)
+        return mix.linear_partials(u, self.w_o)
 
 
 class LinearPairMixer(ScaledPairMixer):
@@ -612,7 +612,7 @@ class RerozenLM:
                 meta.kv_hook(li)
             if lw.up is not None:
                 h = boundary(lw.norm2, lw.canon2, st[li]["canon2"])
-                y = mix.linear(mix.gelu_act(mix.linear(h, lw.up)), lw.down)
+                y = mix.linear_partials(mix.gelu_act(mix.linear(h, lw.up)), lw.down)
         h = boundary(self.norm_out)
         if layer_hook is not None:
             layer_hook(len(self.layers) - 1, x)

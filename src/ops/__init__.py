@@ -669,6 +669,19 @@ def _bucket(m: int) -> int:
     return 32 if m <= 32 else (64 if m <= 64 else 128)
 
 
+def split_k_tile(x: torch.Tensor, w: torch.Tensor):
+    """(wr, kc, sk) of the slab decode GEMM (mode 2) for x @ w^T where splitting K fills the chip better than full-K
+    tiles; None where it does not apply."""
+    n, k = w.shape
+    if not _decode_gemm_ok(x, w) or n % 32 or n > DECODE_GEMM_MAX_N:
+        return None
+    try:
+        wr, kc, sk = decode_tile(n, k, 2, _bucket(x.shape[0]))
+    except ValueError:
+        return None
+    return (wr, kc, sk) if sk > 1 and gd_tile_valid(wr, kc, _bucket(x.shape[0])) else None
+
+
 def linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y = x @ w^T. Decode-sized M (<= 128 rows) runs on the weight-streaming
     gfx950 kernel (gemm_decode.hip); larger M goes to hipBLASLt."""

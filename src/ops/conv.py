@@ -29,7 +29,7 @@ def conv_norm(resid: torch.Tensor, y: Optional[torch.Tensor], w: torch.Tensor, e
     """(x, h): x = resid + y (fp32 [T, W]; ``resid`` itself without y), n = rms(x) * w and
     h[t] = n[t] + sum_j conv_wt[j] * n[t - (taps - 1) + j] in ``out_dtype`` — over the row's own sequence, the rows
     before the step from conv_state [slots, taps - 1, W] (fp32, the most recent last), zeros before the sequence's start;
-    without ``conv_wt`` h = n. conv_state takes the sequence's last taps - 1 rows of n. ``max_q``: most rows of one
+    without ``conv_wt`` h = n. ``y`` may be fp32 partial sums [n, T, W] (:func:`src.ops.mix.linear_partials`). conv_state takes the sequence's last taps - 1 rows of n. ``max_q``: most rows of one
     sequence in the step. x is written in place where no other row of the step reads the row, else into ``spare``
     (a buffer like ``resid``, or a new one); the one not returned is free afterwards."""
     T, W = resid.shape
@@ -44,7 +44,7 @@ def conv_norm(resid: torch.Tensor, y: Optional[torch.Tensor], w: torch.Tensor, e
             _kern().conv_norm(h, resid, x, y, w, float(eps), conv_wt, conv_state, max_q, rag.positions, rag.cu_q,
                               rag.state_slots)
         return x, h
-    x = resid if y is None else resid + y.float()
+    x = resid if y is None else resid + (y.sum(0) if y.dim() == 3 else y.float())
     n = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w
     if conv_wt is None:
         return x, n.to(out_dtype)

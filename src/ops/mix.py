@@ -140,6 +140,21 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return F.linear(x, w)
 
 
+def linear_partials(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w^T for a consumer that sums partial products itself: bf16 steps of up to 128 rows split K over workgroups where
+    full-K tiles would leave most CUs idle and return fp32 partial sums [n, T, N]; everything else is :func:`linear`'s
+    [T, N]."""
+    if x.is_cuda and x.dtype == torch.bfloat16 and 0 < x.shape[0] <= 128 and x.is_contiguous():
+        from src import ops
+
+        if ops.native_available():
+            tile = ops.split_k_tile(x, w)
+            if tile is not None:
+                wr, kc, sk = tile
+                return ops.gemm_decode(x, w, 2, wr, sk, kc=kc)
+    return linear(x, w)
+
+
 # (token, expert) rows up to which the experts' weights are gathered per row for two batched GEMMs (no host
 # read, hipGraph-capturable: decode steps); above it each expert runs one library GEMM pair over its rows
 MOE_BMM_MAX_ROWS = 64

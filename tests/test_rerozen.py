@@ -186,7 +186,7 @@ LENS = (81, 14)
 
 # ---------------------------------------------------------------------------------------------- mechanisms alone
 @pytest.mark.parametrize("device", DEVICES)
-@pytest.mark.parametrize("W,taps", [(48, 3), (30, 2), (1032, 4), (24, 1), (40, 7), (2100, 3)])
+@pytest.mark.parametrize("W,taps", [(48, 3), (30, 2), (1032, 4), (24, 1), (40, 7), (2100, 3), (4200, 2), (8200, 3), (1500, 5)])
 def test_input_convolution_with_norm_and_residual(device, W, taps):
     """conv_norm: two sequences in shared steps (portions down to one token and longer than a workgroup's tile), in slots
     that hold stale rows; the residual takes the sublayer's output, the convolution runs over the normed rows of earlier
@@ -224,6 +224,17 @@ def test_input_convolution_with_norm_and_residual(device, W, taps):
             assert float(state[1].min()) == 7.0 and float(state[3].max()) == 7.0    # other slots untouched
             keep = (orc.rms(sums[0], eps) * w.to(F64))[-(taps - 1):]
             assert torch.allclose(state[2].cpu().double(), keep, atol=1e-5)
+        # the sublayer's output as fp32 partial sums, as a split product leaves it; one row per sequence
+        if dt == torch.float32:
+            parts = torch.randn(3, 2, W, generator=g)
+            x2 = torch.stack([xs[0][0], xs[1][0]])
+            state.fill_(7.0)
+            new, h = conv.conv_norm(x2.to(device), parts.to(device), w.to(device), eps, dt, cw.t().contiguous().to(device), state,
+                                    _rag(device, [0, 0], None, [3, 1]), 1)
+            ref = x2.to(F64) + parts.to(F64).sum(0)
+            assert float((new.cpu().double() - ref).abs().max()) < 1e-5
+            want2 = orc.rms(ref, eps) * w.to(F64) * (1.0 + cw[:, -1].to(F64))
+            assert torch.allclose(h.cpu().double(), want2, atol=tol, rtol=tol)
         # no convolution, no sublayer output: the plain norm
         x = xs[0].to(device)
         same, h = conv.conv_norm(x, None, w.to(device), eps, dt)
