@@ -5,6 +5,7 @@
 #include <c10/hip/HIPStream.h>
 #include <torch/extension.h>
 
+#include "kernels/conv_launchers.h"
 #include "kernels/seq_launchers.h"
 
 using at::Tensor;
@@ -356,14 +357,21 @@ void qkv_prep(Tensor q_out, Tensor cache, Tensor q, Tensor k, OptTensor v, int64
 void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTensor cu_q, Tensor ctx_lens,
                Tensor positions, OptTensor sink, OptTensor bias, int64_t max_q, int64_t heads, int64_t kv_heads,
                int64_t dim, int64_t vdim, int64_t window, double scale, int64_t impl, double softcap,
-               OptTensor slopes, int64_t seg) {
+               OptTensor slopes, int64_t seg, OptTensor gate, OptTensor out_inv_freq, double gate_mult) {
   die::SinkAttnArgs a;
   a.f32 = is_f32(q, "q");
   TORCH_CHECK(is_f32(out, "out") == a.f32 && is_f32(cache, "cache") == a.f32, "one dtype");
   TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && q.size(1) == heads * dim, "q [T, H * dim] contiguous");
   const int64_t T = q.size(0);
-  TORCH_CHECK(out.is_contiguous() && out.numel() == T * heads * vdim, "out [T, H * vdim] contiguous");
+  check_rows(out, "out");
+  TORCH_CHECK(out.size(0) == T && out.size(1) == heads * vdim && (gate.has_value() || out.is_contiguous()),
+              "out [T, H * vdim], contiguous without a gate");
   TORCH_CHECK(heads >= 1 && kv_heads >= 1 && heads % kv_heads == 0, "heads % kv_heads == 0");
+  if (gate.has_value()) {
+    check_rows(*gate, "gate");
+    TORCH_CHECK(is_f32(*gate, "gate") == a.f32 && gate->size(0) == T && gate->size(1) == heads, "gate [T, H] in q's dtype");
+  }
+  TORCH_CHECK(!out_inv_freq.has_value() || (gate.has_value() && vdim % 2 == 0), "turned outputs: with a gate, an even vdim");
   TORCH_CHECK(cache.dim() == 3 && cache.is_contiguous() && cache.size(2) == kv_heads * (dim + vdim), "cache layout");
   check_c(ctx_lens, at::kInt, "ctx_lens");
   check_c(positions, at::kLong, "positions");
@@ -447,7 +455,41 @@ void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTenso
       a.nsplit = 1;
     }
   }
+  a.gate = nullptr;
+  a.gstride = 0;
+  a.out_inv_freq = nullptr;
+  a.gate_mult = (float)gate_mult;
+  a.ostride = out.stride(0);
+  if (!gate.has_value()) {
+    HIP_OK(die::launch_sink_attn(a, cur_stream()));
+    return;
+  }
+  if (die::sink_attn_fuses_gate(a)) {
+    a.gate = gate->data_ptr();
+    a.gstride = gate->stride(0);
+    a.out_inv_freq = f32_ptr(out_inv_freq, vdim / 2, "out_inv_freq");
+    HIP_OK(die::launch_sink_attn(a, cur_stream()));
+    return;
+  }
+  // the other forms write plain rows; the gate is a launch of its own
+  Tensor raw = at::empty({T, heads * vdim}, q.options());
+  a.out = raw.data_ptr();
+  a.ostride = heads * vdim;
   HIP_OK(die::launch_sink_attn(a, cur_stream()));
+  die::RotHeadGateArgs g;
+  g.out = out.data_ptr();
+  g.ostride = out.stride(0);
+  g.o = raw.data_ptr();
+  g.g = gate->data_ptr();
+  g.gstride = gate->stride(0);
+  g.f32 = a.f32;
+  g.positions = a.positions;
+  g.inv_freq = f32_ptr(out_inv_freq, vdim / 2, "out_inv_freq");
+  g.mult = (float)gate_mult;
+  g.T = (int)T;
+  g.heads = (int)heads;
+  g.vdim = (int)vdim;
+  HIP_OK(die::launch_rot_head_gate(g, cur_stream()));
 }
 
 }  // namespace

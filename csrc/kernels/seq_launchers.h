@@ -162,11 +162,21 @@ struct SinkAttnArgs {
   float* ws_o;
   float* ws_ml;
   int nsplit, chunk;
+  // epilogue of the decode-step and the split-key forms (sink_attn_fuses_gate): with gate [T, H] (bf16, row stride gstride)
+  // head h's output, turned by -positions[t] * out_inv_freq[i] over pairs (i, i + vdim / 2) if out_inv_freq is given, times
+  // gate_mult * sigmoid(gate[t, h]). These forms write rows of stride ostride; the others contiguous rows and no gate.
+  const void* gate;
+  int64_t gstride;
+  const float* out_inv_freq;
+  float gate_mult;
+  int64_t ostride;
 };
 hipError_t launch_sink_attn(const SinkAttnArgs& a, hipStream_t s);
 bool sink_attn_uses_mfma(const SinkAttnArgs& a);
 // whether launch_sink_attn would run the decode-step kernel (impl 0, one bf16 query token per sequence); it splits
 // the keys in multiples of 128
 bool sink_attn_uses_decode(const SinkAttnArgs& a);
+// whether launch_sink_attn would apply the gate epilogue (nsplit already chosen)
+bool sink_attn_fuses_gate(const SinkAttnArgs& a);
 
 }  // namespace die

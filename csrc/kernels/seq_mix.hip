@@ -56,6 +56,10 @@ __device__ __forceinline__ void st4(void* p, int64_t i, bool f32, float4 v, floa
   }
 }
 
+// n / d for 0 <= n < 2^21 with inv = 1.0f / d: the nearest a quotient comes to the next integer, 0.5 / d, is far above the
+// rounding of the product
+__device__ __forceinline__ int qdiv(int n, float inv) { return (int)(((float)n + 0.5f) * inv); }
+
 // sequence of a row: the largest s with cu_q[s] <= row (cu_q == nullptr: the row itself)
 __device__ __forceinline__ int seq_of_row(const int* cu_q, int num_seqs, int row) {
   if (cu_q == nullptr) return row;
@@ -316,29 +320,20 @@ __global__ void __launch_bounds__(NT) poly_norm_act_kernel(void* out, const void
 // ------------------------------------------------------------------------------------------ gated delta rule
 constexpr int TAPS_MAX = 16;
 
-// A row of a short causal convolution over the sequence: row `row` of x is row i of its sequence in this step, at
-// position p; inputs before the step come from st [taps - 1, C] (the most recent last), inputs before the sequence's
-// start are zero. 8 channels (bf16 rows, tap-major weights, 16-byte loads):
-__device__ __forceinline__ void conv8(float* acc, const bf16_t* x, int64_t row, int64_t xstride, int c8, const float* st,
-                                      const float* wt, int taps, int C, int i, int64_t p) {
+// A short causal convolution over each row's own sequence. Row `row` of x is row i of its sequence in this step, at position
+// p; inputs before the step come from st [taps - 1, C] (the most recent last), inputs before the sequence's start are
+// zero. The channels 8 c8 .. 8 c8 + 7 of the input `back` rows ago (bf16 rows, 16-byte loads):
+__device__ __forceinline__ void conv_in8(float* xv, const bf16_t* x, int64_t row, int64_t xstride, int c8, const float* st,
+                                         int taps, int C, int i, int64_t p, int back) {
+  if (p - back < 0) {
 #pragma unroll
-  for (int e = 0; e < 8; ++e) acc[e] = 0.f;
-  for (int j = 0; j < taps; ++j) {
-    const int back = taps - 1 - j;
-    if (p - back < 0) continue;
-    const int src = i - back;
-    float xv[8];
-    if (src >= 0) {
-      unpack8(*reinterpret_cast<const uint4*>(x + (row - back) * xstride + 8 * c8), xv);
-    } else {
-      const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(taps - 1 + src) * C + 8 * c8);
-      const float4 s0 = sp[0], s1 = sp[1];
-      xv[0] = s0.x, xv[1] = s0.y, xv[2] = s0.z, xv[3] = s0.w, xv[4] = s1.x, xv[5] = s1.y, xv[6] = s1.z, xv[7] = s1.w;
-    }
-    const float4* wp = reinterpret_cast<const float4*>(wt + (int64_t)j * C + 8 * c8);
-    const float4 w0 = wp[0], w1 = wp[1];
-    acc[0] += w0.x * xv[0], acc[1] += w0.y * xv[1], acc[2] += w0.z * xv[2], acc[3] += w0.w * xv[3];
-    acc[4] += w1.x * xv[4], acc[5] += w1.y * xv[5], acc[6] += w1.z * xv[6], acc[7] += w1.w * xv[7];
+    for (int e = 0; e < 8; ++e) xv[e] = 0.f;
+  } else if (i - back >= 0) {
+    unpack8(*reinterpret_cast<const uint4*>(x + (row - back) * xstride + 8 * c8), xv);
+  } else {
+    const float4* sp = reinterpret_cast<const float4*>(st + (int64_t)(taps - 1 + i - back) * C + 8 * c8);
+    const float4 s0 = sp[0], s1 = sp[1];
+    xv[0] = s0.x, xv[1] = s0.y, xv[2] = s0.z, xv[3] = s0.w, xv[4] = s1.x, xv[5] = s1.y, xv[6] = s1.z, xv[7] = s1.w;
   }
 }
 // One row per sequence: the calling thread is the only reader of its channels' tail, so it shifts it: state row k takes
@@ -362,6 +357,126 @@ __device__ __forceinline__ void conv8_shift(const bf16_t* x, int64_t row, int64_
     dp[1] = make_float4(xv[4], xv[5], xv[6], xv[7]);
   }
 }
+// rows of a tile: of row rr, its place i in its sequence's rows of this step, its position and its sequence's state
+struct ConvRow {
+  int i;
+  int64_t p;
+  float* st;
+};
+constexpr int CONV_WIN = 4;   // taps held in registers; more are read again for every row
+// The convolution of nr consecutive rows for 8 channels, tap-major weights: the weights and the rows (with the CONV_WIN - 1
+// rows in front of the tile) are loaded once, all in flight together. put(rr, values): takes a row's 8 results. one_row: a
+// step of one row per sequence (nr = 1), whose inputs behind the row are all state; the state then also takes the row.
+template <int R, typename F>
+__device__ __forceinline__ void conv_rows8(const bf16_t* x, int64_t row0, int nr, int64_t xstride, int c8, const ConvRow* cr,
+                                           const float* wt, int taps, int C, bool one_row, F&& put) {
+  constexpr int B = CONV_WIN - 1;
+  uint4 xr[R + B];   // row row0 - B + j
+#pragma unroll
+  for (int j = 0; j < R + B; ++j) {
+    xr[j] = make_uint4(0, 0, 0, 0);
+    if (j < B && (R == 1 || j < CONV_WIN - taps)) continue;   // (single rows: below)
+    const int64_t row = row0 + min(j - B, nr - 1);
+    xr[j] = *reinterpret_cast<const uint4*>(x + (row < 0 ? 0 : row) * xstride + 8 * c8);
+  }
+  float w[CONV_WIN][8];
+#pragma unroll
+  for (int b = 0; b < CONV_WIN; ++b) {   // [taps back]
+    const float4* wp = reinterpret_cast<const float4*>(wt + (int64_t)max(0, taps - 1 - b) * C + 8 * c8);
+    const float4 w0 = wp[0], w1 = wp[1];
+    w[b][0] = w0.x, w[b][1] = w0.y, w[b][2] = w0.z, w[b][3] = w0.w, w[b][4] = w1.x, w[b][5] = w1.y, w[b][6] = w1.z, w[b][7] = w1.w;
+  }
+  if (R == 1 && one_row && taps <= CONV_WIN) {
+    const ConvRow c = cr[0];
+    float4 s0[B], s1[B];   // b + 1 rows back
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      const int k = taps - 2 - b;
+      s0[b] = s1[b] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (k < 0) continue;
+      const float4* sp = reinterpret_cast<const float4*>(c.st + (int64_t)k * C + 8 * c8);
+      s0[b] = sp[0], s1[b] = sp[1];
+    }
+    float win[CONV_WIN][8], acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    unpack8(xr[B], win[0]);
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      const bool past = c.p - (b + 1) >= 0;   // before the sequence's start: zeros, whatever the slot holds
+      const float4 u0 = past ? s0[b] : make_float4(0.f, 0.f, 0.f, 0.f), u1 = past ? s1[b] : make_float4(0.f, 0.f, 0.f, 0.f);
+      win[b + 1][0] = u0.x, win[b + 1][1] = u0.y, win[b + 1][2] = u0.z, win[b + 1][3] = u0.w;
+      win[b + 1][4] = u1.x, win[b + 1][5] = u1.y, win[b + 1][6] = u1.z, win[b + 1][7] = u1.w;
+    }
+#pragma unroll
+    for (int b = CONV_WIN - 1; b >= 0; --b) {
+      if (b < taps) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] += w[b][e] * win[b][e];
+      }
+    }
+    put(0, acc);
+#pragma unroll
+    for (int b = 0; b < B; ++b) {   // the input b rows back lands in place taps - 2 - b
+      const int k = taps - 2 - b;
+      if (k < 0) continue;
+      float4* dp = reinterpret_cast<float4*>(c.st + (int64_t)k * C + 8 * c8);
+      dp[0] = make_float4(win[b][0], win[b][1], win[b][2], win[b][3]);
+      dp[1] = make_float4(win[b][4], win[b][5], win[b][6], win[b][7]);
+    }
+    return;
+  }
+  float xf[R + B][8];
+#pragma unroll
+  for (int j = 0; j < R + B; ++j) unpack8(xr[j], xf[j]);
+#pragma unroll
+  for (int rr = 0; rr < R; ++rr) {
+    if (rr >= nr) break;
+    const ConvRow c = cr[rr];
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (R > 1 && taps <= CONV_WIN && c.i >= taps - 1) {   // every input is a row of this step
+#pragma unroll
+      for (int b = CONV_WIN - 1; b >= 0; --b) {
+        if (b < taps) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) acc[e] += w[b][e] * xf[rr + B - b][e];
+        }
+      }
+    } else {
+      for (int b = taps - 1; b >= 0; --b) {
+        float xv[8];
+        conv_in8(xv, x, row0 + rr, xstride, c8, c.st, taps, C, c.i, c.p, b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] += wt[(int64_t)(taps - 1 - b) * C + 8 * c8 + e] * xv[e];
+      }
+    }
+    put(rr, acc);
+  }
+  if (one_row) conv8_shift(x, row0, xstride, c8, cr[0].st, taps, C, cr[0].p);
+}
+// Fills cr for rows row0 .. row0 + nr - 1. Every thread looks at its own sequences, so that finding the rows' sequences costs
+// one round of loads (a binary search would be a chain of them).
+__device__ __forceinline__ void conv_rows_of(ConvRow* cr, int64_t row0, int nr, const RaggedRows& r, float* conv_state, int taps,
+                                             int C) {
+  auto fill = [&](int rr, int s, int first) {
+    cr[rr].i = (int)row0 + rr - first;
+    cr[rr].p = r.positions[row0 + rr];
+    cr[rr].st = conv_state + (int64_t)r.state_slots[s] * (taps - 1) * C;
+  };
+  if (r.cu_q == nullptr) {
+    for (int rr = threadIdx.x; rr < nr; rr += NT) fill(rr, (int)row0 + rr, (int)row0 + rr);
+  } else {
+    for (int s = threadIdx.x; s < r.num_seqs; s += NT) {
+      const int lo = r.cu_q[s], hi = r.cu_q[s + 1];
+      for (int rr = max(0, lo - (int)row0); rr < nr && (int)row0 + rr < hi; ++rr) fill(rr, s, lo);
+    }
+  }
+  __syncthreads();
+}
+// rows per workgroup: as many as fit 48 KB of LDS (fp32 [R][n]), at most 4; one in a step of one row per sequence
+static int conv_tile(const RaggedRows& r, int64_t n) {
+  if (r.cu_q == nullptr) return 1;
+  const int64_t fit = 48 * 1024 / (4 * n);
+  return fit >= 4 ? 4 : (fit >= 2 ? 2 : 1);
+}
 // the same for one channel; wc / wj: strides of the weight's channel and tap
 __device__ __forceinline__ float conv1(const void* x, bool f32, int64_t row, int64_t xstride, int c, const float* st,
                                        const float* w, int64_t wc, int64_t wj, int taps, int C, int i, int64_t p) {
@@ -382,64 +497,89 @@ __device__ __forceinline__ void conv1_shift(const void* x, bool f32, int64_t row
   if (taps > 1) st[(int64_t)(taps - 2) * C + c] = ldv(x, row * xstride + c, f32);
 }
 
+// a lane's share of the sum of squares of a head of d values in LDS, 16 lanes per head (gl: the lane); rows of n values.
+// 16 bytes per lane where that is aligned: heads a multiple of the bank count apart then do not collide
+__device__ __forceinline__ float lane_sumsq(const float* v, int d, int gl, int n) {
+  float ss = 0.f;
+  if (((d | n) & 3) == 0) {
+    for (int c = 4 * gl; c < d; c += 64) {
+      const float4 x = *reinterpret_cast<const float4*>(v + c);
+      ss += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+    }
+  } else {
+    for (int c = gl; c < d; c += 16) ss += v[c] * v[c];
+  }
+  return ss;
+}
+
+template <int R>
 __global__ void __launch_bounds__(NT) delta_prep_kernel(float* qkv32, float* bg, const void* x, const void* b,
                                                        const void* a, int64_t xstride, bool f32, const float* conv_w,
                                                        const float* conv_wt, float* conv_state, const float* A_log,
                                                        const float* dt_bias, DeltaShape sh, RaggedRows r) {
-  extern __shared__ __attribute__((aligned(16))) float vals[];  // [C]
-  const int row = blockIdx.x;
-  const int s = seq_of_row(r.cu_q, r.num_seqs, row);
-  const int first = r.cu_q ? r.cu_q[s] : s;
-  const int i = row - first;
-  const int64_t p = r.positions[row];
+  extern __shared__ __attribute__((aligned(16))) float vals[];  // [R][C]
+  __shared__ ConvRow cr[R];
+  const int64_t row0 = (int64_t)blockIdx.x * R;
+  const int nr = min(R, (int)(r.total_rows - row0));
   const int C = sh.channels(), taps = sh.taps;
-  float* st = conv_state + (int64_t)r.state_slots[s] * (taps - 1) * C;
-  // bf16 steps with the weights also given tap-major ([taps, C]): 8 channels per thread and trip, 16-byte loads of
-  // inputs, weights and state (a decode row is then two dependent trips per thread instead of C / 256)
+  conv_rows_of(cr, row0, nr, r, conv_state, taps, C);
+  // bf16 steps with the weights also given tap-major ([taps, C]): 8 channels per thread and trip
   const bool wide = conv_wt != nullptr && !f32 && C % 8 == 0 && xstride % 8 == 0 && aligned16(x);
   const bf16_t* xb = reinterpret_cast<const bf16_t*>(x);
   for (int c8 = threadIdx.x; wide && c8 < C / 8; c8 += NT) {
-    float acc[8];
-    conv8(acc, xb, row, xstride, c8, st, conv_wt, taps, C, i, p);
+    conv_rows8<R>(xb, row0, nr, xstride, c8, cr, conv_wt, taps, C, r.cu_q == nullptr, [&](int rr, const float* acc) {
+      float4* dst = reinterpret_cast<float4*>(vals + rr * C + 8 * c8);
+      float v[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) vals[8 * c8 + e] = rnd(siluf(rnd(acc[e], false)), false);
-    if (r.cu_q == nullptr) conv8_shift(xb, row, xstride, c8, st, taps, C, p);
+      for (int e = 0; e < 8; ++e) v[e] = rnd(siluf(rnd(acc[e], false)), false);
+      dst[0] = make_float4(v[0], v[1], v[2], v[3]);
+      dst[1] = make_float4(v[4], v[5], v[6], v[7]);
+    });
   }
   for (int c = threadIdx.x; !wide && c < C; c += NT) {
-    vals[c] = rnd(siluf(rnd(conv1(x, f32, row, xstride, c, st, conv_w, taps, 1, taps, C, i, p), f32)), f32);
-    if (r.cu_q == nullptr) conv1_shift(x, f32, row, xstride, c, st, taps, C, p);
+    for (int rr = 0; rr < nr; ++rr)
+      vals[rr * C + c] = rnd(siluf(rnd(conv1(x, f32, row0 + rr, xstride, c, cr[rr].st, conv_w, taps, 1, taps, C, cr[rr].i, cr[rr].p), f32)), f32);
+    if (r.cu_q == nullptr) conv1_shift(x, f32, row0, xstride, c, cr[0].st, taps, C, cr[0].p);
   }
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  // unit q and k: 16 lanes per head
+  const int gl = threadIdx.x & 15, grp = threadIdx.x >> 4;
   const int G = sh.kv_heads, d = sh.dim;
-  for (int hh = wave; hh < 2 * G; hh += NT / 64) {
-    float* v = vals + hh * d;
-    float ss = 0.f;
-    for (int c = lane; c < d; c += 64) ss += v[c] * v[c];
-    ss = wave_sum(ss);
-    float sc = 1.0f / sqrtf(ss + 1e-6f);
+  const float inv_2g = 1.0f / (float)(2 * G);
+  for (int u = grp; u < nr * 2 * G; u += NT / 16) {
+    const int rr = R == 1 ? 0 : qdiv(u, inv_2g), hh = u - rr * 2 * G;
+    float* v = vals + rr * C + hh * d;
+    float sc = 1.0f / sqrtf(group_sum<16>(lane_sumsq(v, d, gl, C)) + 1e-6f);
     if (hh < G) sc *= 1.0f / sqrtf((float)d);
-    for (int c = lane; c < d; c += 64) v[c] *= sc;
+    if (((d | C) & 3) == 0) {
+      for (int c = 4 * gl; c < d; c += 64) {
+        const float4 x = *reinterpret_cast<const float4*>(v + c);
+        *reinterpret_cast<float4*>(v + c) = make_float4(x.x * sc, x.y * sc, x.z * sc, x.w * sc);
+      }
+    } else {
+      for (int c = gl; c < d; c += 16) v[c] *= sc;
+    }
   }
   __syncthreads();
   if (C % 4 == 0) {
-    float4* dst = reinterpret_cast<float4*>(qkv32 + (int64_t)row * C);
-    for (int c4 = threadIdx.x; c4 < C / 4; c4 += NT) dst[c4] = reinterpret_cast<const float4*>(vals)[c4];
+    float4* dst = reinterpret_cast<float4*>(qkv32 + row0 * C);
+    for (int c4 = threadIdx.x; c4 < nr * C / 4; c4 += NT) dst[c4] = reinterpret_cast<const float4*>(vals)[c4];
   } else {
-    for (int c = threadIdx.x; c < C; c += NT) qkv32[(int64_t)row * C + c] = vals[c];
+    for (int c = threadIdx.x; c < nr * C; c += NT) qkv32[row0 * C + c] = vals[c];
   }
   const int H = sh.heads;
-  if (a == nullptr) {   // the decay is the recurrence kernel's (per key channel)
-    for (int h = threadIdx.x; h < H; h += NT)
-      bg[(int64_t)row * H + h] = 1.0f / (1.0f + expf(-ldv(b, (int64_t)row * xstride + h, f32)));
-    return;
-  }
-  for (int h = threadIdx.x; h < H; h += NT) {
-    const float bv = ldv(b, (int64_t)row * xstride + h, f32);
-    const float av = ldv(a, (int64_t)row * xstride + h, f32) + dt_bias[h];
-    const float sp = av > 20.f ? av : log1pf(expf(av));
-    bg[(int64_t)row * 2 * H + h] = 1.0f / (1.0f + expf(-bv));
-    bg[(int64_t)row * 2 * H + H + h] = expf(-expf(A_log[h]) * sp);
+  const float inv_h = 1.0f / (float)H;
+  for (int u = threadIdx.x; u < nr * H; u += NT) {
+    const int rr = R == 1 ? 0 : qdiv(u, inv_h), h = u - rr * H;
+    const int64_t row = row0 + rr;
+    const float beta = sigmoidf(ldv(b, row * xstride + h, f32));
+    if (a == nullptr) {   // the decay is the recurrence kernel's (per key channel)
+      bg[row * H + h] = beta;
+      continue;
+    }
+    const float sp = softplus_of<false>(ldv(a, row * xstride + h, f32) + dt_bias[h]);
+    bg[row * 2 * H + h] = beta;
+    bg[row * 2 * H + H + h] = expf(-expf(A_log[h]) * sp);
   }
 }
 
@@ -660,42 +800,43 @@ __global__ void __launch_bounds__(1024) gated_delta_kernel(GatedDeltaArgs a, Rag
 }
 
 // --------------------------------------------------------------------------------------------------- qkv prep
+// One workgroup per R rows (R > 1 with a convolution only, which then reads its weights once for all of them).
+template <int R, bool CONV>
 __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
-  extern __shared__ float sm[];
+  extern __shared__ __attribute__((aligned(16))) float sm[];
   __shared__ float red[NT / 64];
+  __shared__ ConvRow cr[CONV ? R : 1];
   const int H = a.heads, G = a.kv_heads, d = a.dim, dv = a.vdim;
-  const int nq = H * d, nk = G * d, nv = G * dv;
-  float* qv = sm;
+  const int nq = H * d, nk = G * d, nv = G * dv, C = nq + nk + nv;
+  float* qv = sm;               // row rr: [q | k | v] at rr * C
   float* kv = qv + nq;
   float* vv = kv + nk;
-  // cosine / sine of the row's rotation angles, shared by the heads: keys and queries, then values
-  const int half = a.rot_dims / 2, vhalf = a.v_inv_freq != nullptr ? dv / 2 : 0;
-  float* ct = vv + nv;
-  float* snt = ct + half + vhalf;
-  const int64_t t = blockIdx.x;
+  // cosine / sine of the rows' rotation angles, shared by the heads: keys and queries, then values
+  const int half = a.rot_dims / 2, vhalf = a.v_inv_freq != nullptr ? dv / 2 : 0, nang = half + vhalf;
+  float* ct = sm + R * C;
+  float* snt = ct + R * nang;
+  const int64_t t0 = (int64_t)blockIdx.x * R;
+  const int nr = R == 1 ? 1 : min(R, (int)(a.T - t0));
   const bool f32 = a.f32;
-  {
-    const float p = (float)a.positions[t];
-    for (int e = threadIdx.x; e < half + vhalf; e += NT) {
-      const bool kq = e < half;
-      float sn, cs;
-      sincosf(p * (kq ? a.inv_freq[e] : a.v_inv_freq[e - half]), &sn, &cs);
-      const float gain = kq ? a.rot_gain : 1.0f;
-      ct[e] = cs * gain;
-      snt[e] = sn * gain;
-    }
+  // cache row of key/value head 0 (head g: g * block_size further; a block's interior is head-major), < 0: not written
+  __shared__ int64_t crow[R];
+  if (threadIdx.x < nr) {
+    const int64_t slot = a.slots[t0 + threadIdx.x];
+    const int64_t blk = slot / a.block_size;
+    crow[threadIdx.x] = slot < 0 ? -1 : blk * G * a.block_size + (slot - blk * a.block_size);
   }
-  // short convolution over the sequence of the channels q | k | v (adjacent columns)
-  const int C = nq + nk + nv;
-  const int taps = a.conv_wt != nullptr ? a.taps : 0;
-  int ci = 0;
-  float* cst = nullptr;
-  if (taps > 0) {
-    const int sq_ = seq_of_row(a.r.cu_q, a.r.num_seqs, (int)t);
-    ci = (int)t - (a.r.cu_q ? a.r.cu_q[sq_] : sq_);
-    cst = a.conv_state + (int64_t)a.r.state_slots[sq_] * (taps - 1) * C;
+  const float inv_ang = 1.0f / (float)max(1, nang), inv_half = 1.0f / (float)max(1, half), inv_vhalf = 1.0f / (float)max(1, vhalf),
+              inv_hg = 1.0f / (float)(H + G), inv_g = 1.0f / (float)G, inv_d = 1.0f / (float)d, inv_dv = 1.0f / (float)dv;
+  for (int e = threadIdx.x; e < nr * nang; e += NT) {
+    const int rr = R == 1 ? 0 : qdiv(e, inv_ang), i = e - rr * nang;
+    const bool kq = i < half;
+    float sn, cs;
+    sincosf((float)a.positions[t0 + rr] * (kq ? a.inv_freq[i] : a.v_inv_freq[i - half]), &sn, &cs);
+    const float gain = kq ? a.rot_gain : 1.0f;
+    ct[e] = cs * gain;
+    snt[e] = sn * gain;
   }
-  float sq = 0.f, sk = 0.f;
+  float sq = 0.f, sk = 0.f;   // sums of squares over the whole projections (used with R == 1)
   float lam = 0.f;
   if (a.v_lambda != nullptr) lam = a.v_lambda[0];
   // bf16 with head sizes that are multiples of 8: 16-byte loads and stores, 8 values per thread and trip
@@ -703,102 +844,105 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
   const bool wide = !f32 && d % 8 == 0 && dv % 8 == 0 && a.xstride % 8 == 0 && aligned16(a.q) && aligned16(a.k) &&
                     aligned16(a.v) && aligned16(a.q_out) && aligned16(a.cache) &&
                     (a.v_first == nullptr || (a.vfstride % 8 == 0 && aligned16(a.v_first)));
-  if (wide) {
-    const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.q) + t * a.xstride;
-    const bf16_t* kp = reinterpret_cast<const bf16_t*>(a.k) + t * a.xstride;
-    const bf16_t* vp = reinterpret_cast<const bf16_t*>(a.v) + t * a.xstride;
-    for (int c8 = threadIdx.x; c8 < (v_is_k ? nq + nk : nq + nk + nv) / 8; c8 += NT) {
+  if (CONV) {
+    // short convolution over the sequence of the channels q | k | v (adjacent columns)
+    conv_rows_of(cr, t0, nr, a.r, a.conv_state, a.taps, C);
+    const bf16_t* xb = reinterpret_cast<const bf16_t*>(a.q);
+    for (int c8 = threadIdx.x; wide && c8 < C / 8; c8 += NT) {
+      conv_rows8<R>(xb, t0, nr, a.xstride, c8, cr, a.conv_wt, a.taps, C, a.r.cu_q == nullptr, [&](int rr, const float* acc) {
+        float4* dst = reinterpret_cast<float4*>(qv + rr * C + 8 * c8);
+        dst[0] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+        dst[1] = make_float4(acc[4], acc[5], acc[6], acc[7]);
+        if (R == 1) {
+          float ss = 0.f;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) ss += acc[e] * acc[e];
+          if (8 * c8 < nq)
+            sq += ss;
+          else if (8 * c8 < nq + nk)
+            sk += ss;
+        }
+      });
+    }
+    for (int c = threadIdx.x; !wide && c < C; c += NT) {
+      for (int rr = 0; rr < nr; ++rr) {
+        const float x = conv1(a.q, f32, t0 + rr, a.xstride, c, cr[rr].st, a.conv_wt, 1, C, a.taps, C, cr[rr].i, cr[rr].p);
+        qv[rr * C + c] = x;
+        if (c < nq)
+          sq += x * x;
+        else if (c < nq + nk)
+          sk += x * x;
+      }
+      if (a.r.cu_q == nullptr) conv1_shift(a.q, f32, t0, a.xstride, c, cr[0].st, a.taps, C, cr[0].p);
+    }
+  } else if (wide) {
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.q) + t0 * a.xstride;
+    const bf16_t* kp = reinterpret_cast<const bf16_t*>(a.k) + t0 * a.xstride;
+    const bf16_t* vp = reinterpret_cast<const bf16_t*>(a.v) + t0 * a.xstride;
+    for (int c8 = threadIdx.x; c8 < (v_is_k ? nq + nk : C) / 8; c8 += NT) {
       const int c = 8 * c8;
       float f[8];
-      if (taps > 0 || a.bias != nullptr) {   // q, k and v are adjacent columns here
-        if (taps > 0) {
-          conv8(f, reinterpret_cast<const bf16_t*>(a.q), t, a.xstride, c8, cst, a.conv_wt, taps, C, ci, a.positions[t]);
-          if (a.r.cu_q == nullptr)
-            conv8_shift(reinterpret_cast<const bf16_t*>(a.q), t, a.xstride, c8, cst, taps, C, a.positions[t]);
-        } else {
-          unpack8(*reinterpret_cast<const uint4*>(qp + c), f);
-#pragma unroll
-          for (int e = 0; e < 8; ++e) f[e] += a.bias[c + e];
-        }
+      unpack8(*reinterpret_cast<const uint4*>(c < nq ? qp + c : (c < nq + nk ? kp + c - nq : vp + c - nq - nk)), f);
+      if (a.bias != nullptr) {
+        const float4* bp = reinterpret_cast<const float4*>(a.bias + c);
+        const float4 b0 = bp[0], b1 = bp[1];
+        f[0] += b0.x, f[1] += b0.y, f[2] += b0.z, f[3] += b0.w, f[4] += b1.x, f[5] += b1.y, f[6] += b1.z, f[7] += b1.w;
+      }
+      if (c < nq + nk) {
         float ss = 0.f;
 #pragma unroll
         for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
         if (c < nq)
           sq += ss;
-        else if (c < nq + nk)
+        else
           sk += ss;
-      } else if (c < nq) {
-        unpack8(*reinterpret_cast<const uint4*>(qp + c), f);
+      } else if (a.v_lambda != nullptr) {
+        float g8[8];
+        unpack8(*reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(a.v_first) + t0 * a.vfstride + c - nq - nk), g8);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) sq += f[e] * f[e];
-      } else if (c < nq + nk) {
-        unpack8(*reinterpret_cast<const uint4*>(kp + c - nq), f);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) sk += f[e] * f[e];
-      } else {
-        unpack8(*reinterpret_cast<const uint4*>(vp + c - nq - nk), f);
-        if (a.v_lambda != nullptr) {
-          float g8[8];
-          unpack8(*reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(a.v_first) + t * a.vfstride + c - nq - nk), g8);
-#pragma unroll
-          for (int e = 0; e < 8; ++e) f[e] = (1.0f - lam) * f[e] + lam * g8[e];
-        }
+        for (int e = 0; e < 8; ++e) f[e] = (1.0f - lam) * f[e] + lam * g8[e];
       }
-#pragma unroll
-      for (int e = 0; e < 8; ++e) qv[c + e] = f[e];   // qv, kv and vv are adjacent
+      float4* dst = reinterpret_cast<float4*>(qv + c);   // qv, kv and vv are adjacent
+      dst[0] = make_float4(f[0], f[1], f[2], f[3]);
+      dst[1] = make_float4(f[4], f[5], f[6], f[7]);
     }
   } else {
-    const bool pre = taps > 0 || a.bias != nullptr;
-    for (int c = threadIdx.x; pre && c < C; c += NT) {   // q, k and v are adjacent columns here
-      float x;
-      if (taps > 0) {
-        x = conv1(a.q, f32, t, a.xstride, c, cst, a.conv_wt, 1, C, taps, C, ci, a.positions[t]);
-        if (a.r.cu_q == nullptr) conv1_shift(a.q, f32, t, a.xstride, c, cst, taps, C, a.positions[t]);
-      } else {
-        x = ldv(a.q, t * a.xstride + c, f32) + a.bias[c];
-      }
-      qv[c] = x;
-      if (c < nq)
-        sq += x * x;
-      else if (c < nq + nk)
-        sk += x * x;
-    }
-    for (int c = threadIdx.x; !pre && c < nq; c += NT) {
-      const float x = ldv(a.q, t * a.xstride + c, f32);
+    for (int c = threadIdx.x; c < nq; c += NT) {
+      const float x = ldv(a.q, t0 * a.xstride + c, f32) + (a.bias != nullptr ? a.bias[c] : 0.f);
       qv[c] = x;
       sq += x * x;
     }
-    for (int c = threadIdx.x; !pre && c < nk; c += NT) {
-      const float x = ldv(a.k, t * a.xstride + c, f32);
+    for (int c = threadIdx.x; c < nk; c += NT) {
+      const float x = ldv(a.k, t0 * a.xstride + c, f32) + (a.bias != nullptr ? a.bias[nq + c] : 0.f);
       kv[c] = x;
       sk += x * x;
     }
-    for (int c = threadIdx.x; !pre && c < (v_is_k ? 0 : nv); c += NT) {
-      float x = ldv(a.v, t * a.xstride + c, f32);
-      if (a.v_lambda != nullptr) x = (1.0f - lam) * x + lam * ldv(a.v_first, t * a.vfstride + c, f32);
+    for (int c = threadIdx.x; c < (v_is_k ? 0 : nv); c += NT) {
+      float x = ldv(a.v, t0 * a.xstride + c, f32) + (a.bias != nullptr ? a.bias[nq + nk + c] : 0.f);
+      if (a.v_lambda != nullptr) x = (1.0f - lam) * x + lam * ldv(a.v_first, t0 * a.vfstride + c, f32);
       vv[c] = x;
     }
   }
   const bool per_head = a.q_norm != nullptr && a.head_norm;
   auto rotate = [&]() {
-    for (int e = threadIdx.x; e < (H + G) * half; e += NT) {
-      const int hd = e / half, i = e % half;
-      float* base = hd < H ? qv + hd * d : kv + (hd - H) * d;
-      const float cs = ct[i], sn = snt[i];
+    for (int e = threadIdx.x; e < nr * (H + G) * half; e += NT) {
+      const int hr = qdiv(e, inv_half), i = e - hr * half;
+      const int rr = R == 1 ? 0 : qdiv(hr, inv_hg), hd = hr - rr * (H + G);
+      float* base = (hd < H ? qv + hd * d : kv + (hd - H) * d) + rr * C;
+      const float cs = ct[rr * nang + i], sn = snt[rr * nang + i];
       const float u = base[i], v = base[i + half];
       base[i] = u * cs - v * sn;
       base[i + half] = v * cs + u * sn;
     }
   };
+  // query temperature of row rr
+  auto temperature = [&](int rr) {
+    return 1.0f + a.q_temp_coef * logf((float)((a.positions[t0 + rr] + 1) / a.q_temp_every) + 1.0f);
+  };
   const bool rot_first = per_head && a.norm_after_rot;
   if (a.rot_dims > 0 && rot_first) {
     __syncthreads();   // every thread's loads are in LDS
     rotate();
-  }
-  float qm = 1.0f;   // query temperature
-  if (a.q_temp_coef != 0.f) {
-    const int64_t p = a.positions[t];
-    qm = 1.0f + a.q_temp_coef * logf((float)((p + 1) / a.q_temp_every) + 1.0f);
   }
   if (v_is_k && !per_head) {
     __syncthreads();
@@ -809,23 +953,28 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
     // (values taken from the keys) and folds the query temperature into the q heads' factor
     __syncthreads();
     const int grp = threadIdx.x >> 4, gl = threadIdx.x & 15;
-    for (int hd = grp; hd < H + G; hd += NT / 16) {
-      float* base = hd < H ? qv + hd * d : kv + (hd - H) * d;
+    for (int u = grp; u < nr * (H + G); u += NT / 16) {
+      const int rr = R == 1 ? 0 : qdiv(u, inv_hg), hd = u - rr * (H + G);
+      float* base = (hd < H ? qv + hd * d : kv + (hd - H) * d) + rr * C;
       const float* w = hd < H ? a.q_norm : a.k_norm;
       float* raw = (v_is_k && hd >= H) ? vv + (hd - H) * d : nullptr;
-      float ss = 0.f;
-      for (int c = gl; c < d; c += 16) ss += base[c] * base[c];
-#pragma unroll
-      for (int off = 8; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
-      float rs = 1.0f / sqrtf(ss / (float)d + a.eps);
-      if (hd < H) rs *= qm;
+      float rs = 1.0f / sqrtf(group_sum<16>(lane_sumsq(base, d, gl, C)) / (float)d + a.eps);
+      if (hd < H && a.q_temp_coef != 0.f) rs *= temperature(rr);
+      if (((d | C) & 3) == 0) {
+        for (int c = 4 * gl; c < d; c += 64) {
+          const float4 x = *reinterpret_cast<const float4*>(base + c), ww = *reinterpret_cast<const float4*>(w + c);
+          if (raw != nullptr) *reinterpret_cast<float4*>(raw + c) = x;
+          *reinterpret_cast<float4*>(base + c) = make_float4(x.x * rs * ww.x, x.y * rs * ww.y, x.z * rs * ww.z, x.w * rs * ww.w);
+        }
+        continue;
+      }
       for (int c = gl; c < d; c += 16) {
         const float x = base[c];
         if (raw != nullptr) raw[c] = x;
         base[c] = x * rs * w[c];
       }
     }
-  } else if (a.q_norm != nullptr) {
+  } else if (a.q_norm != nullptr) {   // over the whole projection (R == 1)
     sq = block_sum<NT>(sq, red);   // (a barrier: every thread's loads are in LDS)
     sk = block_sum<NT>(sk, red);
     const float rq = 1.0f / sqrtf(sq / (float)nq + a.eps), rk = 1.0f / sqrtf(sk / (float)nk + a.eps);
@@ -834,51 +983,62 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
   }
   __syncthreads();
   if (a.q_temp_coef != 0.f && !per_head) {
-    for (int c = threadIdx.x; c < nq; c += NT) qv[c] *= qm;
+    for (int rr = 0; rr < nr; ++rr) {
+      const float qm = temperature(rr);
+      for (int c = threadIdx.x; c < nq; c += NT) qv[rr * C + c] *= qm;
+    }
     __syncthreads();
   }
   if (a.rot_dims > 0 && !rot_first) rotate();
-  for (int e = threadIdx.x; e < G * vhalf; e += NT) {   // rotated values
-    const int g = e / vhalf, i = e % vhalf;
-    float* base = vv + g * dv;
-    const float cs = ct[half + i], sn = snt[half + i];
+  for (int e = threadIdx.x; e < nr * G * vhalf; e += NT) {   // rotated values
+    const int rg = qdiv(e, inv_vhalf), i = e - rg * vhalf, rr = R == 1 ? 0 : qdiv(rg, inv_g);
+    float* base = vv + rr * C + (rg - rr * G) * dv;
+    const float cs = ct[rr * nang + half + i], sn = snt[rr * nang + half + i];
     const float u = base[i], v = base[i + vhalf];
     base[i] = u * cs - v * sn;
     base[i + vhalf] = v * cs + u * sn;
   }
   if (a.v_unit) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    for (int g = wave; g < G; g += NT / 64) {
+    for (int rg = wave; rg < nr * G; rg += NT / 64) {
+      const int rr = R == 1 ? 0 : qdiv(rg, inv_g);
+      float* base = vv + rr * C + (rg - rr * G) * dv;
       float ss = 0.f;
-      for (int c = lane; c < dv; c += 64) ss += vv[g * dv + c] * vv[g * dv + c];
+      for (int c = lane; c < dv; c += 64) ss += base[c] * base[c];
       ss = wave_sum(ss);
       const float rs = 1.0f / sqrtf(ss / (float)dv + a.eps);
-      for (int c = lane; c < dv; c += 64) vv[g * dv + c] *= rs;
+      for (int c = lane; c < dv; c += 64) base[c] *= rs;
     }
   }
   __syncthreads();
-  const int64_t slot = a.slots[t];
-  // the block's interior is head-major: [G][block_size][K | V]
-  const int64_t blk = slot / a.block_size, off = slot % a.block_size;
-  if (wide) {
-    bf16_t* qo = reinterpret_cast<bf16_t*>(a.q_out) + t * nq;
-    for (int c8 = threadIdx.x; c8 < nq / 8; c8 += NT) *reinterpret_cast<uint4*>(qo + 8 * c8) = pack8(qv + 8 * c8);
-    if (slot < 0) return;
-    bf16_t* cb = reinterpret_cast<bf16_t*>(a.cache);
-    for (int c8 = threadIdx.x; c8 < (nk + nv) / 8; c8 += NT) {
-      const int c = 8 * c8;
-      const int g = c < nk ? c / d : (c - nk) / dv;
-      const int e = c < nk ? c % d : d + (c - nk) % dv;
-      *reinterpret_cast<uint4*>(cb + ((blk * G + g) * a.block_size + off) * (int64_t)(d + dv) + e) = pack8(kv + c);
+  for (int rr = 0; rr < nr; ++rr) {
+    const int64_t t = t0 + rr;
+    const int64_t row = crow[rr];
+    const float* q = qv + rr * C;
+    if (wide) {
+      bf16_t* qo = reinterpret_cast<bf16_t*>(a.q_out) + t * nq;
+      bf16_t* cb = reinterpret_cast<bf16_t*>(a.cache);
+      for (int c8 = threadIdx.x; c8 < C / 8; c8 += NT) {
+        const int c = 8 * c8;
+        const uint4 w = pack8(q + c);
+        if (c < nq) {
+          *reinterpret_cast<uint4*>(qo + c) = w;
+        } else if (row >= 0) {
+          const int k = c - nq;
+          const int g = k < nk ? qdiv(k, inv_d) : qdiv(k - nk, inv_dv);
+          const int e = k < nk ? k - g * d : d + (k - nk) - g * dv;
+          *reinterpret_cast<uint4*>(cb + (row + (int64_t)g * a.block_size) * (d + dv) + e) = w;
+        }
+      }
+      continue;
     }
-    return;
-  }
-  for (int c = threadIdx.x; c < nq; c += NT) stv(a.q_out, t * nq + c, f32, qv[c]);
-  if (slot < 0) return;
-  for (int c = threadIdx.x; c < nk + nv; c += NT) {
-    const int g = c < nk ? c / d : (c - nk) / dv;
-    const int e = c < nk ? c % d : d + (c - nk) % dv;
-    stv(a.cache, ((blk * G + g) * a.block_size + off) * (int64_t)(d + dv) + e, f32, kv[c]);  // kv and vv are adjacent
+    for (int c = threadIdx.x; c < nq; c += NT) stv(a.q_out, t * nq + c, f32, q[c]);
+    if (row < 0) continue;
+    for (int k = threadIdx.x; k < nk + nv; k += NT) {
+      const int g = k < nk ? qdiv(k, inv_d) : qdiv(k - nk, inv_dv);
+      const int e = k < nk ? k - g * d : d + (k - nk) - g * dv;
+      stv(a.cache, (row + (int64_t)g * a.block_size) * (d + dv) + e, f32, q[nq + k]);
+    }
   }
 }
 
@@ -929,14 +1089,15 @@ hipError_t launch_delta_prep(float* qkv32, float* bg, const void* x, const void*
                              const float* A_log, const float* dt_bias, DeltaShape sh, RaggedRows r, hipStream_t s) {
   if (r.total_rows == 0) return hipSuccess;
   if (!delta_ok(sh) || !rows_ok(r)) return hipErrorInvalidValue;
-  const size_t lds = sizeof(float) * sh.channels();
+  const int R = conv_tile(r, sh.channels());
+  const size_t lds = sizeof(float) * R * sh.channels();
   if (lds > 150 * 1024) return hipErrorInvalidValue;
+  auto* fn = R == 4 ? delta_prep_kernel<4> : (R == 2 ? delta_prep_kernel<2> : delta_prep_kernel<1>);
   if (lds > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prep_kernel),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
   }
-  hipLaunchKernelGGL(delta_prep_kernel, dim3(r.total_rows), dim3(NT), lds, s, qkv32, bg, x, b, a, xstride, f32, conv_w,
+  hipLaunchKernelGGL(fn, dim3((r.total_rows + R - 1) / R), dim3(NT), lds, s, qkv32, bg, x, b, a, xstride, f32, conv_w,
                      conv_wt, conv_state, A_log, dt_bias, sh, r);
   return hipGetLastError();
 }
@@ -1004,15 +1165,18 @@ hipError_t launch_qkv_prep(const QkvPrepArgs& a, hipStream_t s) {
                                a.taps > TAPS_MAX || !rows_ok(a.r) || (a.taps > 1 && a.conv_state == nullptr)))
     return hipErrorInvalidValue;
   if (a.bias != nullptr && (a.v == nullptr || a.v_lambda != nullptr)) return hipErrorInvalidValue;
-  const size_t lds = sizeof(float) * ((size_t)a.heads * a.dim + (size_t)a.kv_heads * (a.dim + a.vdim) + a.rot_dims +
-                                      (a.v_inv_freq != nullptr ? a.vdim : 0));
+  const size_t C = (size_t)a.heads * a.dim + (size_t)a.kv_heads * (a.dim + a.vdim);   // (150 KB of LDS bound every index below 2^21)
+  const bool conv = a.conv_wt != nullptr;
+  const int R = conv && (a.q_norm == nullptr || a.head_norm) ? conv_tile(a.r, C) : 1;
+  const size_t lds = sizeof(float) * R * (C + a.rot_dims + (a.v_inv_freq != nullptr ? a.vdim : 0));
   if (lds > 150 * 1024) return hipErrorInvalidValue;
+  auto* fn = !conv ? qkv_prep_kernel<1, false>
+                   : (R == 4 ? qkv_prep_kernel<4, true> : (R == 2 ? qkv_prep_kernel<2, true> : qkv_prep_kernel<1, true>));
   if (lds > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(qkv_prep_kernel),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
   }
-  hipLaunchKernelGGL(qkv_prep_kernel, dim3(a.T), dim3(NT), lds, s, a);
+  hipLaunchKernelGGL(fn, dim3((a.T + R - 1) / R), dim3(NT), lds, s, a);
   return hipGetLastError();
 }
 

@@ -516,6 +516,20 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
 }
 
 
+// column c of an output row (token t, head h) after the optional turn and gate, from the row's raw columns o(c)
+template <typename F>
+__device__ __forceinline__ float gated_out(const SinkAttnArgs& a, int64_t t, int h, int c, F&& o) {
+  float v = o(c);
+  if (a.gate == nullptr) return v;
+  if (a.out_inv_freq != nullptr) {
+    const int half = a.vdim / 2, i = c < half ? c : c - half;
+    float sn, cs;
+    sincosf((float)a.positions[t] * a.out_inv_freq[i], &sn, &cs);
+    v = c < half ? v * cs + o(c + half) * sn : v * cs - o(c - half) * sn;
+  }
+  return v * a.gate_mult / (1.0f + expf(-bf2f(reinterpret_cast<const bf16_t*>(a.gate)[t * a.gstride + h])));
+}
+
 // ---------------------------------------------------------------------------------------------------
 // Decode steps (one query token per sequence) in bf16, dim % 8 == 0 <= 256, vdim % 8 == 0 <= 256, at most 8 query
 // heads per key/value head: no matrix cores and no staging of keys in LDS. A workgroup of 256 threads owns one
@@ -681,31 +695,39 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
   __syncthreads();
   for (int idx = tid; idx < QPG * DV; idx += 256) {
     const int r = idx / DV, c = idx % DV;
-    float o = 0.f;
+    auto column = [&](int col) {
+      float v = 0.f;
 #pragma unroll
-    for (int k = 0; k < NV; ++k) o += red[((int64_t)k * R + r) * DV + c];
+      for (int k = 0; k < NV; ++k) v += red[((int64_t)k * R + r) * DV + col];
+      return v;
+    };
     const int64_t orow = (int64_t)s * H + g * QPG + r;
     if (nsplit > 1) {
-      ws_o[((int64_t)z * wrows + orow) * DV + c] = o;
+      ws_o[((int64_t)z * wrows + orow) * DV + c] = column(c);
       if (c == 0) {
         ws_ml[((int64_t)z * wrows + orow) * 2] = ml[r * 4];
         ws_ml[((int64_t)z * wrows + orow) * 2 + 1] = ml[r * 4 + 1];
       }
     } else {
-      const float l = ml[r * 4 + 1];
-      reinterpret_cast<bf16_t*>(a.out)[orow * DV + c] = f2bf(l > 0.f ? o / l : 0.f);
+      const float l = ml[r * 4 + 1], inv = l > 0.f ? 1.0f / l : 0.f;
+      const int h = g * QPG + r;
+      reinterpret_cast<bf16_t*>(a.out)[(int64_t)s * a.ostride + h * DV + c] =
+          f2bf(gated_out(a, s, h, c, [&](int col) { return column(col) * inv; }));
     }
   }
 }
 
-// out[row] = sum_z O_z 2^(m_z - m*) / sum_z l_z 2^(m_z - m*), m* = max_z m_z (running maxima in log2 units).
-__global__ void __launch_bounds__(128) sink_attn_merge_kernel(bf16_t* out, const float* ws_o, const float* ws_ml,
-                                                              int nsplit, int64_t rows, int DV) {
+// out[row] = sum_z O_z 2^(m_z - m*) / sum_z l_z 2^(m_z - m*), m* = max_z m_z (running maxima in log2 units), then the
+// optional turn and gate. One workgroup per (token, head).
+__global__ void __launch_bounds__(128) sink_attn_merge_kernel(SinkAttnArgs a) {
   __shared__ float wz[128];   // a split's weight 2^(m_z - m*) / sum (nsplit <= 128)
-  const int64_t row = blockIdx.x;
+  __shared__ float orow[256];
+  const int64_t row = blockIdx.x, rows = (int64_t)a.heads * a.total_q;
+  const int64_t t = row / a.heads;
+  const int h = (int)(row - t * a.heads), DV = a.vdim, nsplit = a.nsplit;
   const int z = threadIdx.x;
-  const float mz = z < nsplit ? ws_ml[((int64_t)z * rows + row) * 2] : -1e30f;
-  const float lz = z < nsplit ? ws_ml[((int64_t)z * rows + row) * 2 + 1] : 0.f;
+  const float mz = z < nsplit ? a.ws_ml[((int64_t)z * rows + row) * 2] : -1e30f;
+  const float lz = z < nsplit ? a.ws_ml[((int64_t)z * rows + row) * 2 + 1] : 0.f;
   float mstar = wave_max(mz);
   __shared__ float red2[4];
   if ((threadIdx.x & 63) == 0) red2[threadIdx.x >> 6] = mstar;
@@ -722,10 +744,13 @@ __global__ void __launch_bounds__(128) sink_attn_merge_kernel(bf16_t* out, const
     float acc = 0.f;
     for (int k = 0; k < nsplit; ++k) {
       const float wk = wz[k];
-      if (wk != 0.f) acc += ws_o[((int64_t)k * rows + row) * DV + c] * wk;
+      if (wk != 0.f) acc += a.ws_o[((int64_t)k * rows + row) * DV + c] * wk;
     }
-    out[row * DV + c] = f2bf(acc);
+    orow[c] = acc;
   }
+  if (a.out_inv_freq != nullptr) __syncthreads();   // (else every thread reads its own columns)
+  bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + t * a.ostride + h * DV;
+  for (int c = threadIdx.x; c < DV; c += 128) out[c] = f2bf(gated_out(a, t, h, c, [&](int col) { return orow[col]; }));
 }
 
 template <int NDB, int NW, int NKC> hipError_t launch_mfma(const SinkAttnArgs& a, hipStream_t s) {
@@ -754,8 +779,7 @@ template <int NDB, int NW, int NKC> hipError_t launch_mfma(const SinkAttnArgs& a
   hipLaunchKernelGGL(fn, grid, dim3(64 * NW), lds, s, a, kp, qp, qr, btc, a.ws_o, a.ws_ml, nsplit, a.chunk);
   hipError_t e = hipGetLastError();
   if (e != hipSuccess || nsplit <= 1) return e;
-  hipLaunchKernelGGL(sink_attn_merge_kernel, dim3((unsigned)((int64_t)a.heads * a.total_q)), dim3(128), 0, s,
-                     reinterpret_cast<bf16_t*>(a.out), a.ws_o, a.ws_ml, nsplit, (int64_t)a.heads * a.total_q, a.vdim);
+  hipLaunchKernelGGL(sink_attn_merge_kernel, dim3((unsigned)((int64_t)a.heads * a.total_q)), dim3(128), 0, s, a);
   return hipGetLastError();
 }
 
@@ -798,8 +822,7 @@ template <int R, int LK, int VL> hipError_t launch_decode_one(const SinkAttnArgs
   hipLaunchKernelGGL(fn, dim3(nsplit, a.num_seqs, a.kv_heads), dim3(256), lds, s, a, a.ws_o, a.ws_ml, nsplit, a.chunk);
   hipError_t e = hipGetLastError();
   if (e != hipSuccess || nsplit <= 1) return e;
-  hipLaunchKernelGGL(sink_attn_merge_kernel, dim3((unsigned)((int64_t)a.heads * a.total_q)), dim3(128), 0, s,
-                     reinterpret_cast<bf16_t*>(a.out), a.ws_o, a.ws_ml, nsplit, (int64_t)a.heads * a.total_q, a.vdim);
+  hipLaunchKernelGGL(sink_attn_merge_kernel, dim3((unsigned)((int64_t)a.heads * a.total_q)), dim3(128), 0, s, a);
   return hipGetLastError();
 }
 
@@ -831,11 +854,15 @@ inline bool mfma_ok(const SinkAttnArgs& a) {
 
 bool sink_attn_uses_mfma(const SinkAttnArgs& a) { return a.impl != 1 && mfma_ok(a); }
 bool sink_attn_uses_decode(const SinkAttnArgs& a) { return a.impl == 0 && decode_ok(a); }
+bool sink_attn_fuses_gate(const SinkAttnArgs& a) {
+  return sink_attn_uses_decode(a) || (sink_attn_uses_mfma(a) && a.ws_o != nullptr && a.nsplit > 1);
+}
 
 hipError_t launch_sink_attn(const SinkAttnArgs& a, hipStream_t s) {
   if (a.num_seqs == 0 || a.total_q == 0) return hipSuccess;
   if (a.heads < 1 || a.kv_heads < 1 || a.heads % a.kv_heads != 0 || a.dim < 1 || a.dim > 512 || a.vdim < 1 ||
-      a.vdim > 256 || a.block_size < 1 || a.max_q < 1 || a.window < 0 || a.seg < 0 || (a.bias != nullptr && a.bias_rows < 1))
+      a.vdim > 256 || a.block_size < 1 || a.max_q < 1 || a.window < 0 || a.seg < 0 || (a.gate != nullptr && !sink_attn_fuses_gate(a)) ||
+      (a.out_inv_freq != nullptr && (a.vdim & 1)) || (a.bias != nullptr && a.bias_rows < 1))
     return hipErrorInvalidValue;
   if (sink_attn_uses_decode(a)) {
     if (a.dim <= 64) return launch_decode_v<8>(a, s);

@@ -399,9 +399,11 @@ class SinkAttentionMixer:
 
     def heads_out(self, p: torch.Tensor, positions: torch.Tensor, meta, cache: torch.Tensor, eps: float,
                   shared: Dict[str, Any], state: Optional[Dict[str, torch.Tensor]] = None,
-                  rag: Optional[seq.Ragged] = None) -> torch.Tensor:
-        """The heads' outputs [T, H * vdim] before gate and output projection, for the same p. ``state`` / ``rag``: the
-        layer's state slots and the step's rows, for a mixer with a convolution."""
+                  rag: Optional[seq.Ragged] = None, gate: Optional[torch.Tensor] = None, mult: float = 1.0,
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """The heads' outputs [T, H * vdim] before the output projection, for the same p. ``state`` / ``rag``: the layer's
+        state slots and the step's rows, for a mixer with a convolution. ``gate`` [T, H]: the raw head gates; the outputs
+        are then (turned back and) gated, times ``mult``, in ``out`` (any row stride)."""
         s = self.spec
         q, k = p[:, : self.nq], p[:, self.nq: self.nq + self.nk]
         v = p[:, self.nq + self.nk: self.nq + self.nk + self.nv] if self.nv else None
@@ -421,7 +423,8 @@ class SinkAttentionMixer:
             rec.conv_tail_update(state["qkv_conv"], p[:, : s.channels], rag)
         return seq.sink_attn(qr, cache, meta.block_tables, meta.cu_q if meta.is_prefill else None, meta.ctx_lens,
                              positions, self.sink, self.bias, meta.max_q_len if meta.is_prefill else 1, s.heads,
-                             s.kv_heads, s.dim, s.vdim, s.window, s.scale, softcap=s.softcap, slopes=self.slopes, seg=s.seg)
+                             s.kv_heads, s.dim, s.vdim, s.window, s.scale, softcap=s.softcap, slopes=self.slopes, seg=s.seg,
+                             gate=gate, out_inv_freq=self.v_inv_freq if gate is not None else None, gate_mult=mult, out=out)
 
     def forward_streams(self, h, positions, meta, cache, eps, state, shared, rag):
         """(y1, y2, a1, a2): the mixer's output is a1 * y1 (+ a2 * y2)."""

@@ -406,9 +406,8 @@ class ScaledPairMixer:
         low = mix.linear(p[:, self.low_cols[0]: self.low_cols[1]], self.w_low)
         nl = s.left.heads * s.left.vdim
         u = torch.empty(h.shape[0], self.w_o.shape[1], dtype=h.dtype, device=h.device)
-        o = l.heads_out(p, positions, meta, cache, eps, shared if shared is not None else {}, state, rag)
-        conv.rot_head_gate(o, p[:, self.gate_at: self.gate_at + s.left.heads], s.left.heads, s.left.vdim, s.left_scale,
-                           positions, l.v_inv_freq, out=u[:, :nl])
+        l.heads_out(p, positions, meta, cache, eps, shared if shared is not None else {}, state, rag,
+                    gate=p[:, self.gate_at: self.gate_at + s.left.heads], mult=s.left_scale, out=u[:, :nl])
         self.right.recur(p, self.at, low, eps, state, rag, s.right_scale, u[:, nl:])
         return mix.linear_partials(u, self.w_o)
 
@@ -619,7 +618,8 @@ class RerozenLM:
         return h
 
     def compute_logits(self, hidden: torch.Tensor, argmax_parts=None) -> torch.Tensor:
-        """fp32 logits [rows, vocab] = head(hidden); the logit scale is already in ``hidden``."""
+        """Logits [rows, vocab] = head(hidden) in the model dtype (what the sampling kernel reads; the logit scale is
+        already in ``hidden``)."""
         if argmax_parts is not None:
             raise ValueError("this head writes no per-tile argmax candidates")
-        return mix.linear(hidden, self.lm_head).float()
+        return mix.linear(hidden, self.lm_head)

@@ -357,23 +357,28 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
               ctx_lens: torch.Tensor, positions: torch.Tensor, sink: Optional[torch.Tensor],
               bias: Optional[torch.Tensor], max_q: int, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
               scale: float, impl: int = 0, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
-              seg: int = 0) -> torch.Tensor:
+              seg: int = 0, gate: Optional[torch.Tensor] = None, out_inv_freq: Optional[torch.Tensor] = None,
+              gate_mult: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Grouped-query attention over the cache that :func:`qkv_prep` writes. The query at position p sees the cached
     positions j <= p with p - j < window (0: all) and, with ``seg`` > 0, of its own segment: floor(j / seg) =
     floor(p / seg). Score: s = (q . k_j) * scale; with ``softcap`` > 0,
     s <- softcap * tanh(s / softcap); then - slopes[h] * (p - j) (``slopes`` [H] fp32, a linear distance penalty)
     and + bias[min(p - j, rows - 1), h]. The softmax denominator has one more term exp(sink[h]) when ``sink`` is
     given. Returns [T, H * vdim]. ``impl``: 0 = the matrix-core kernel where it applies, 1 = the FMA kernel, 2 = the
-    matrix-core kernel or an error."""
+    matrix-core kernel or an error. ``gate`` [T, H] (any row stride): head h's output is turned back by its query's position
+    (``out_inv_freq`` [vdim / 2], as :func:`src.ops.conv.rot_head_gate`) and multiplied by gate_mult * sigmoid(gate[t, h]) —
+    in the launch that writes it for decode steps and split keys, else in one of its own — and ``out`` may be a slice of a
+    wider buffer."""
     T = q.shape[0]
     if q.is_cuda:
-        out = torch.empty(T, heads * vdim, dtype=q.dtype, device=q.device)
+        if out is None:
+            out = torch.empty(T, heads * vdim, dtype=q.dtype, device=q.device)
         _kern().sink_attn(out, q, cache, block_tables, cu_q, ctx_lens, positions, sink, bias, max_q, heads, kv_heads,
-                          dim, vdim, window, scale, impl, float(softcap), slopes, int(seg))
+                          dim, vdim, window, scale, impl, float(softcap), slopes, int(seg), gate, out_inv_freq, float(gate_mult))
         return out
     bs = cache.shape[1]
     hm = _head_major(cache, kv_heads)
-    out = torch.zeros(T, heads, vdim)
+    res = torch.zeros(T, heads, vdim)
     qh = q.float().view(T, heads, dim)
     S = block_tables.shape[0]
     cu = cu_q.tolist() if cu_q is not None else list(range(S + 1))
@@ -403,5 +408,10 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
             if sink is not None:
                 sc = torch.cat([sc, sink[:, None]], 1)
             p = torch.softmax(sc, -1)[:, :n_ctx]
-            out[t] = torch.einsum("hj,jhv->hv", p, vv)
-    return out.reshape(T, heads * vdim).to(q.dtype)
+            res[t] = torch.einsum("hj,jhv->hv", p, vv)
+    res = res.reshape(T, heads * vdim).to(q.dtype)
+    if gate is not None:
+        from .conv import rot_head_gate
+
+        return rot_head_gate(res, gate, heads, vdim, gate_mult, positions, out_inv_freq, out=out)
+    return res if out is None else out.copy_(res)
