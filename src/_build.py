@@ -28,6 +28,8 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 
 KERNELS = ["norm_act", "rope_cache", "attention", "sampling", "moe", "gemm_decode", "decode_step", "allreduce"]
 CONTRACT_ON = {"attention", "gemm_decode"}
+# hipcc only: keeps -O3 from forming packed fp32 instructions out of ordinary float code
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _torch_paths():
@@ -70,7 +72,7 @@ def build_kernels(force: bool = False, jobs: int = 8, verbose: bool = False) -> 
         if force or _newer(obj, [src] + hdrs + [os.path.abspath(__file__)]):
             # the decode kernels fuse multiply-adds per source expression only (not across statements)
             contract = ["-ffp-contract=on"] if k in CONTRACT_ON else []
-            jobs_list.append([HIPCC, f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", *contract, "-I",
+            jobs_list.append([HIPCC, f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", *NO_PACKED_FP32, *contract, "-I",
                               CSRC, "-c", src, "-o", obj])
     bsrc = os.path.join(CSRC, "bindings.cpp")
     bobj = os.path.join(OBJ, "bindings.o")
@@ -97,8 +99,6 @@ def build_kernels(force: bool = False, jobs: int = 8, verbose: bool = False) -> 
 
 MIX_KERNELS = ["mix_ops", "latent_attn", "moe", "seq_mix", "sink_attn", "lin_mix", "rec_mix", "conv_mix"]
 MIX_BINDINGS = ["bindings_mix", "bindings_seq", "bindings_lin", "bindings_rec", "bindings_conv"]
-# hipcc only: keeps -O3 from forming packed fp32 instructions out of ordinary float code
-NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def build_mix(force: bool = False, jobs: int = 8, verbose: bool = False) -> str:
