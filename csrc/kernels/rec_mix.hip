@@ -425,11 +425,11 @@ template <bool F32, bool VEC> __device__ __forceinline__ float4 ld4z(const void*
 // runs a trip's tokens over the staged k and q once more after its columns and reduces the TB dot products n . q over its
 // lanes. (As a column of its own the normaliser would add a ninth wave to workgroups of 512 threads; measured, that ran
 // 1.8x slower than the kernel without it, and a one-wave launch beside it 1.7x.) CD: a decay per row of the state instead
-// of one per head. VEC: dim, vdim, the column offsets and the row strides are multiples of 4.
-template <int LN, int M, bool F32, bool CD, bool VEC>
-__global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs a, RaggedRows r, int VC, int TT) {
+// of one per head. NE: float4s of q (and of k) per thread and trip. VEC: dim, vdim, the column offsets and the row strides are multiples of 4.
+template <int LN, int M, int NE, bool F32, bool CD, bool VEC>
+__global__ void __launch_bounds__(512) gated_linear_attn_kernel(GatedLinearArgs a, RaggedRows r, int VC, int TT) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  constexpr int DPAD = 4 * LN * M, NE = 2, NV = 4;
+  constexpr int DPAD = 4 * LN * M, NV = 4;
   const int d = a.dim, dv = a.vdim, H = a.heads;
   const int vcp = (VC + 3) & ~3;
   float* qs = sm;                  // [TB][DPAD], zero beyond dim
@@ -613,21 +613,27 @@ __global__ void __launch_bounds__(1024) gated_linear_attn_kernel(GatedLinearArgs
   }
 }
 
-template <int LN, int M, bool F32, bool CD, bool VEC> hipError_t launch_gla_one(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
+template <int LN, int M, int NE, bool F32, bool CD, bool VEC> hipError_t launch_gla_ne(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
   const int VC = a.vdim < 128 ? a.vdim : 128;
   const int nvc = (a.vdim + VC - 1) / VC, groups = (VC + 3) / 4;
   const int threads = (LN * groups + 63) / 64 * 64;
-  // tokens per trip: what two float4s of q and k per thread can hold
-  int tt = 2 * threads / (LN * M);
+  // tokens per trip: what NE float4s of q and k per thread can hold
+  int tt = NE * threads / (LN * M);
   tt = tt > TB ? TB : tt;
   const size_t smem = (size_t)((CD ? 3 : 2) * TB * 4 * LN * M + TB * 4 * groups + 2 * TB) * sizeof(float);
-  auto* fn = gated_linear_attn_kernel<LN, M, F32, CD, VEC>;
+  auto* fn = gated_linear_attn_kernel<LN, M, NE, F32, CD, VEC>;
   if (smem > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     if (e != hipSuccess) return e;
   }
   hipLaunchKernelGGL(fn, dim3(a.heads, r.num_seqs, nvc), dim3(threads), smem, s, a, r, VC, tt);
   return hipGetLastError();
+}
+template <int LN, int M, bool F32, bool CD, bool VEC>
+hipError_t launch_gla_one(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
+  // one float4 per thread where that holds 8 tokens or more
+  const int groups = ((a.vdim < 128 ? a.vdim : 128) + 3) / 4;
+  return groups >= 8 * M ? launch_gla_ne<LN, M, 1, F32, CD, VEC>(a, r, s) : launch_gla_ne<LN, M, 2, F32, CD, VEC>(a, r, s);
 }
 template <int LN, int M> hipError_t launch_gla_dp(const GatedLinearArgs& a, RaggedRows r, hipStream_t s) {
   auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };

@@ -634,13 +634,13 @@ template <bool F32, bool VEC> __device__ __forceinline__ float4 ld4z(const void*
 // costs a lane 4 multiply-adds per value and two sums over its group (S^T k and S^T q, on DPP adds); k, q (and with CD
 // the decays) are read from LDS as consecutive float4s, one read per 16 values of the state. Up to TB tokens are staged
 // per trip, the next trip's rows are already in flight; the read-outs of a trip are normed and gated afterwards, one wave
-// per token. CD: a decay per key channel, computed while a trip is staged. VEC: dim, vdim and the row strides are multiples
+// per token. NE: float4s of q (and of k) per thread and trip. CD: a decay per key channel, computed while a trip is staged. VEC: dim, vdim and the row strides are multiples
 // of 4.
-template <int LN, int M, bool F32, bool CD, bool VEC>
-__global__ void __launch_bounds__(1024) gated_delta_kernel(GatedDeltaArgs a, RaggedRows r, int TT) {
+template <int LN, int M, int NE, bool F32, bool CD, bool VEC>
+__global__ void __launch_bounds__(M > 2 && NE == 1 ? 512 : 1024) gated_delta_kernel(GatedDeltaArgs a, RaggedRows r, int TT) {
   const DeltaShape& sh = a.sh;
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  constexpr int DPAD = 4 * LN * M, NE = 2, NV = 4;
+  constexpr int DPAD = 4 * LN * M, NV = 4;
   const int d = sh.dim, dv = sh.vdim, H = sh.heads, G = sh.kv_heads, C = sh.channels();
   const int dvp = (dv + 3) & ~3;
   float* qs = sm;                  // [TB][DPAD], zero beyond dim
@@ -1111,20 +1111,28 @@ hipError_t launch_conv_state_update(float* conv_state, const void* x, int64_t xs
   return hipGetLastError();
 }
 
-template <int LN, int M, bool F32, bool CD, bool VEC> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+template <int LN, int M, int NE, bool F32, bool CD, bool VEC> static hipError_t launch_ne(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
   const int groups = (a.sh.vdim + 3) / 4;
   const int nthr = (LN * groups + 63) / 64 * 64;
-  // tokens per trip: what two float4s of q and k per thread can hold
-  int tt = 2 * nthr / (LN * M);
+  // tokens per trip: what NE float4s of q and k per thread can hold
+  int tt = NE * nthr / (LN * M);
   tt = tt > TB ? TB : tt;
   const size_t lds = sizeof(float) * (TB * ((CD ? 3 : 2) * 4 * LN * M + 2 * 4 * groups) + 2 * TB);
-  auto* fn = gated_delta_kernel<LN, M, F32, CD, VEC>;
+  auto* fn = gated_delta_kernel<LN, M, NE, F32, CD, VEC>;
   if (lds > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
   }
   hipLaunchKernelGGL(fn, dim3(a.sh.heads, r.num_seqs), dim3(nthr), lds, s, a, r, tt);
   return hipGetLastError();
+}
+template <int LN, int M, bool F32, bool CD, bool VEC>
+static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
+  // one float4 per thread where that holds 8 tokens or more (and, for the larger states, the workgroup has at most 512
+  // threads, so that a lane may use 256 registers)
+  const int groups = (a.sh.vdim + 3) / 4;
+  return groups >= 8 * M && (M <= 2 || LN * groups <= 512) ? launch_ne<LN, M, 1, F32, CD, VEC>(a, r, s)
+                                                           : launch_ne<LN, M, 2, F32, CD, VEC>(a, r, s);
 }
 template <int LN, int M> static hipError_t launch_gd(const GatedDeltaArgs& a, RaggedRows r, hipStream_t s) {
   auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
