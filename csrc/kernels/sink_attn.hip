@@ -596,35 +596,28 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
 #pragma unroll
     for (int e = 0; e < 8; ++e) acc[r][e] = 0.f;
 
+  const int bs_shift = (a.block_size & (a.block_size - 1)) == 0 ? __builtin_ctz(a.block_size) : -1;
   for (int j0 = jlo; j0 <= jhi; j0 += DCH) {
-    const int b_lo = j0 / a.block_size;
+    const int b_lo = bs_shift >= 0 ? j0 >> bs_shift : j0 / a.block_size;
     __syncthreads();   // the previous trip's weights and block-table entries are no longer read
     {
       const int nb = min(jhi, j0 + DCH - 1) / a.block_size - b_lo + 1;
       if (tid < nb) btl[tid] = bt[b_lo + tid];
     }
     __syncthreads();
+    // every load is unconditional, so that all of the trip's are in flight together: keys beyond the last repeat it (their
+    // weights are zero), lanes beyond a row's width repeat its start (their query or output columns are not used)
     uint4 kq[NPK], vq[NPV];
+    auto row_at = [&](int j) {
+      const int jc = min(j, jhi);
+      const int jb = bs_shift >= 0 ? jc >> bs_shift : jc / a.block_size;
+      return (((int64_t)btl[jb - b_lo] * G + g) * a.block_size + (jc - jb * a.block_size)) * roww;
+    };
 #pragma unroll
-    for (int u = 0; u < NPK; ++u) {
-      const int j = j0 + u * NG + kg;
-      kq[u] = make_uint4(0, 0, 0, 0);
-      if (j <= jhi && 8 * kl < D) {
-        const int jb = j / a.block_size;
-        kq[u] = *reinterpret_cast<const uint4*>(
-            cache + (((int64_t)btl[jb - b_lo] * G + g) * a.block_size + (j - jb * a.block_size)) * roww + 8 * kl);
-      }
-    }
+    for (int u = 0; u < NPK; ++u) kq[u] = *reinterpret_cast<const uint4*>(cache + row_at(j0 + u * NG + kg) + (8 * kl < D ? 8 * kl : 0));
 #pragma unroll
-    for (int u = 0; u < NPV; ++u) {
-      const int j = j0 + u * NV + vg;
-      vq[u] = make_uint4(0, 0, 0, 0);
-      if (j <= jhi && 8 * vl < DV) {
-        const int jb = j / a.block_size;
-        vq[u] = *reinterpret_cast<const uint4*>(
-            cache + (((int64_t)btl[jb - b_lo] * G + g) * a.block_size + (j - jb * a.block_size)) * roww + D + 8 * vl);
-      }
-    }
+    for (int u = 0; u < NPV; ++u)
+      vq[u] = *reinterpret_cast<const uint4*>(cache + row_at(j0 + u * NV + vg) + D + (8 * vl < DV ? 8 * vl : 0));
 #pragma unroll
     for (int u = 0; u < NPK; ++u) {
       float f[8];
