@@ -471,10 +471,10 @@ __device__ __forceinline__ void conv_rows_of(ConvRow* cr, int64_t row0, int nr, 
   }
   __syncthreads();
 }
-// rows per workgroup: as many as fit 48 KB of LDS (fp32 [R][n]), at most 4; one in a step of one row per sequence
+// rows per workgroup: as many as fit 64 KB of LDS (fp32 [R][n]), at most 4; one in a step of one row per sequence
 static int conv_tile(const RaggedRows& r, int64_t n) {
   if (r.cu_q == nullptr) return 1;
-  const int64_t fit = 48 * 1024 / (4 * n);
+  const int64_t fit = 64 * 1024 / (4 * n);
   return fit >= 4 ? 4 : (fit >= 2 ? 2 : 1);
 }
 // the same for one channel; wc / wj: strides of the weight's channel and tap
