@@ -41,13 +41,19 @@ const float* f32_vec(const OptTensor& t, int64_t n, const char* name) {
   return t->data_ptr<float>();
 }
 
-void conv_norm(Tensor h, Tensor resid_in, OptTensor resid_out, OptTensor y, Tensor w, double eps, OptTensor conv_wt,
+void conv_norm(Tensor h, OptTensor resid_in, OptTensor resid_out, OptTensor y, OptTensor w, double eps, OptTensor conv_wt,
                OptTensor conv_state, int64_t max_q, OptTensor positions, OptTensor cu_q, OptTensor state_slots) {
-  check_c(resid_in, at::kFloat, "resid_in");
-  TORCH_CHECK(resid_in.dim() == 2, "resid_in [T, W]");
-  const int64_t T = resid_in.size(0), W = resid_in.size(1);
+  check_rows(h, "h");
+  const int64_t T = h.size(0), W = h.size(1);
+  TORCH_CHECK(resid_in.has_value() || y.has_value(), "resid_in or y");
+  TORCH_CHECK(!conv_wt.has_value() || (w.has_value() && resid_in.has_value()), "a convolution runs over the normed residual");
   die::ConvNormArgs a;
-  a.resid_in = resid_in.data_ptr<float>();
+  a.resid_in = nullptr;
+  if (resid_in.has_value()) {
+    check_c(*resid_in, at::kFloat, "resid_in");
+    TORCH_CHECK(resid_in->sizes() == h.sizes(), "resid_in [T, W]");
+    a.resid_in = resid_in->data_ptr<float>();
+  }
   a.resid_out = nullptr;
   a.y = nullptr;
   a.ystride = 0;
@@ -67,17 +73,19 @@ void conv_norm(Tensor h, Tensor resid_in, OptTensor resid_out, OptTensor y, Tens
       TORCH_CHECK(y->size(0) == T && y->size(1) == W, "y [T, W]");
       a.ystride = y->stride(0);
     }
-    TORCH_CHECK(resid_out.has_value(), "y needs resid_out");
-    check_c(*resid_out, at::kFloat, "resid_out");
-    TORCH_CHECK(resid_out->sizes() == resid_in.sizes(), "resid_out like resid_in");
+    TORCH_CHECK(resid_out.has_value() || !conv_wt.has_value(), "y needs resid_out");
     a.y = y->data_ptr();
-    a.resid_out = resid_out->data_ptr<float>();
+    if (resid_out.has_value()) {
+      check_c(*resid_out, at::kFloat, "resid_out");
+      TORCH_CHECK(resid_out->sizes() == h.sizes(), "resid_out [T, W]");
+      a.resid_out = resid_out->data_ptr<float>();
+    }
   }
   a.w = f32_vec(w, W, "w");
   a.eps = (float)eps;
   a.h_f32 = is_f32(h, "h");
-  TORCH_CHECK(h.is_contiguous() && h.sizes() == resid_in.sizes(), "h [T, W] contiguous");
   a.h = h.data_ptr();
+  a.hstride = h.stride(0);
   a.W = (int)W;
   a.max_q = (int)max_q;
   a.conv_wt = nullptr;

@@ -88,6 +88,61 @@ void gelu_act(Tensor out, Tensor z) {
   HIP_OK(die::launch_gelu_act(out.data_ptr(), z.data_ptr(), f, z.numel(), cur_stream()));
 }
 
+void relu2_act(Tensor out, Tensor z) {
+  const bool f = is_f32(z, "z");
+  TORCH_CHECK(is_f32(out, "out") == f && out.is_contiguous() && z.is_contiguous() && out.sizes() == z.sizes(),
+              "relu2_act: same dtype and shape, contiguous");
+  HIP_OK(die::launch_relu2_act(out.data_ptr(), z.data_ptr(), f, z.numel(), cur_stream()));
+}
+
+const float* opt_f32(const OptTensor& t, int64_t n, const char* name) {
+  if (!t.has_value()) return nullptr;
+  check_i(*t, at::kFloat, name);
+  TORCH_CHECK(t->numel() == n, name, ": expected ", n, " values");
+  return t->data_ptr<float>();
+}
+
+void embed_norm(Tensor resid, OptTensor copy, Tensor embed, Tensor ids, OptTensor w, double eps) {
+  const bool f = is_f32(embed, "embed");
+  check_i(resid, at::kFloat, "resid");
+  check_i(ids, at::kLong, "ids");
+  TORCH_CHECK(resid.dim() == 2 && embed.dim() == 2 && embed.is_contiguous() && embed.size(1) == resid.size(1),
+              "resid [T, W], embed [V, W]");
+  const int64_t T = resid.size(0), W = resid.size(1);
+  TORCH_CHECK(ids.numel() >= T, "ids [T]");
+  void* cp = nullptr;
+  int64_t cs = 0;
+  if (copy.has_value()) {
+    check_rows(*copy, "copy");
+    TORCH_CHECK(is_f32(*copy, "copy") == f && copy->sizes() == resid.sizes(), "copy: the table's dtype, the residual's shape");
+    cp = copy->data_ptr();
+    cs = copy->stride(0);
+  }
+  HIP_OK(die::launch_embed_norm(resid.data_ptr<float>(), cp, cs, embed.data_ptr(), f, ids.data_ptr<int64_t>(),
+                                opt_f32(w, W, "w"), (float)eps, (int)T, (int)W, cur_stream()));
+}
+
+void route_grouped_topk(Tensor w, Tensor ids, Tensor x, Tensor wr, int64_t count, int64_t keep, double scale) {
+  check_rows(x, "x");
+  const bool xf = is_f32(x, "x"), wf = is_f32(wr, "wr");
+  check_i(w, at::kFloat, "w");
+  check_i(ids, at::kInt, "ids");
+  TORCH_CHECK(wr.dim() == 2 && wr.is_contiguous() && wr.size(1) == x.size(1), "wr [E, H]");
+  TORCH_CHECK(w.dim() == 2 && w.size(0) == x.size(0) && ids.sizes() == w.sizes(), "w, ids [T, K]");
+  HIP_OK(die::launch_route_grouped_topk(w.data_ptr<float>(), ids.data_ptr<int>(), x.data_ptr(), x.stride(0), xf,
+                                        wr.data_ptr(), wf, (int)x.size(0), (int)x.size(1), (int)wr.size(0),
+                                        (int)w.size(1), (int)count, (int)keep, (float)scale, cur_stream()));
+}
+
+void topk_grouped(Tensor w, Tensor ids, Tensor z, int64_t count, int64_t keep, double scale) {
+  check_i(w, at::kFloat, "w");
+  check_i(ids, at::kInt, "ids");
+  check_i(z, at::kFloat, "z");
+  TORCH_CHECK(z.dim() == 2 && w.dim() == 2 && w.size(0) == z.size(0) && ids.sizes() == w.sizes(), "z [T, E]; w, ids [T, K]");
+  HIP_OK(die::launch_topk_grouped(w.data_ptr<float>(), ids.data_ptr<int>(), z.data_ptr<float>(), (int)z.size(0),
+                                  (int)z.size(1), (int)w.size(1), (int)count, (int)keep, (float)scale, cur_stream()));
+}
+
 void route_sigmoid_topk(Tensor w, Tensor ids, Tensor x, Tensor wr) {
   check_rows(x, "x");
   const bool xf = is_f32(x, "x"), wf = is_f32(wr, "wr");
@@ -132,13 +187,6 @@ void gather_scaled(Tensor xs, Tensor x, OptTensor sorted, OptTensor w, int64_t t
                                    (int)topk, (int)x.size(1), cur_stream()));
 }
 
-const float* opt_f32(const OptTensor& t, int64_t n, const char* name) {
-  if (!t.has_value()) return nullptr;
-  check_i(*t, at::kFloat, name);
-  TORCH_CHECK(t->numel() == n, name, ": expected ", n, " values");
-  return t->data_ptr<float>();
-}
-
 void route_softmax_topk(Tensor w, Tensor ids, OptTensor gate, Tensor x, Tensor wr, int64_t n_route, OptTensor corr) {
   check_rows(x, "x");
   const bool xf = is_f32(x, "x"), wf = is_f32(wr, "wr");
@@ -169,9 +217,16 @@ void topk_softmax_corrected(Tensor w, Tensor ids, OptTensor gate, Tensor z, int6
                                             (int)n_route, (int)w.size(1), cur_stream()));
 }
 
-void combine_weighted(OptTensor out, OptTensor resid, OptTensor act, Tensor ys, OptTensor pos, Tensor x, Tensor wk,
-                      Tensor ids, int64_t num_experts, OptTensor extra, OptTensor gate, OptTensor w, bool unit_offset,
-                      double eps, double mult) {
+// what both forms of the weighted expert sum read
+struct ExpertSum {
+  bool f;
+  int64_t T, H, K;
+  const int* pos;
+  const void* extra;
+  const float* gate;
+};
+ExpertSum expert_sum(const Tensor& ys, const OptTensor& pos, const Tensor& x, const Tensor& wk, const Tensor& ids,
+                     int64_t num_experts, const OptTensor& extra, const OptTensor& gate) {
   const bool f = is_f32(x, "x");
   TORCH_CHECK(x.dim() == 2 && x.is_contiguous(), "x [T, H] contiguous");
   const int64_t T = x.size(0), H = x.size(1);
@@ -196,6 +251,15 @@ void combine_weighted(OptTensor out, OptTensor resid, OptTensor act, Tensor ys, 
     ep = extra->data_ptr();
   }
   TORCH_CHECK(!gate.has_value() || extra.has_value(), "gate without extra");
+  return {f, T, H, K, pp, ep, opt_f32(gate, T, "gate")};
+}
+
+void combine_weighted(OptTensor out, OptTensor resid, OptTensor act, Tensor ys, OptTensor pos, Tensor x, Tensor wk,
+                      Tensor ids, int64_t num_experts, OptTensor extra, OptTensor gate, OptTensor w, bool unit_offset,
+                      double eps, double mult) {
+  const ExpertSum e = expert_sum(ys, pos, x, wk, ids, num_experts, extra, gate);
+  const bool f = e.f;
+  const int64_t T = e.T, H = e.H;
   float* op = nullptr;
   if (out.has_value()) {
     check_i(*out, at::kFloat, "out");
@@ -220,9 +284,30 @@ void combine_weighted(OptTensor out, OptTensor resid, OptTensor act, Tensor ys, 
     }
   }
   TORCH_CHECK(op != nullptr || rp != nullptr, "out or resid");
-  HIP_OK(die::launch_combine_weighted(op, rp, ap, ys.data_ptr(), f, pp, x.data_ptr(), wk.data_ptr<float>(),
-                                      ids.data_ptr<int>(), (int)num_experts, ep, opt_f32(gate, T, "gate"), (int)T,
-                                      (int)K, (int)H, wp, wf, unit_offset, (float)eps, (float)mult, cur_stream()));
+  HIP_OK(die::launch_combine_weighted(op, rp, ap, ys.data_ptr(), f, e.pos, x.data_ptr(), wk.data_ptr<float>(),
+                                      ids.data_ptr<int>(), (int)num_experts, e.extra, e.gate, (int)T, (int)e.K, (int)H, wp,
+                                      wf, unit_offset, (float)eps, (float)mult, cur_stream()));
+}
+
+void combine_pre_norm(Tensor resid, Tensor act, Tensor ys, OptTensor pos, Tensor x, Tensor wk, Tensor ids,
+                      int64_t num_experts, OptTensor extra, OptTensor gate, OptTensor w, bool unit_offset, double eps,
+                      double mult) {
+  const ExpertSum e = expert_sum(ys, pos, x, wk, ids, num_experts, extra, gate);
+  check_i(resid, at::kFloat, "resid");
+  TORCH_CHECK(resid.dim() == 2 && resid.size(0) == e.T && resid.size(1) == e.H, "resid [T, H]");
+  check_rows(act, "act");
+  TORCH_CHECK(is_f32(act, "act") == e.f && act.sizes() == resid.sizes(), "act: x's dtype, the residual's shape");
+  const void* wp = nullptr;
+  bool wf = false;
+  if (w.has_value()) {
+    wf = is_f32(*w, "w");
+    TORCH_CHECK(w->is_contiguous() && w->numel() == e.H, "w [H]");
+    wp = w->data_ptr();
+  }
+  HIP_OK(die::launch_combine_pre_norm(resid.data_ptr<float>(), act.data_ptr(), act.stride(0), ys.data_ptr(), e.f, e.pos,
+                                      x.data_ptr(), wk.data_ptr<float>(), ids.data_ptr<int>(), (int)num_experts, e.extra,
+                                      e.gate, (int)e.T, (int)e.K, (int)e.H, wp, wf, unit_offset, (float)eps, (float)mult,
+                                      cur_stream()));
 }
 
 void combine_sum(Tensor out, Tensor ys, OptTensor pos, OptTensor extra, int64_t topk) {
@@ -442,6 +527,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route_softmax_topk", &route_softmax_topk);
   m.def("topk_softmax_corrected", &topk_softmax_corrected);
   m.def("combine_weighted", &combine_weighted);
+  m.def("combine_pre_norm", &combine_pre_norm);
+  m.def("embed_norm", &embed_norm);
+  m.def("relu2_act", &relu2_act);
+  m.def("route_grouped_topk", &route_grouped_topk);
+  m.def("topk_grouped", &topk_grouped);
   m.def("rms_norm_ext", &rms_norm_ext);
   m.def("post_norm_residual", &post_norm_residual);
   m.def("gated_act", &gated_act);

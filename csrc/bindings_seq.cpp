@@ -357,8 +357,12 @@ void qkv_prep(Tensor q_out, Tensor cache, Tensor q, Tensor k, OptTensor v, int64
 void sink_attn(Tensor out, Tensor q, Tensor cache, Tensor block_tables, OptTensor cu_q, Tensor ctx_lens,
                Tensor positions, OptTensor sink, OptTensor bias, int64_t max_q, int64_t heads, int64_t kv_heads,
                int64_t dim, int64_t vdim, int64_t window, double scale, int64_t impl, double softcap,
-               OptTensor slopes, int64_t seg, OptTensor gate, OptTensor out_inv_freq, double gate_mult) {
+               OptTensor slopes, int64_t seg, OptTensor gate, OptTensor out_inv_freq, double gate_mult, bool sigmoid,
+               OptTensor head_bias) {
   die::SinkAttnArgs a;
+  TORCH_CHECK(sigmoid ? !sink.has_value() : !head_bias.has_value(), "a sink goes with softmax, a head bias with sigmoid weights");
+  a.sigmoid = sigmoid;
+  a.head_bias = f32_ptr(head_bias, heads, "head_bias");
   a.f32 = is_f32(q, "q");
   TORCH_CHECK(is_f32(out, "out") == a.f32 && is_f32(cache, "cache") == a.f32, "one dtype");
   TORCH_CHECK(q.dim() == 2 && q.is_contiguous() && q.size(1) == heads * dim, "q [T, H * dim] contiguous");

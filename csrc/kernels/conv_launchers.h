@@ -13,20 +13,21 @@
 namespace die {
 
 struct ConvNormArgs {
-  const float* resid_in;   // [T, W]
-  float* resid_out;        // [T, W]: resid_in + y; not written without y. May equal resid_in only where no other row
-                           // reads the row: without a convolution, or with one row per sequence
+  const float* resid_in;   // [T, W], or nullptr: zeros (x = y)
+  float* resid_out;        // [T, W]: resid_in + y; not written without y, or nullptr: not kept. May equal resid_in only
+                           // where no other row reads the row: without a convolution, or with one row per sequence
   const void* y;           // [T, W], row stride ystride, or nullptr
   int64_t ystride;
   bool y_f32;
   int yslabs;              // fp32 y as the sum of this many partial sums, yslab elements apart (else 1)
   int64_t yslab;
-  const float* w;          // [W]
+  const float* w;          // [W], or nullptr: no norm, n = x (without a convolution)
   float eps;
   const float* conv_wt;    // [taps, W], tap-major, the current row's weights last; nullptr: no convolution
   float* conv_state;       // [slots, taps - 1, W]: the last normed rows before the step, the most recent last
   int taps;
-  void* h;                 // [T, W]
+  void* h;                 // [T, W], row stride hstride
+  int64_t hstride;
   bool h_f32;
   int W, max_q;            // max_q: most rows of one sequence in this step
 };

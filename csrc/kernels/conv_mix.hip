@@ -1,7 +1,8 @@
 // Kernels for layers whose sublayers read a convolved input (gfx950). Storage of activations is bf16 or fp32, arithmetic
 // is fp32; the residual, the norms and the convolution's rows and state are fp32 in both modes.
 //
-//   conv_norm        residual sum, RMS norm and the causal convolution over the normed rows, one launch
+//   conv_norm        residual sum, RMS norm and the causal convolution over the normed rows, one launch (any of the three
+//                    may be absent)
 //   rot_head_gate    attention output turned back by the query's position, sigmoid gate per head, scale
 #include "common.h"
 #include "conv_launchers.h"
@@ -117,7 +118,12 @@ __global__ void __launch_bounds__(NT) conv_norm_kernel(ConvNormArgs a, RaggedRow
     for (int t = 0; t < TR; ++t) {
       const int c = VEC * (t * NT + tid);
       if (c < W) {
-        nx[t] = ldf<VEC>(a.resid_in + row * W + c);
+        if (a.resid_in != nullptr) {
+          nx[t] = ldf<VEC>(a.resid_in + row * W + c);
+        } else {
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) nx[t].v[e] = 0.f;
+        }
         if (a.y != nullptr) ny[t] = ldy<VEC, YF32>(a, row * a.ystride + c);
       }
     }
@@ -136,23 +142,28 @@ __global__ void __launch_bounds__(NT) conv_norm_kernel(ConvNormArgs a, RaggedRow
         if (a.y != nullptr) {
 #pragma unroll
           for (int e = 0; e < VEC; ++e) x[t].v[e] += ny[t].v[e];
-          if (own) stf<VEC>(a.resid_out + row * W + c, x[t]);
+          if (own && a.resid_out != nullptr) stf<VEC>(a.resid_out + row * W + c, x[t]);
         }
 #pragma unroll
         for (int e = 0; e < VEC; ++e) ss += x[t].v[e] * x[t].v[e];
       }
     }
     if (n + 1 < n1 + n2) load(n + 1);
-    ss = block_sum<NT>(ss, red);
-    const float rs = 1.0f / sqrtf(ss / (float)W + a.eps);
+    float rs = 1.0f;
+    if (a.w != nullptr) {
+      ss = block_sum<NT>(ss, red);
+      rs = 1.0f / sqrtf(ss / (float)W + a.eps);
+    }
     const int64_t p = p0 + i;
 #pragma unroll
     for (int t = 0; t < TR; ++t) {
       const int c = VEC * (t * NT + tid);
       if (c >= W) continue;
-      const Vals<VEC> w = ldf<VEC>(a.w + c);
+      if (a.w != nullptr) {
+        const Vals<VEC> w = ldf<VEC>(a.w + c);
 #pragma unroll
-      for (int e = 0; e < VEC; ++e) x[t].v[e] *= rs * w.v[e];
+        for (int e = 0; e < VEC; ++e) x[t].v[e] *= rs * w.v[e];
+      }
       if (own) {
         Vals<VEC> o = x[t];
         if (a.conv_wt != nullptr) {
@@ -168,7 +179,7 @@ __global__ void __launch_bounds__(NT) conv_norm_kernel(ConvNormArgs a, RaggedRow
             for (int e = 0; e < VEC; ++e) o.v[e] += wb.v[e] * past.v[e];
           }
         }
-        sta<VEC>(a.h, row * W + c, a.h_f32, o);
+        sta<VEC>(a.h, row * a.hstride + c, a.h_f32, o);
       }
       if (H > 0) stf<VEC>(ring + (i % H) * W + c, x[t]);
     }
@@ -234,7 +245,10 @@ __global__ void __launch_bounds__(NTH) conv_norm_reg_kernel(ConvNormArgs a, Ragg
 #pragma unroll
       for (int t = 0; t < TR; ++t) {
         const int c = min(4 * (t * NTH + tid), W - 4);
-        nx[b][t] = ldf<4>(a.resid_in + row * W + c);
+        if (a.resid_in != nullptr)
+          nx[b][t] = ldf<4>(a.resid_in + row * W + c);
+        else
+          nx[b][t].v[0] = nx[b][t].v[1] = nx[b][t].v[2] = nx[b][t].v[3] = 0.f;
         if (has_y) ny[b][t] = ldy<4, YF32>(a, row * a.ystride + c);
       }
     }
@@ -247,7 +261,10 @@ __global__ void __launch_bounds__(NTH) conv_norm_reg_kernel(ConvNormArgs a, Ragg
 #pragma unroll
   for (int t = 0; t < TR; ++t) {
     const int c = min(4 * (t * NTH + tid), W - 4);
-    w[t] = ldf<4>(a.w + c);
+    if (a.w != nullptr)
+      w[t] = ldf<4>(a.w + c);
+    else
+      w[t].v[0] = w[t].v[1] = w[t].v[2] = w[t].v[3] = 1.0f;
 #pragma unroll
     for (int b = 0; b <= H; ++b) {   // cw[b]: weights of the row b back
       if (conv) cw[b][t] = ldf<4>(a.conv_wt + (int64_t)(H - b) * W + c);
@@ -277,7 +294,7 @@ __global__ void __launch_bounds__(NTH) conv_norm_reg_kernel(ConvNormArgs a, Ragg
         if (has_y) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) x[b][t].v[e] += ny[b][t].v[e];
-          if (own && c < W) stf<4>(a.resid_out + (int64_t)(q0 + i) * W + c, x[b][t]);
+          if (own && c < W && a.resid_out != nullptr) stf<4>(a.resid_out + (int64_t)(q0 + i) * W + c, x[b][t]);
         }
         if (c < W) {
 #pragma unroll
@@ -302,7 +319,7 @@ __global__ void __launch_bounds__(NTH) conv_norm_reg_kernel(ConvNormArgs a, Ragg
       float tot = 0.f;
 #pragma unroll
       for (int k = 0; k < NW; ++k) tot += red[buf][b][k];
-      const float rs = 1.0f / sqrtf(tot / (float)W + a.eps);
+      const float rs = a.w != nullptr ? 1.0f / sqrtf(tot / (float)W + a.eps) : 1.0f;
 #pragma unroll
       for (int t = 0; t < TR; ++t) {
         const int c = 4 * (t * NTH + tid);
@@ -318,7 +335,7 @@ __global__ void __launch_bounds__(NTH) conv_norm_reg_kernel(ConvNormArgs a, Ragg
               for (int k = 0; k < H; ++k) o.v[e] += cw[k + 1][t].v[e] * past[k][t].v[e];
             }
           }
-          sta<4>(a.h, (int64_t)(q0 + i) * W + c, a.h_f32, o);
+          sta<4>(a.h, (int64_t)(q0 + i) * a.hstride + c, a.h_f32, o);
         }
 #pragma unroll
         for (int k = H - 1; k > 0; --k) past[k][t] = past[k - 1][t];
@@ -427,7 +444,9 @@ hipError_t launch_conv_norm(const ConvNormArgs& a, RaggedRows r0, hipStream_t s)
   RaggedRows r = r0;
   if (r.total_rows == 0 || r.num_seqs == 0) return hipSuccess;
   const bool conv = a.conv_wt != nullptr;
-  if (a.W < 1 || a.w == nullptr || a.h == nullptr || (a.y != nullptr && (a.resid_out == nullptr || a.yslabs < 1 || (a.yslabs > 1 && !a.y_f32))))
+  if (a.W < 1 || a.h == nullptr || a.hstride < a.W || (a.y == nullptr && a.resid_in == nullptr) ||
+      (conv && (a.w == nullptr || a.resid_in == nullptr || (a.y != nullptr && a.resid_out == nullptr))) ||
+      (a.y != nullptr && (a.yslabs < 1 || (a.yslabs > 1 && !a.y_f32))))
     return hipErrorInvalidValue;
   if (conv && (a.taps < 1 || a.taps > TAPS_MAX || r.positions == nullptr || r.state_slots == nullptr || a.max_q < 1 ||
                (a.taps > 1 && a.conv_state == nullptr)))
@@ -448,7 +467,7 @@ hipError_t launch_conv_norm(const ConvNormArgs& a, RaggedRows r0, hipStream_t s)
     if (a.y != nullptr && tiles > 1 && a.resid_out == a.resid_in) return hipErrorInvalidValue;
   }
   if ((int64_t)tiles * r.num_seqs > 0x7fffffff) return hipErrorInvalidValue;
-  const bool vec = a.W % 4 == 0 && a16(a.resid_in) && a16(a.w) && a16(a.h) && (!conv || (a16(a.conv_wt) && a16(a.conv_state))) &&
+  const bool vec = a.W % 4 == 0 && a.hstride % 4 == 0 && a16(a.resid_in) && a16(a.w) && a16(a.h) && (!conv || (a16(a.conv_wt) && a16(a.conv_state))) &&
                    (a.y == nullptr || (a16(a.resid_out) && a16(a.y) && a.ystride % 4 == 0 && (a.yslabs == 1 || a.yslab % 4 == 0)));
   if (vec && a.W <= 8192 && (!conv || a.taps <= 4))
     return r.cu_q != nullptr ? launch_cr<CONV_RB>(a, r, R, tiles, s) : launch_cr<1>(a, r, R, tiles, s);

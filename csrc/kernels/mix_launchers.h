@@ -25,6 +25,12 @@ hipError_t launch_gated_act(void* out, const void* gu, bool f32, int rows, int f
 
 // out[i] = 0.5 z[i] (1 + erf(z[i] / sqrt 2)), n contiguous elements
 hipError_t launch_gelu_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s);
+// out[i] = max(z[i], 0)^2
+hipError_t launch_relu2_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s);
+// resid[t] (fp32 [T, W]) = rmsnorm(embed[ids[t]]) * w (fp32 [W] or nullptr); copy[t] (optional, row stride cstride, the
+// table's type) = the same
+hipError_t launch_embed_norm(float* resid, void* copy, int64_t cstride, const void* embed, bool f32, const int64_t* ids,
+                             const float* w, float eps, int T, int W, hipStream_t s);
 
 // Router: z = x . Wr[e] in fp32, score = sigmoid(z), the K largest per token (lowest index on ties);
 // w [T, K] fp32 = the chosen scores (not renormalised), ids [T, K] int32
@@ -38,13 +44,28 @@ hipError_t launch_topk_sigmoid(float* w, int* ids, const float* z, int T, int E,
 hipError_t launch_route_softmax_topk(float* w, int* ids, float* gate, const void* x, int64_t xstride, bool x_f32,
                                      const void* wr, bool wr_f32, const float* corr, int T, int H, int E, int K,
                                      hipStream_t s);
-// the same selection from fp32 logits z [T, zstride] computed elsewhere (the gate's logit at column E)
+// Router with softmax scores and group-limited choice: z = x . Wr[e] in fp32, s = softmax(z) over all E; experts form
+// `count` equal groups of neighbours, only those of the `keep` groups with the largest single score are open; the K
+// largest open scores are chosen (lowest index on ties), w [T, K] = scale * s, not renormalised.
+hipError_t launch_route_grouped_topk(float* w, int* ids, const void* x, int64_t xstride, bool x_f32, const void* wr,
+                                     bool wr_f32, int T, int H, int E, int K, int count, int keep, float scale,
+                                     hipStream_t s);
+// the same selection from fp32 logits z [T, E] computed elsewhere
+hipError_t launch_topk_grouped(float* w, int* ids, const float* z, int T, int E, int K, int count, int keep, float scale,
+                               hipStream_t s);
+// the softmax selection from fp32 logits z [T, zstride] computed elsewhere (the gate's logit at column E)
 hipError_t launch_topk_softmax_corrected(float* w, int* ids, float* gate, const float* z, int zstride,
                                          const float* corr, int T, int E, int K, hipStream_t s);
 // sum[t] = sum_k wk[t, k] * (ids[t, k] < E ? ys[pos[t * K + k]] : x[t]) + gate[t] * extra[t]  (pos == nullptr:
 // t * K + k; extra, gate optional). out != nullptr: out[t] (fp32) = sum[t]. resid != nullptr:
 // resid[t] += mult * rmsnorm(sum[t]) * (w or 1 + w), act[t] (optional, the activation type) = resid[t].
 hipError_t launch_combine_weighted(float* out, float* resid, void* act, const void* ys, bool f32, const int* pos,
+                                   const void* x, const float* wk, const int* ids, int E, const void* extra,
+                                   const float* gate, int T, int K, int H, const void* w, bool w_f32, bool unit_offset,
+                                   float eps, float mult, hipStream_t s);
+// resid[t] (fp32) += mult * sum[t] as above; act[t] (the activation type, row stride astride) = rmsnorm(resid[t]) *
+// (w or 1 + w), or without w a copy of resid[t]
+hipError_t launch_combine_pre_norm(float* resid, void* act, int64_t astride, const void* ys, bool f32, const int* pos,
                                    const void* x, const float* wk, const int* ids, int E, const void* extra,
                                    const float* gate, int T, int K, int H, const void* w, bool w_f32, bool unit_offset,
                                    float eps, float mult, hipStream_t s);

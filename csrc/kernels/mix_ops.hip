@@ -4,9 +4,11 @@
 //
 //   rms_norm_ext          y = x / sqrt(mean(x^2) + eps) * (w | 1 + w)
 //   post_norm_residual    resid(fp32) += rmsnorm(y) * (w | 1 + w); optional bf16 copy of the new residual
-//   gelu_act              0.5 z (1 + erf(z / sqrt 2))
+//   embed_norm            rmsnorm(embed[id]) * w into the fp32 residual and a copy in the activation type
+//   gelu_act, relu2_act   0.5 z (1 + erf(z / sqrt 2)), relu(z)^2
 //   gated_act             silu(g) * u, or the clamped variant g' * sigmoid(alpha g') * (u' + 1)
 //   route_sigmoid_topk    router logits (fp32), sigmoid scores, top-K without renormalisation
+//   route_grouped_topk    softmax scores, top-K among the experts of the best groups, scores times a constant
 //   gather_scaled         expert input rows scaled by their routing weight
 //   combine_sum           per-token sum of its experts' outputs (+ a shared expert), fp32
 //   latent_kv_write       compressed-KV cache row: normalised latent | rotated shared key part
@@ -53,6 +55,43 @@ __global__ void __launch_bounds__(NT) rms_norm_ext_kernel(void* out, int64_t ost
 }
 
 __device__ __forceinline__ bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+
+// resid[t] (fp32) = rmsnorm(embed[ids[t]]) * w (fp32 weights; nullptr: the plain vectors' norm), copy[t] (optional, the
+// table's type, row stride cstride) = the same
+__global__ void __launch_bounds__(NT) embed_norm_kernel(float* resid, void* copy, int64_t cstride, const void* embed,
+                                                       bool f32, const int64_t* ids, const float* w, float eps, int W) {
+  __shared__ float red[NT / 64];
+  const int64_t t = blockIdx.x, base = ids[t] * (int64_t)W;
+  if (!f32 && W % 8 == 0 && cstride % 8 == 0 && aligned16(embed) && aligned16(resid) && aligned16(w) && aligned16(copy)) {
+    const uint4* er = reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(embed) + base);
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < W / 8; c += NT) {
+      float f[8];
+      unpack8(er[c], f);
+#pragma unroll
+      for (int q = 0; q < 8; ++q) ss += f[q] * f[q];
+    }
+    ss = block_sum<NT>(ss, red);
+    const float rs = 1.0f / sqrtf(ss / (float)W + eps);
+    float4* rr = reinterpret_cast<float4*>(resid + t * W);
+    for (int c = threadIdx.x; c < W / 8; c += NT) {
+      float f[8];
+      unpack8(er[c], f);
+#pragma unroll
+      for (int q = 0; q < 8; ++q) f[q] *= w != nullptr ? rs * w[8 * c + q] : rs;
+      rr[2 * c] = make_float4(f[0], f[1], f[2], f[3]);
+      rr[2 * c + 1] = make_float4(f[4], f[5], f[6], f[7]);
+      if (copy) reinterpret_cast<uint4*>(reinterpret_cast<bf16_t*>(copy) + t * cstride)[c] = pack8(f);
+    }
+    return;
+  }
+  const float rs = row_rs(embed, base, f32, W, eps, red);
+  for (int c = threadIdx.x; c < W; c += NT) {
+    const float v = ldv(embed, base + c, f32) * (w != nullptr ? rs * w[c] : rs);
+    resid[t * W + c] = v;
+    if (copy) stv(copy, t * cstride + c, f32, v);
+  }
+}
 
 __global__ void __launch_bounds__(NT) post_norm_residual_kernel(float* resid, void* act, const void* y,
                                                                int64_t ystride, bool y_f32, const void* w, bool w_f32,
@@ -129,20 +168,36 @@ __global__ void __launch_bounds__(NT) gated_act_kernel(void* out, const void* gu
 // the exact (erf) GELU
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
+// an activation of one argument: the exact GELU or relu(z)^2
+constexpr int ACT1_GELU = 0, ACT1_RELU2 = 1;
+template <int KIND> __device__ __forceinline__ float act1(float z) {
+  if constexpr (KIND == ACT1_RELU2) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  }
+  return gelu_erf(z);
+}
+
 // grid-stride over the flattened tensor; bf16 with a multiple of 8 elements: 16 bytes per access
-__global__ void __launch_bounds__(NT) gelu_act_kernel(void* out, const void* z, bool f32, int64_t n) {
+template <int KIND> __global__ void __launch_bounds__(NT) act1_kernel(void* out, const void* z, bool f32, int64_t n) {
   const int64_t stride = (int64_t)gridDim.x * NT, i0 = (int64_t)blockIdx.x * NT + threadIdx.x;
   if (!f32 && n % 8 == 0 && aligned16(z) && aligned16(out)) {
     for (int64_t c = i0; c < n / 8; c += stride) {
       float v[8];
       unpack8(reinterpret_cast<const uint4*>(z)[c], v);
 #pragma unroll
-      for (int q = 0; q < 8; ++q) v[q] = gelu_erf(v[q]);
+      for (int q = 0; q < 8; ++q) v[q] = act1<KIND>(v[q]);
       reinterpret_cast<uint4*>(out)[c] = pack8(v);
     }
     return;
   }
-  for (int64_t c = i0; c < n; c += stride) stv(out, c, f32, gelu_erf(ldv(z, c, f32)));
+  for (int64_t c = i0; c < n; c += stride) stv(out, c, f32, act1<KIND>(ldv(z, c, f32)));
+}
+template <int KIND> hipError_t launch_act1(void* out, const void* z, bool f32, int64_t n, hipStream_t s) {
+  if (n == 0) return hipSuccess;
+  const int64_t blocks = (n / (f32 ? 1 : 8) + NT - 1) / NT + 1;
+  hipLaunchKernelGGL((act1_kernel<KIND>), dim3((unsigned)(blocks < 16384 ? blocks : 16384)), dim3(NT), 0, s, out, z, f32, n);
+  return hipGetLastError();
 }
 
 constexpr int ROUTE_E_MAX = 256;
@@ -309,6 +364,144 @@ __device__ __forceinline__ void softmax_select(const float* z, float* sc, const 
   for (int k = 0; k < K; ++k) w_out[k] *= rn;
 }
 
+// ---- softmax scores with group-limited choice: one wave selects, GE experts per lane
+constexpr int GROUP_E_MAX = 512;
+constexpr int GE = GROUP_E_MAX / 64;
+
+// the larger of all lanes' keys (every lane receives it)
+__device__ __forceinline__ uint64_t wave_max_key(uint64_t k) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const uint64_t other = ((uint64_t)(uint32_t)__shfl_xor((int)(k >> 32), o, 64) << 32) | (uint32_t)__shfl_xor((int)(uint32_t)k, o, 64);
+    k = other > k ? other : k;
+  }
+  return k;
+}
+// scores are >= 0, so their bits are ordered; the smaller index wins a tie; 0: no candidate
+__device__ __forceinline__ uint64_t score_key(float s, int i) {
+  return ((uint64_t)__float_as_uint(s) << 32) | (uint32_t)(0x7fffffff - i);
+}
+__device__ __forceinline__ int key_index(uint64_t k, int n) { return k == 0 ? 0 : min(0x7fffffff - (int)(uint32_t)k, n - 1); }
+
+// z [E] -> s = softmax(z); of `count` equal groups of neighbouring experts the `keep` with the largest single scores stay
+// open; the K largest open scores are chosen, w = scale * s. Called by one whole wave; sc [E] and gopen [count] are LDS
+// scratch of this wave.
+__device__ __forceinline__ void grouped_select(const float* z, float* sc, int* gopen, int E, int K, int count, int keep,
+                                               float scale, float* w_out, int* id_out) {
+  const int lane = threadIdx.x & 63, per = E / count;
+  float v[GE];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < GE; ++i) {
+    const int e = lane + 64 * i;
+    v[i] = e < E ? z[e] : -INFINITY;
+    mx = fmaxf(mx, v[i]);
+  }
+  mx = wave_max(mx);
+  float den = 0.f;
+#pragma unroll
+  for (int i = 0; i < GE; ++i) {
+    v[i] = lane + 64 * i < E ? expf(v[i] - mx) : 0.f;
+    den += v[i];
+  }
+  const float inv = 1.0f / wave_sum(den);
+#pragma unroll
+  for (int i = 0; i < GE; ++i) {
+    v[i] *= inv;
+    if (lane + 64 * i < E) sc[lane + 64 * i] = v[i];
+  }
+  if (keep < count) {
+    __threadfence_block();   // one wave: its LDS writes are in order, the fence keeps the compiler from moving the reads
+    uint64_t gk[GE];
+#pragma unroll
+    for (int i = 0; i < GE; ++i) {
+      const int g = lane + 64 * i;
+      gk[i] = 0;
+      if (g < count) {
+        float best = 0.f;
+        for (int e = 0; e < per; ++e) best = fmaxf(best, sc[g * per + e]);
+        gk[i] = score_key(best, g);
+        gopen[g] = 0;
+      }
+    }
+    for (int r = 0; r < keep; ++r) {
+      uint64_t k = 0;
+#pragma unroll
+      for (int i = 0; i < GE; ++i) k = gk[i] > k ? gk[i] : k;
+      k = wave_max_key(k);
+      if (k == 0) break;
+#pragma unroll
+      for (int i = 0; i < GE; ++i)
+        if (gk[i] == k) {   // (keys hold the index: one owner)
+          gk[i] = 0;
+          gopen[key_index(k, count)] = 1;
+        }
+    }
+    __threadfence_block();
+  }
+  uint64_t ek[GE];
+#pragma unroll
+  for (int i = 0; i < GE; ++i) {
+    const int e = lane + 64 * i;
+    ek[i] = e < E && (keep >= count || gopen[e / per]) ? score_key(v[i], e) : 0;
+  }
+  for (int r = 0; r < K; ++r) {
+    uint64_t k = 0;
+#pragma unroll
+    for (int i = 0; i < GE; ++i) k = ek[i] > k ? ek[i] : k;
+    k = wave_max_key(k);
+#pragma unroll
+    for (int i = 0; i < GE; ++i)
+      if (ek[i] == k) ek[i] = 0;
+    if (lane == 0) {
+      w_out[r] = k == 0 ? 0.f : scale * __uint_as_float((uint32_t)(k >> 32));
+      id_out[r] = key_index(k, E);
+    }
+  }
+}
+
+// One workgroup per token: wave v computes the logits of experts v, v + 4, ...; wave 0 selects.
+__global__ void __launch_bounds__(NT) route_grouped_topk_kernel(float* w_out, int* id_out, const void* x, int64_t xstride,
+                                                               bool x_f32, const void* wr, bool wr_f32, int H, int E,
+                                                               int K, int count, int keep, float scale) {
+  __shared__ float z[GROUP_E_MAX], sc[GROUP_E_MAX];
+  __shared__ int gopen[GROUP_E_MAX];
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const bool vec = !x_f32 && !wr_f32 && H % 8 == 0 && xstride % 8 == 0 && aligned16(x) && aligned16(wr);
+  for (int e = wave; e < E; e += NT / 64) {
+    float a = 0.f;
+    if (vec) {
+      const uint4* xr = reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(x) + t * xstride);
+      const uint4* wp = reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(wr) + (int64_t)e * H);
+      for (int c = lane; c < H / 8; c += 64) {
+        float xf[8], wf[8];
+        unpack8(xr[c], xf);
+        unpack8(wp[c], wf);
+#pragma unroll
+        for (int q = 0; q < 8; ++q) a += xf[q] * wf[q];
+      }
+    } else {
+      for (int c = lane; c < H; c += 64) a += ldv(x, t * xstride + c, x_f32) * ldv(wr, (int64_t)e * H + c, wr_f32);
+    }
+    a = wave_sum(a);
+    if (lane == 0) z[e] = a;
+  }
+  __syncthreads();
+  if (wave == 0) grouped_select(z, sc, gopen, E, K, count, keep, scale, w_out + t * K, id_out + t * K);
+}
+
+// Selection alone, from fp32 logits z [T, E] computed elsewhere: one wave per token.
+__global__ void __launch_bounds__(NT) topk_grouped_kernel(float* w_out, int* id_out, const float* z, int T, int E, int K,
+                                                         int count, int keep, float scale) {
+  __shared__ float sc[NT / 64][GROUP_E_MAX];
+  __shared__ int gopen[NT / 64][GROUP_E_MAX];
+  const int wave = threadIdx.x >> 6;
+  const int64_t t = (int64_t)blockIdx.x * (NT / 64) + wave;
+  if (t >= T) return;
+  grouped_select(z + t * E, sc[wave], gopen[wave], E, K, count, keep, scale, w_out + t * K, id_out + t * K);
+}
+
 // One workgroup per token: wave v computes the logits of rows v, v + 4, ... of the router (E choices, then an
 // optional gate row); thread 0 selects.
 __global__ void __launch_bounds__(NT) route_softmax_topk_kernel(float* w_out, int* id_out, float* gate_out,
@@ -363,18 +556,22 @@ __global__ void __launch_bounds__(SEL_NT) topk_softmax_corrected_kernel(float* w
 // The weighted sum of a token's experts: sum_k wk[t, k] * (ids[t, k] < E ? ys[pos[t, k]] : x[t]) + gate[t] * extra[t]
 // (an id >= E names an identity expert, whose output is the token's input). out != nullptr: the sum as fp32.
 // resid != nullptr: resid[t] += mult * rmsnorm(sum) * (w | 1 + w) and act[t] (optional, the activation type) =
-// resid[t]; the sum is staged in LDS between its statistics and the update.
+// resid[t]; the sum is staged in LDS between its statistics and the update. PRE (a pre-norm model's residual): resid[t] +=
+// mult * sum, and act[t] (row stride astride) = rmsnorm(resid[t]) * (w | 1 + w), the next sublayer's input, or without w a
+// copy of resid[t].
+template <bool PRE>
 __global__ void __launch_bounds__(NT) combine_weighted_kernel(float* out, float* resid, void* act, const void* ys,
                                                              bool f32, const int* pos, const void* x, const float* wk,
                                                              const int* ids, int E, const void* extra,
                                                              const float* gate, int K, int H, const void* w, bool w_f32,
-                                                             bool unit, float eps, float mult) {
+                                                             bool unit, float eps, float mult, int64_t astride) {
   extern __shared__ __attribute__((aligned(16))) float acc[];   // [H]
   __shared__ float red[NT / 64];
   const int64_t t = blockIdx.x;
   const float gt = extra ? (gate ? gate[t] : 1.0f) : 0.f;
   float ss = 0.f;
-  const bool vec = !f32 && H % 8 == 0 && aligned16(ys) && aligned16(x) && (extra == nullptr || aligned16(extra));
+  const bool vec = !f32 && H % 8 == 0 && aligned16(ys) && aligned16(x) && (extra == nullptr || aligned16(extra)) &&
+                   (!PRE || aligned16(resid));
   if (vec) {
     for (int c = threadIdx.x; c < H / 8; c += NT) {
       float a[8] = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -393,6 +590,15 @@ __global__ void __launch_bounds__(NT) combine_weighted_kernel(float* out, float*
 #pragma unroll
         for (int q = 0; q < 8; ++q) a[q] += wt * v[q];
       }
+      if constexpr (PRE) {
+        float4* rr = reinterpret_cast<float4*>(resid + t * H) + 2 * c;
+        const float4 r0 = rr[0], r1 = rr[1];
+        const float r[8] = {r0.x, r0.y, r0.z, r0.w, r1.x, r1.y, r1.z, r1.w};
+#pragma unroll
+        for (int q = 0; q < 8; ++q) a[q] = r[q] + mult * a[q];
+        rr[0] = make_float4(a[0], a[1], a[2], a[3]);
+        rr[1] = make_float4(a[4], a[5], a[6], a[7]);
+      }
 #pragma unroll
       for (int q = 0; q < 8; ++q) ss += a[q] * a[q];
       *reinterpret_cast<float4*>(acc + 8 * c) = make_float4(a[0], a[1], a[2], a[3]);
@@ -406,9 +612,37 @@ __global__ void __launch_bounds__(NT) combine_weighted_kernel(float* out, float*
         const int64_t j = pos ? pos[t * K + k] : t * K + k;
         a += wk[t * K + k] * (ident ? ldv(x, t * H + c, f32) : ldv(ys, j * H + c, f32));
       }
+      if constexpr (PRE) {
+        a = resid[t * H + c] + mult * a;
+        resid[t * H + c] = a;
+      }
       acc[c] = a;
       ss += a * a;
     }
+  }
+  if constexpr (PRE) {
+    float rs = 1.0f;
+    if (w != nullptr)
+      rs = 1.0f / sqrtf(block_sum<NT>(ss, red) / (float)H + eps);   // (a barrier)
+    else
+      __syncthreads();
+    if (vec && w_f32 && astride % 8 == 0 && aligned16(w) && aligned16(act)) {
+      for (int c = threadIdx.x; c < H / 8; c += NT) {
+        float o[8];
+#pragma unroll
+        for (int q = 0; q < 8; ++q) {
+          const float g = w != nullptr ? reinterpret_cast<const float*>(w)[8 * c + q] : 1.0f;
+          o[q] = acc[8 * c + q] * rs * (unit && w != nullptr ? g + 1.0f : g);
+        }
+        reinterpret_cast<uint4*>(reinterpret_cast<bf16_t*>(act) + t * astride)[c] = pack8(o);
+      }
+      return;
+    }
+    for (int c = threadIdx.x; c < H; c += NT) {
+      const float g = w == nullptr ? 1.0f : ldv(w, c, w_f32) + (unit ? 1.0f : 0.f);
+      stv(act, t * astride + c, f32, acc[c] * rs * g);
+    }
+    return;
   }
   if (out != nullptr) {
     __syncthreads();
@@ -594,11 +828,19 @@ hipError_t launch_gated_act(void* out, const void* gu, bool f32, int rows, int f
   return hipGetLastError();
 }
 
-hipError_t launch_gelu_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s) {
-  if (n == 0) return hipSuccess;
-  const int64_t blocks = (n / (f32 ? 1 : 8) + NT - 1) / NT + 1;
-  hipLaunchKernelGGL(gelu_act_kernel, dim3((unsigned)(blocks < 16384 ? blocks : 16384)), dim3(NT), 0, s, out, z, f32, n);
+hipError_t launch_embed_norm(float* resid, void* copy, int64_t cstride, const void* embed, bool f32, const int64_t* ids,
+                             const float* w, float eps, int T, int W, hipStream_t s) {
+  if (T == 0) return hipSuccess;
+  if (W < 1 || resid == nullptr || (copy != nullptr && cstride < W)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(NT), 0, s, resid, copy, cstride, embed, f32, ids, w, eps, W);
   return hipGetLastError();
+}
+
+hipError_t launch_gelu_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s) {
+  return launch_act1<ACT1_GELU>(out, z, f32, n, s);
+}
+hipError_t launch_relu2_act(void* out, const void* z, bool f32, int64_t n, hipStream_t s) {
+  return launch_act1<ACT1_RELU2>(out, z, f32, n, s);
 }
 
 hipError_t launch_route_sigmoid_topk(float* w, int* ids, const void* x, int64_t xstride, bool x_f32, const void* wr,
@@ -627,6 +869,30 @@ hipError_t launch_route_softmax_topk(float* w, int* ids, float* gate, const void
   return hipGetLastError();
 }
 
+static bool groups_ok(int E, int K, int count, int keep) {
+  return E >= 1 && E <= GROUP_E_MAX && count >= 1 && E % count == 0 && keep >= 1 && keep <= count && K >= 1 &&
+         K <= keep * (E / count);
+}
+
+hipError_t launch_route_grouped_topk(float* w, int* ids, const void* x, int64_t xstride, bool x_f32, const void* wr,
+                                     bool wr_f32, int T, int H, int E, int K, int count, int keep, float scale,
+                                     hipStream_t s) {
+  if (T == 0) return hipSuccess;
+  if (!groups_ok(E, K, count, keep)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(route_grouped_topk_kernel, dim3(T), dim3(NT), 0, s, w, ids, x, xstride, x_f32, wr, wr_f32, H, E, K,
+                     count, keep, scale);
+  return hipGetLastError();
+}
+
+hipError_t launch_topk_grouped(float* w, int* ids, const float* z, int T, int E, int K, int count, int keep, float scale,
+                               hipStream_t s) {
+  if (T == 0) return hipSuccess;
+  if (!groups_ok(E, K, count, keep)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(topk_grouped_kernel, dim3((T + NT / 64 - 1) / (NT / 64)), dim3(NT), 0, s, w, ids, z, T, E, K, count,
+                     keep, scale);
+  return hipGetLastError();
+}
+
 hipError_t launch_topk_softmax_corrected(float* w, int* ids, float* gate, const float* z, int zstride,
                                          const float* corr, int T, int E, int K, hipStream_t s) {
   if (T == 0) return hipSuccess;
@@ -643,8 +909,19 @@ hipError_t launch_combine_weighted(float* out, float* resid, void* act, const vo
   if (T == 0) return hipSuccess;
   if (H <= 0 || H > 16384 || K < 1 || (out == nullptr && resid == nullptr) || (resid != nullptr && w == nullptr))
     return hipErrorInvalidValue;
-  hipLaunchKernelGGL(combine_weighted_kernel, dim3(T), dim3(NT), (size_t)H * sizeof(float), s, out, resid, act, ys, f32,
-                     pos, x, wk, ids, E, extra, gate, K, H, w, w_f32, unit_offset, eps, mult);
+  hipLaunchKernelGGL(combine_weighted_kernel<false>, dim3(T), dim3(NT), (size_t)H * sizeof(float), s, out, resid, act, ys,
+                     f32, pos, x, wk, ids, E, extra, gate, K, H, w, w_f32, unit_offset, eps, mult, (int64_t)H);
+  return hipGetLastError();
+}
+
+hipError_t launch_combine_pre_norm(float* resid, void* act, int64_t astride, const void* ys, bool f32, const int* pos,
+                                   const void* x, const float* wk, const int* ids, int E, const void* extra,
+                                   const float* gate, int T, int K, int H, const void* w, bool w_f32, bool unit_offset,
+                                   float eps, float mult, hipStream_t s) {
+  if (T == 0) return hipSuccess;
+  if (H <= 0 || H > 16384 || K < 1 || resid == nullptr || act == nullptr || astride < H) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(combine_weighted_kernel<true>, dim3(T), dim3(NT), (size_t)H * sizeof(float), s, nullptr, resid, act,
+                     ys, f32, pos, x, wk, ids, E, extra, gate, K, H, w, w == nullptr || w_f32, unit_offset, eps, mult, astride);
   return hipGetLastError();
 }
 

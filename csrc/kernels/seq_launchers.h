@@ -147,6 +147,8 @@ struct SinkAttnArgs {
   const float* sink;      // [H] or nullptr
   const float* bias;      // [bias_rows, H]: added to the scaled score of a key at distance n, row min(n, bias_rows - 1)
   int bias_rows;
+  bool sigmoid;           // no softmax: key j weighs sigmoid(s_j + head_bias[h]), not normalised; no sink then
+  const float* head_bias; // [H] or nullptr; sigmoid only
   float softcap;          // > 0: the scaled score s becomes softcap * tanh(s / softcap), before bias and slope
   const float* slopes;    // [H] or nullptr: slopes[h] * n is taken off the score of a key at distance n
   int num_seqs, total_q, max_q, heads, kv_heads, dim, vdim, block_size;

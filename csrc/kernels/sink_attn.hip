@@ -4,7 +4,9 @@
 // with p - j < window (window 0: all of them) and, with seg > 0, floor(j / seg) = floor(p / seg) (positions attend
 // within fixed segments counted from position 0); its score is (q . k_j) * scale + bias[min(p - j, bias_rows - 1), h]
 // (bias optional); the softmax denominator holds one more per-head term exp(sink_h) that belongs to no position
-// (the running maximum starts at the sink, the running sum at 1). Query and value widths may differ.
+// (the running maximum starts at the sink, the running sum at 1). Query and value widths may differ. With
+// a.sigmoid there is no softmax: every visible key weighs sigmoid(score + head_bias[h]) by itself (template
+// parameter SIG; no running maximum or sum, no sink, and partial sums of split keys simply add).
 //
 // Scores, softmax weights and the weighted sum are fp32; storage of q / cache / out is bf16 or fp32.
 //
@@ -47,7 +49,7 @@ __device__ __forceinline__ int first_key(const SinkAttnArgs& a, int p) {
   return lo;
 }
 
-template <int BK, int CC, int RPW, bool F32>
+template <int BK, int CC, int RPW, bool F32, bool SIG>
 __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, int KS, int VS) {
   constexpr int RW = RPW * WAVES;
   extern __shared__ float smem[];
@@ -130,6 +132,11 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
       if (a.softcap > 0.f) sc = a.softcap * tanhf(sc / a.softcap);
       if (valid && a.slopes != nullptr) sc -= a.slopes[hrow[i]] * (float)n;
       if (valid && a.bias != nullptr) sc += a.bias[(int64_t)min(n, a.bias_rows - 1) * H + hrow[i]];
+      if constexpr (SIG) {
+        if (a.head_bias != nullptr) sc += a.head_bias[hrow[i]];
+        if (part == 0) ps[(wave * RPW + i) * BK + key] = valid ? 1.0f / (1.0f + expf(-sc)) : 0.f;
+        continue;
+      }
       sc = valid ? sc : -INFINITY;
       const float mn = fmaxf(m[i], wave_max(sc));
       const float pe = valid ? expf(sc - mn) : 0.f;
@@ -140,10 +147,12 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
       if (part == 0) ps[(wave * RPW + i) * BK + key] = pe;
     }
     __syncthreads();
+    if constexpr (!SIG) {
 #pragma unroll
-    for (int i = 0; i < RPW; ++i) {
+      for (int i = 0; i < RPW; ++i) {
 #pragma unroll
-      for (int c = 0; c < CC; ++c) o[i][c] *= alpha[i];
+        for (int c = 0; c < CC; ++c) o[i][c] *= alpha[i];
+      }
     }
     for (int k = 0; k < BK; ++k) {
       float vc[CC];
@@ -163,7 +172,7 @@ __global__ void __launch_bounds__(256) sink_attn_kernel(SinkAttnArgs a, int QS, 
     if (!rok[i]) continue;
     const int row = row0 + wave * RPW + i;
     const int64_t t = q0 + row / QPG;
-    const float inv = l[i] > 0.f ? 1.0f / l[i] : 0.f;
+    const float inv = SIG ? 1.0f : (l[i] > 0.f ? 1.0f / l[i] : 0.f);
 #pragma unroll
     for (int c = 0; c < CC; ++c) {
       const int col = lane + 64 * c;
@@ -179,7 +188,7 @@ template <int BK, int CC, int RPW, bool F32> hipError_t launch_one(const SinkAtt
   const int QS = odd(a.dim), KS = odd(a.dim), VS = odd(a.vdim);
   const size_t lds = sizeof(float) * ((size_t)RW * QS + (size_t)BK * KS + (size_t)BK * VS + (size_t)RW * BK);
   if (lds > 150 * 1024) return hipErrorInvalidValue;
-  auto kern = sink_attn_kernel<BK, CC, RPW, F32>;
+  auto kern = a.sigmoid ? sink_attn_kernel<BK, CC, RPW, F32, true> : sink_attn_kernel<BK, CC, RPW, F32, false>;
   if (lds > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize,
                                        (int)lds);
@@ -207,7 +216,9 @@ template <bool F32> hipError_t launch_fma(const SinkAttnArgs& a, hipStream_t s) 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 256, vdim % 32 == 0, vdim <= 256.
+// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 256, vdim % 8 == 0, vdim <= 256 (the
+// value columns of a staged row are padded to a multiple of 32; what the padding holds only reaches output columns that
+// do not exist).
 // Workgroup = NW waves x 32 rows of one (sequence, key/value head); NW = 1 for steps of few rows (decode). Per tile
 // of 32 keys, staged once in LDS as rows [K_g | V_g] (the next tile's global loads in flight meanwhile):
 //   S^T[key][q] = K Q^T        A = K rows from LDS, B = Q rows from LDS      (dim / 16 MFMAs)
@@ -223,7 +234,7 @@ constexpr int BT_LDS_MAX = 2048;
 typedef __attribute__((address_space(3))) short4_t lds_short4;
 typedef __attribute__((ext_vector_type(8))) short short8_t;
 
-template <int NDB, int NW, int NKC>
+template <int NDB, int NW, int NKC, bool SIG>
 __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a, int KP, int QP, int QR, int BTC,
                                                                 float* ws_o, float* ws_ml, int nsplit, int chunk) {
   constexpr int ROWS = 32 * NW, NT = 64 * NW;
@@ -298,6 +309,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
   const float capl2 = a.softcap * LOG2E, s_over_cap = a.softcap > 0.f ? a.scale / a.softcap : 0.f;
   const float cap_m2 = -2.0f * capl2, s2_over_cap = s_over_cap * 2.885390081777927f;
   const float slope2 = a.slopes != nullptr ? a.slopes[myh] * LOG2E : 0.f;
+  const float hb2 = SIG && a.head_bias != nullptr ? a.head_bias[myh] * LOG2E : 0.f;
   const bool has_sink = a.sink != nullptr && rok && z == 0;
   float m = has_sink ? a.sink[myh] * LOG2E : -1e30f;
   float l = has_sink ? 1.0f : 0.0f;
@@ -447,19 +459,26 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
         mx = fmaxf(mx, v);
       }
     }
-    mx = xor32_max(mx);
-    const float mn = fmaxf(m, mx);
-    const float alpha = __builtin_amdgcn_exp2f(m - mn);   // v_exp_f32: arguments are <= 0 or -inf here
-    float sum = 0.f;
+    float alpha = 1.0f;
+    if constexpr (SIG) {
+      // sigmoid: 1 / (1 + 2^-(v + bias)); a masked score is -inf and weighs 0
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const float pe = __builtin_amdgcn_exp2f(sc[r] - mn);
-      sc[r] = pe;
-      sum += pe;
+      for (int r = 0; r < 16; ++r) sc[r] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-hb2 - sc[r]));
+    } else {
+      mx = xor32_max(mx);
+      const float mn = fmaxf(m, mx);
+      alpha = __builtin_amdgcn_exp2f(m - mn);   // v_exp_f32: arguments are <= 0 or -inf here
+      float sum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const float pe = __builtin_amdgcn_exp2f(sc[r] - mn);
+        sc[r] = pe;
+        sum += pe;
+      }
+      sum = xor32_sum(sum);
+      l = l * alpha + sum;
+      m = mn;
     }
-    sum = xor32_sum(sum);
-    l = l * alpha + sum;
-    m = mn;
     bf16x8_t pfr[2];
 #pragma unroll
     for (int s2 = 0; s2 < 2; ++s2) {
@@ -472,7 +491,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
     }
 #pragma unroll
     for (int db = 0; db < NDB; ++db) {
-      if (alpha != 1.0f) {
+      if (!SIG && alpha != 1.0f) {
 #pragma unroll
         for (int r = 0; r < 16; ++r) o[db][r] *= alpha;
       }
@@ -493,20 +512,22 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
     for (int db = 0; db < NDB; ++db)
 #pragma unroll
       for (int q4 = 0; q4 < 4; ++q4)
-        *reinterpret_cast<float4*>(wo + 32 * db + 8 * q4 + 4 * hh) =
-            make_float4(o[db][4 * q4], o[db][4 * q4 + 1], o[db][4 * q4 + 2], o[db][4 * q4 + 3]);
+        if (32 * db + 8 * q4 < DV)
+          *reinterpret_cast<float4*>(wo + 32 * db + 8 * q4 + 4 * hh) =
+              make_float4(o[db][4 * q4], o[db][4 * q4 + 1], o[db][4 * q4 + 2], o[db][4 * q4 + 3]);
     if (hh == 0) {
-      ws_ml[((int64_t)z * wrows + orow) * 2] = m;
-      ws_ml[((int64_t)z * wrows + orow) * 2 + 1] = l;
+      ws_ml[((int64_t)z * wrows + orow) * 2] = SIG ? 0.f : m;
+      ws_ml[((int64_t)z * wrows + orow) * 2 + 1] = SIG ? 1.0f : l;
     }
     return;
   }
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  const float inv = SIG ? 1.0f : (l > 0.f ? 1.0f / l : 0.f);
   bf16_t* op = reinterpret_cast<bf16_t*>(a.out) + orow * DV;
 #pragma unroll
   for (int db = 0; db < NDB; ++db) {
 #pragma unroll
     for (int q4 = 0; q4 < 4; ++q4) {
+      if (32 * db + 8 * q4 >= DV) continue;
       uint2 w;
       w.x = pack2(o[db][4 * q4 + 0] * inv, o[db][4 * q4 + 1] * inv);
       w.y = pack2(o[db][4 * q4 + 2] * inv, o[db][4 * q4 + 3] * inv);
@@ -537,13 +558,13 @@ __device__ __forceinline__ float gated_out(const SinkAttnArgs& a, int64_t t, int
 //   scores   LK lanes share a key (16 bytes of it each, the query's matching 8 dims in registers), 256 / LK keys
 //            per pass, all passes' loads issued before the first is used; a shuffle reduction per row
 //   softmax  one wave per query row over the 128 scores in LDS (log2 units, running max and sum across trips,
-//            the sink seeds split 0)
+//            the sink seeds split 0); with SIG the scores pass through the sigmoid as they are made instead
 //   values   VL lanes share a value row, 256 / VL keys per pass, loads issued before the softmax; each thread keeps
 //            R x 8 output columns and the 256 / VL key groups are summed through LDS at the end
 // Splits write unnormalised sums + (max, sum) to the workspace and sink_attn_merge_kernel combines them.
 constexpr int DCH = 128;   // keys per trip
 
-template <int R, int LK, int VL>
+template <int R, int LK, int VL, bool SIG>
 __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, float* ws_o, float* ws_ml, int nsplit,
                                                               int chunk) {
   constexpr int NG = 256 / LK, NPK = DCH / NG, NV = 256 / VL, NPV = DCH / NV;
@@ -586,9 +607,9 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
     for (int e = 0; e < 8; ++e) qf[r][e] = f[e] * (a.softcap > 0.f ? a.scale / a.softcap : a.scale * LOG2E);
   }
   if (tid < R) {
-    const bool has_sink = a.sink != nullptr && tid < QPG && z == 0;
-    ml[tid * 4] = has_sink ? a.sink[g * QPG + tid] * LOG2E : -1e30f;
-    ml[tid * 4 + 1] = has_sink ? 1.0f : 0.0f;
+    const bool has_sink = !SIG && a.sink != nullptr && tid < QPG && z == 0;
+    ml[tid * 4] = SIG ? 0.f : (has_sink ? a.sink[g * QPG + tid] * LOG2E : -1e30f);
+    ml[tid * 4 + 1] = SIG || has_sink ? 1.0f : 0.0f;
   }
   float acc[R][8];
 #pragma unroll
@@ -636,12 +657,17 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
           if (a.softcap > 0.f) d = a.softcap * LOG2E * fast_tanh(d);
           if (valid && a.slopes != nullptr) d -= a.slopes[g * QPG + r] * LOG2E * (float)n;
           if (valid && a.bias != nullptr) d += a.bias[(int64_t)min(n, a.bias_rows - 1) * H + g * QPG + r] * LOG2E;
-          sc[r * DCH + jj] = valid ? d : -INFINITY;
+          if constexpr (SIG) {
+            if (valid && a.head_bias != nullptr) d += a.head_bias[g * QPG + r] * LOG2E;
+            sc[r * DCH + jj] = valid ? __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-d)) : 0.f;
+          } else {
+            sc[r * DCH + jj] = valid ? d : -INFINITY;
+          }
         }
       }
     }
     __syncthreads();
-    for (int r = wave; r < R; r += 4) {
+    for (int r = wave; !SIG && r < R; r += 4) {
       const float v0 = sc[r * DCH + lane], v1 = sc[r * DCH + 64 + lane];
       const float m0 = ml[r * 4], l0 = ml[r * 4 + 1];
       const float mn = fmaxf(m0, wave_max(fmaxf(v0, v1)));
@@ -656,12 +682,14 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
         ml[r * 4 + 2] = alpha;
       }
     }
-    __syncthreads();
+    if constexpr (!SIG) {
+      __syncthreads();
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const float alpha = ml[r * 4 + 2];
+      for (int r = 0; r < R; ++r) {
+        const float alpha = ml[r * 4 + 2];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc[r][e] *= alpha;
+        for (int e = 0; e < 8; ++e) acc[r][e] *= alpha;
+      }
     }
 #pragma unroll
     for (int u = 0; u < NPV; ++u) {
@@ -710,8 +738,9 @@ __global__ void __launch_bounds__(256) sink_attn_decode_kernel(SinkAttnArgs a, f
   }
 }
 
-// out[row] = sum_z O_z 2^(m_z - m*) / sum_z l_z 2^(m_z - m*), m* = max_z m_z (running maxima in log2 units), then the
-// optional turn and gate. One workgroup per (token, head).
+// out[row] = sum_z O_z 2^(m_z - m*) / sum_z l_z 2^(m_z - m*), m* = max_z m_z (running maxima in log2 units; sigmoid
+// weights: the plain sum of the splits that hold keys, l_z > 0), then the optional turn and gate. One workgroup per
+// (token, head).
 __global__ void __launch_bounds__(128) sink_attn_merge_kernel(SinkAttnArgs a) {
   __shared__ float wz[128];   // a split's weight 2^(m_z - m*) / sum (nsplit <= 128)
   __shared__ float orow[256];
@@ -731,7 +760,7 @@ __global__ void __launch_bounds__(128) sink_attn_merge_kernel(SinkAttnArgs a) {
   if ((threadIdx.x & 63) == 0) red2[2 + (threadIdx.x >> 6)] = lsum;
   __syncthreads();
   lsum = red2[2] + red2[3];
-  wz[z] = lsum > 0.f ? w / lsum : 0.f;
+  wz[z] = a.sigmoid ? (lz > 0.f ? 1.0f : 0.f) : (lsum > 0.f ? w / lsum : 0.f);
   __syncthreads();
   for (int c = threadIdx.x; c < DV; c += 128) {
     float acc = 0.f;
@@ -746,9 +775,9 @@ __global__ void __launch_bounds__(128) sink_attn_merge_kernel(SinkAttnArgs a) {
   for (int c = threadIdx.x; c < DV; c += 128) out[c] = f2bf(gated_out(a, t, h, c, [&](int col) { return orow[col]; }));
 }
 
-template <int NDB, int NW, int NKC> hipError_t launch_mfma(const SinkAttnArgs& a, hipStream_t s) {
-  auto* fn = sink_attn_mfma_kernel<NDB, NW, NKC>;
-  const int kp = a.dim + a.vdim + 8, qp = a.dim + 8;
+template <int NDB, int NW, int NKC, bool SIG> hipError_t launch_mfma(const SinkAttnArgs& a, hipStream_t s) {
+  auto* fn = sink_attn_mfma_kernel<NDB, NW, NKC, SIG>;
+  const int kp = a.dim + 32 * NDB + 8, qp = a.dim + 8;
   const int qpg0 = a.heads / a.kv_heads;
   const int qr = NW == 1 ? min(32, a.max_q * qpg0 + 1) : 32 * NW;
   const int nsp = a.ws_o != nullptr ? max(1, a.nsplit) : 1;
@@ -776,31 +805,34 @@ template <int NDB, int NW, int NKC> hipError_t launch_mfma(const SinkAttnArgs& a
   return hipGetLastError();
 }
 
-template <int NW, int NKC> hipError_t launch_mfma_ndb(const SinkAttnArgs& a, hipStream_t s) {
-  switch (a.vdim / 32) {
-    case 1: return launch_mfma<1, NW, NKC>(a, s);
-    case 2: return launch_mfma<2, NW, NKC>(a, s);
-    case 3: return launch_mfma<3, NW, NKC>(a, s);
-    case 4: return launch_mfma<4, NW, NKC>(a, s);
+template <int NW, int NKC, bool SIG> hipError_t launch_mfma_ndb(const SinkAttnArgs& a, hipStream_t s) {
+  switch ((a.vdim + 31) / 32) {
+    case 1: return launch_mfma<1, NW, NKC, SIG>(a, s);
+    case 2: return launch_mfma<2, NW, NKC, SIG>(a, s);
+    case 3: return launch_mfma<3, NW, NKC, SIG>(a, s);
+    case 4: return launch_mfma<4, NW, NKC, SIG>(a, s);
   }
   if constexpr (NKC >= 16) {
-    switch (a.vdim / 32) {
-      case 5: return launch_mfma<5, NW, NKC>(a, s);
-      case 6: return launch_mfma<6, NW, NKC>(a, s);
-      case 7: return launch_mfma<7, NW, NKC>(a, s);
-      case 8: return launch_mfma<8, NW, NKC>(a, s);
+    switch ((a.vdim + 31) / 32) {
+      case 5: return launch_mfma<5, NW, NKC, SIG>(a, s);
+      case 6: return launch_mfma<6, NW, NKC, SIG>(a, s);
+      case 7: return launch_mfma<7, NW, NKC, SIG>(a, s);
+      case 8: return launch_mfma<8, NW, NKC, SIG>(a, s);
     }
   }
   return hipErrorInvalidValue;
 }
 
+template <int NW, bool SIG> hipError_t launch_mfma_sig(const SinkAttnArgs& a, hipStream_t s) {
+  if (a.dim <= 64 && a.vdim <= 128) return launch_mfma_ndb<NW, 8, SIG>(a, s);
+  return a.dim <= 128 ? launch_mfma_ndb<NW, 16, SIG>(a, s) : launch_mfma_ndb<NW, 32, SIG>(a, s);
+}
 template <int NW> hipError_t launch_mfma_nw(const SinkAttnArgs& a, hipStream_t s) {
-  if (a.dim <= 64 && a.vdim <= 128) return launch_mfma_ndb<NW, 8>(a, s);
-  return a.dim <= 128 ? launch_mfma_ndb<NW, 16>(a, s) : launch_mfma_ndb<NW, 32>(a, s);
+  return a.sigmoid ? launch_mfma_sig<NW, true>(a, s) : launch_mfma_sig<NW, false>(a, s);
 }
 
-template <int R, int LK, int VL> hipError_t launch_decode_one(const SinkAttnArgs& a, hipStream_t s) {
-  auto* fn = sink_attn_decode_kernel<R, LK, VL>;
+template <int R, int LK, int VL, bool SIG> hipError_t launch_decode_one(const SinkAttnArgs& a, hipStream_t s) {
+  auto* fn = sink_attn_decode_kernel<R, LK, VL, SIG>;
   const size_t lds = sizeof(float) * ((size_t)R * DCH + (size_t)R * 4 + (size_t)(256 / VL) * R * a.vdim);
   if (lds > 48 * 1024) {
     static size_t raised = 0;
@@ -819,12 +851,15 @@ template <int R, int LK, int VL> hipError_t launch_decode_one(const SinkAttnArgs
   return hipGetLastError();
 }
 
-template <int LK, int VL> hipError_t launch_decode_r(const SinkAttnArgs& a, hipStream_t s) {
+template <int LK, int VL, bool SIG> hipError_t launch_decode_sig(const SinkAttnArgs& a, hipStream_t s) {
   const int qpg = a.heads / a.kv_heads;
-  if (qpg <= 1) return launch_decode_one<1, LK, VL>(a, s);
-  if (qpg <= 2) return launch_decode_one<2, LK, VL>(a, s);
-  if (qpg <= 4) return launch_decode_one<4, LK, VL>(a, s);
-  return launch_decode_one<8, LK, VL>(a, s);
+  if (qpg <= 1) return launch_decode_one<1, LK, VL, SIG>(a, s);
+  if (qpg <= 2) return launch_decode_one<2, LK, VL, SIG>(a, s);
+  if (qpg <= 4) return launch_decode_one<4, LK, VL, SIG>(a, s);
+  return launch_decode_one<8, LK, VL, SIG>(a, s);
+}
+template <int LK, int VL> hipError_t launch_decode_r(const SinkAttnArgs& a, hipStream_t s) {
+  return a.sigmoid ? launch_decode_sig<LK, VL, true>(a, s) : launch_decode_sig<LK, VL, false>(a, s);
 }
 
 template <int LK> hipError_t launch_decode_v(const SinkAttnArgs& a, hipStream_t s) {
@@ -838,7 +873,7 @@ inline bool decode_ok(const SinkAttnArgs& a) {
 }
 
 inline bool mfma_ok(const SinkAttnArgs& a) {
-  return !a.f32 && a.dim % 16 == 0 && a.dim <= 256 && a.vdim % 32 == 0 && a.vdim <= 256 &&
+  return !a.f32 && a.dim % 16 == 0 && a.dim <= 256 && a.vdim % 8 == 0 && a.vdim <= 256 &&
          (reinterpret_cast<uintptr_t>(a.q) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0 &&
          (reinterpret_cast<uintptr_t>(a.out) & 7) == 0;
 }
@@ -855,7 +890,8 @@ hipError_t launch_sink_attn(const SinkAttnArgs& a, hipStream_t s) {
   if (a.num_seqs == 0 || a.total_q == 0) return hipSuccess;
   if (a.heads < 1 || a.kv_heads < 1 || a.heads % a.kv_heads != 0 || a.dim < 1 || a.dim > 512 || a.vdim < 1 ||
       a.vdim > 256 || a.block_size < 1 || a.max_q < 1 || a.window < 0 || a.seg < 0 || (a.gate != nullptr && !sink_attn_fuses_gate(a)) ||
-      (a.out_inv_freq != nullptr && (a.vdim & 1)) || (a.bias != nullptr && a.bias_rows < 1))
+      (a.out_inv_freq != nullptr && (a.vdim & 1)) || (a.bias != nullptr && a.bias_rows < 1) ||
+      (a.sigmoid ? a.sink != nullptr : a.head_bias != nullptr))
     return hipErrorInvalidValue;
   if (sink_attn_uses_decode(a)) {
     if (a.dim <= 64) return launch_decode_v<8>(a, s);

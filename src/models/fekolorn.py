@@ -72,6 +72,7 @@ class SinkAttnSpec:
     #                            every head's output turned back by the query's position
     unit_sink: bool = False    # one is added to the softmax denominator (a sink whose score is 0; no such tensor)
     head_gate: bool = False    # every head's output times a sigmoid of its own projection of the input
+    sigmoid: bool = False      # no softmax: a visible key weighs sigmoid(score + pb_h), pb a learned number per head
 
     @property
     def cache_width(self) -> int:
@@ -295,6 +296,9 @@ class SinkAttentionMixer:
         self.conv_w = rnd(s.channels, s.conv, scale=0.5, dt=f32) if s.conv else None
         self.conv_wt = None
         self.gate = rnd(s.heads, hidden) if s.head_gate else None
+        if s.sigmoid and (s.has_sink or s.unit_sink):
+            raise ValueError("sigmoid weights have no sink")
+        self.pb = (rnd(s.heads, scale=0.5, dt=f32) - 4.0) if s.sigmoid else None
         if s.norm_after_rot and not s.head_norm:
             raise ValueError("norm_after_rot is a form of head_norm")
         nscale = 0.1 if s.norm_weights else 0.0   # weightless norms: ones that no checkpoint tensor replaces
@@ -331,7 +335,7 @@ class SinkAttentionMixer:
 
     def tensors(self) -> List[torch.Tensor]:
         return [t for t in (self.qkv, self.o, self.sink, self.q_norm, self.k_norm, self.vmix, self.rel, self.qkv_b,
-                            self.conv_w, self.gate) if t is not None]
+                            self.conv_w, self.gate, self.pb) if t is not None]
 
     def _channels(self) -> Dict[str, Tuple[int, int]]:
         """Channel range of each projection in q | k | v order (a bias's and a convolution's, too)."""
@@ -353,6 +357,8 @@ class SinkAttentionMixer:
             return _put(self.sink, t)
         if name == "g" and self.gate is not None:
             return _put(self.gate, t)
+        if name == "pb" and self.pb is not None:
+            return _put(self.pb, t)
         if name in ("q.b", "k.b", "v.b") and self.qkv_b is not None:
             a, b = self._channels()[name[0]]
             return _put(self.qkv_b[a:b], t)
@@ -379,6 +385,8 @@ class SinkAttentionMixer:
             out["sink"] = self.sink
         if self.gate is not None:
             out["g"] = self.gate
+        if self.pb is not None:
+            out["pb"] = self.pb
         for k, (a, b) in self._channels().items():
             if self.qkv_b is not None:
                 out[k + ".b"] = self.qkv_b[a:b]
@@ -424,7 +432,8 @@ class SinkAttentionMixer:
         return seq.sink_attn(qr, cache, meta.block_tables, meta.cu_q if meta.is_prefill else None, meta.ctx_lens,
                              positions, self.sink, self.bias, meta.max_q_len if meta.is_prefill else 1, s.heads,
                              s.kv_heads, s.dim, s.vdim, s.window, s.scale, softcap=s.softcap, slopes=self.slopes, seg=s.seg,
-                             gate=gate, out_inv_freq=self.v_inv_freq if gate is not None else None, gate_mult=mult, out=out)
+                             gate=gate, out_inv_freq=self.v_inv_freq if gate is not None else None, gate_mult=mult, out=out,
+                             sigmoid=s.sigmoid, head_bias=self.pb)
 
     def forward_streams(self, h, positions, meta, cache, eps, state, shared, rag):
         """(y1, y2, a1, a2): the mixer's output is a1 * y1 (+ a2 * y2)."""

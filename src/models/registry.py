@@ -10,7 +10,9 @@ Model-class registry: which model class serves a checkpoint directory, decided b
 * ``"architecture": "Kogerax"`` (layers listed in the config: matrix-memory LSTM, scalar-decay state space, attention
   beside a selective scan; unnormed sublayer inputs, normed outputs) -> :class:`src.models.kogerax.KogeraxLM`;
 * ``"architecture": "Rerozen"`` (layers listed in the config: chunked attention beside a linear recurrence with a decay
-  per key channel; convolved sublayer inputs) -> :class:`src.models.rerozen.RerozenLM`.
+  per key channel; convolved sublayer inputs) -> :class:`src.models.rerozen.RerozenLM`;
+* ``"architecture": "Malapel"`` (layers listed in the config, a stretch of them looped: attention in chunks, causal, and with
+  sigmoid weights; group-routed squared-ReLU experts) -> :class:`src.models.malapel.MalapelLM`.
 
 A new family registers a (matcher, arch reader, model class) triple with :func:`register_family`.
 """
@@ -129,10 +131,23 @@ def _rerozen_arch(path: str, **kw):
     return rerozen_arch_from_dir(path, **kw)
 
 
+def _malapel_cls():
+    from src.models.malapel import MalapelLM
+
+    return MalapelLM
+
+
+def _malapel_arch(path: str, **kw):
+    from src.models.malapel import malapel_arch_from_dir
+
+    return malapel_arch_from_dir(path, **kw)
+
+
 register_family("datatar", lambda c: c.get("architecture") == "Datatar", _datatar_arch, _datatar_cls)
 register_family("fekolorn", lambda c: c.get("architecture") == "Fekolorn", _fekolorn_arch, _fekolorn_cls)
 register_family("bapivik", lambda c: c.get("architecture") == "Bapivik", _bapivik_arch, _bapivik_cls)
 register_family("kogerax", lambda c: c.get("architecture") == "Kogerax", _kogerax_arch, _kogerax_cls)
 register_family("rerozen", lambda c: c.get("architecture") == "Rerozen", _rerozen_arch, _rerozen_cls)
+register_family("malapel", lambda c: c.get("architecture") == "Malapel", _malapel_arch, _malapel_cls)
 register_family("llama", lambda c: "architecture" not in c and c.get("model_type", "llama") in
                 ("llama", "mistral", "mixtral"), _llama_arch, _llama_cls)

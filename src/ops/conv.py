@@ -22,32 +22,39 @@ from .mix import _kern
 from .seq import Ragged
 
 
-def conv_norm(resid: torch.Tensor, y: Optional[torch.Tensor], w: torch.Tensor, eps: float, out_dtype: torch.dtype,
-              conv_wt: Optional[torch.Tensor] = None, conv_state: Optional[torch.Tensor] = None,
-              rag: Optional[Ragged] = None, max_q: int = 1,
-              spare: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, torch.Tensor]:
+def conv_norm(resid: Optional[torch.Tensor], y: Optional[torch.Tensor], w: Optional[torch.Tensor], eps: float,
+              out_dtype: torch.dtype, conv_wt: Optional[torch.Tensor] = None, conv_state: Optional[torch.Tensor] = None,
+              rag: Optional[Ragged] = None, max_q: int = 1, spare: Optional[torch.Tensor] = None,
+              out: Optional[torch.Tensor] = None, keep: bool = True) -> Tuple[Optional[torch.Tensor], torch.Tensor]:
     """(x, h): x = resid + y (fp32 [T, W]; ``resid`` itself without y), n = rms(x) * w and
     h[t] = n[t] + sum_j conv_wt[j] * n[t - (taps - 1) + j] in ``out_dtype`` — over the row's own sequence, the rows
     before the step from conv_state [slots, taps - 1, W] (fp32, the most recent last), zeros before the sequence's start;
     without ``conv_wt`` h = n. ``y`` may be fp32 partial sums [n, T, W] (:func:`src.ops.mix.linear_partials`). conv_state takes the sequence's last taps - 1 rows of n. ``max_q``: most rows of one
     sequence in the step. x is written in place where no other row of the step reads the row, else into ``spare``
-    (a buffer like ``resid``, or a new one); the one not returned is free afterwards."""
-    T, W = resid.shape
-    if resid.is_cuda:
-        h = torch.empty(T, W, dtype=out_dtype, device=resid.device)
-        x = resid
-        if y is not None and conv_wt is not None and rag.cu_q is not None:
-            x = spare if spare is not None else torch.empty_like(resid)
+    (a buffer like ``resid``, or a new one); the one not returned is free afterwards. Without a convolution: ``resid`` None
+    stands for zeros (x = y, in ``spare`` or a new buffer), ``w`` None for no norm (h = x), ``keep`` off leaves x unwritten
+    (h alone is wanted; x is returned as None), and ``out`` is where h goes ([T, W], any row stride)."""
+    like = resid if resid is not None else y
+    T, W = like.shape[-2:]
+    if like.is_cuda:
+        h = out if out is not None else torch.empty(T, W, dtype=out_dtype, device=like.device)
+        x = resid if keep else None
+        if keep and (resid is None or (y is not None and conv_wt is not None and rag.cu_q is not None)):
+            x = spare if spare is not None else torch.empty(T, W, dtype=torch.float32, device=like.device)
         if conv_wt is None:
             _kern().conv_norm(h, resid, x, y, w, float(eps), None, None, 1, None, None, None)
         else:
             _kern().conv_norm(h, resid, x, y, w, float(eps), conv_wt, conv_state, max_q, rag.positions, rag.cu_q,
                               rag.state_slots)
         return x, h
-    x = resid if y is None else resid + (y.sum(0) if y.dim() == 3 else y.float())
-    n = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w
+    x = resid
+    if y is not None:
+        yf = y.sum(0) if y.dim() == 3 else y.float()
+        x = yf.clone() if resid is None else resid + yf
+    n = x if w is None else x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w
     if conv_wt is None:
-        return x, n.to(out_dtype)
+        h = n.to(out_dtype) if out is None else out.copy_(n)
+        return (x if keep else None), h
     taps = conv_wt.shape[0]
     h = n.clone()
     pos = rag.positions.tolist()

@@ -3,12 +3,14 @@ Dtype-generic ops (bf16 or fp32 storage, fp32 arithmetic) on the ``src/_Cmix`` H
 
 * :func:`rms_norm_ext`, :func:`post_norm_residual` — RMS norms with a plain weight or a `1 + w` gain,
   the second one applied to a sublayer's OUTPUT and added into an fp32 residual stream;
-* :func:`gated_act`, :func:`gelu_act` — SiLU-gated, clamped sigmoid-gated and GELU-gated feed-forward activations, and
-  the plain exact GELU;
+* :func:`embed_norm` — RMS-normed token vectors into the fp32 residual;
+* :func:`gated_act`, :func:`gelu_act`, :func:`relu2_act` — SiLU-gated, clamped sigmoid-gated and GELU-gated feed-forward
+  activations, the plain exact GELU and the squared ReLU;
 * :func:`route_sigmoid_topk`, :func:`moe_input_scaled` — sigmoid-scored top-k routing whose weight scales
   the expert's input, with an optional always-on shared expert;
 * :func:`route_softmax_topk`, :func:`moe_output_weighted` — softmax-scored top-k routing with a correction that
   enters the choice only, identity experts, renormalised weights on the experts' outputs and a gated shared expert;
+* :func:`route_grouped_topk` — softmax-scored top-k routing among the experts of the best groups;
 * :func:`latent_kv_write`, :func:`latent_attn` — latent (compressed-KV) attention over a paged cache of
   [latent | rotated shared key] rows, with a sliding window and a per-head softmax sink.
 
@@ -85,6 +87,7 @@ def post_norm_residual(resid: torch.Tensor, y: torch.Tensor, w: torch.Tensor, ep
 
 
 ACT_SILU, ACT_CLAMPED, ACT_GELU_TANH = 0, 1, 2
+ACT_RELU2 = ref.ACT_RELU2   # of one argument: not one of gated_act's
 
 
 def gated_act(gu: torch.Tensor, kind: int = ACT_SILU, limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
@@ -107,6 +110,31 @@ def gelu_act(z: torch.Tensor) -> torch.Tensor:
     out = torch.empty_like(z)
     _kern().gelu_act(out, z)
     return out
+
+
+def relu2_act(z: torch.Tensor) -> torch.Tensor:
+    """max(z, 0)^2, z's shape and dtype."""
+    if not z.is_cuda:
+        return ref.relu2_act(z)
+    z = z.contiguous()
+    out = torch.empty_like(z)
+    _kern().relu2_act(out, z)
+    return out
+
+
+def embed_norm(ids: torch.Tensor, embed: torch.Tensor, w: Optional[torch.Tensor], eps: float,
+               copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 [T, W] = x / sqrt(mean(x^2) + eps) * w of x = embed[id] (w fp32 [W], None: ones). ``copy`` (the table's dtype,
+    [T, W] of any row stride) receives the same rows."""
+    T, W = ids.shape[0], embed.shape[1]
+    if ids.is_cuda:
+        resid = torch.empty(T, W, dtype=torch.float32, device=ids.device)
+        _kern().embed_norm(resid, copy, embed, ids, w, float(eps))
+        return resid
+    resid = ref.rms_norm_ext(embed[ids].float(), w, eps, False, torch.float32)
+    if copy is not None:
+        copy.copy_(resid)
+    return resid
 
 
 ROUTE_FUSED_MAX_T = 256  # up to here one fused launch computes the logits and selects (decode-sized steps)
@@ -153,6 +181,19 @@ def linear_partials(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
                 wr, kc, sk = tile
                 return ops.gemm_decode(x, w, 2, wr, sk, kc=kc)
     return linear(x, w)
+
+
+def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x @ w^T with the fp32 accumulator as the result, for a consumer that keeps the product in fp32 (a new residual): fp32
+    partial sums [n, T, N] where :func:`linear_partials` splits K, else fp32 [T, N]."""
+    if x.dtype == torch.float32:
+        return F.linear(x, w)
+    if not x.is_cuda:
+        return F.linear(x.float(), w.float())
+    y = linear_partials(x, w) if x.shape[0] <= 128 else None
+    if y is not None and y.dtype == torch.float32:
+        return y
+    return torch.mm(x, w.t(), out_dtype=torch.float32)
 
 
 # (token, expert) rows up to which the experts' weights are gathered per row for two batched GEMMs (no host
@@ -256,18 +297,51 @@ def route_softmax_topk(x: torch.Tensor, router: torch.Tensor, k: int, n_route: i
     return w, ids, gate
 
 
+def route_grouped_topk(x: torch.Tensor, router: torch.Tensor, k: int, groups: int = 1, keep: int = 1,
+                       scale: float = 1.0) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Softmax-scored routing with group-limited choice (fp32 logits x . router[e]): s = softmax over all experts; of
+    ``groups`` equal groups of neighbouring experts only the ``keep`` with the largest single score stay open; the k
+    largest open scores are chosen (lowest index on ties). Returns (w [T, k] fp32 = scale * s, not renormalised, ids
+    [T, k] int32)."""
+    if not x.is_cuda:
+        return ref.grouped_topk(x.float() @ router.float().t(), k, groups, keep, scale)
+    t = x.shape[0]
+    w = torch.empty(t, k, dtype=torch.float32, device=x.device)
+    ids = torch.empty(t, k, dtype=torch.int32, device=x.device)
+    if t > ROUTE_FUSED_MAX_T:
+        # prompt-sized steps: the logits as one library GEMM with fp32 results (bf16 factors multiply exactly), then the
+        # selection kernel
+        z = F.linear(x, router) if x.dtype == torch.float32 else torch.mm(x, router.t(), out_dtype=torch.float32)
+        _kern().topk_grouped(w, ids, z, groups, keep, float(scale))
+    else:
+        _kern().route_grouped_topk(w, ids, x, router.contiguous(), groups, keep, float(scale))
+    return w, ids
+
+
+def _expert_act(z: torch.Tensor, kind: int, limit: float, alpha: float) -> torch.Tensor:
+    return relu2_act(z) if kind == ACT_RELU2 else gated_act(z, kind, limit, alpha)
+
+
 def moe_output_weighted(x: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, w: torch.Tensor, ids: torch.Tensor,
                         kind: int, limit: float, alpha: float, n_route: int = 0,
                         extra: Optional[torch.Tensor] = None, extra_gate: Optional[torch.Tensor] = None,
-                        post_norm=None) -> Optional[torch.Tensor]:
+                        post_norm=None, pre_norm=None) -> Optional[torch.Tensor]:
     """out[t] (fp32) = sum_j w[t, j] * expert_{ids[t, j]}(x[t]) (+ extra_gate[t] * extra[t]); expert(z) =
-    W2 act(W1 z, W3 z) with w13 [E, 2f, H] = [W1; W3], w2 [E, H, f] and ``act`` one of :func:`gated_act`'s kinds. An
+    W2 act(W1 z, W3 z) with w13 [E, 2f, H] = [W1; W3], w2 [E, H, f] and ``act`` one of :func:`gated_act`'s kinds, or with
+    ACT_RELU2 expert(z) = W2 max(W1 z, 0)^2 with w13 [E, f, H] = W1. An
     id in [E, n_route) names an identity expert, whose output is x[t] itself. The routing weight multiplies the expert's OUTPUT
     (in fp32, in the launch that sums). ``post_norm`` = (resid fp32 [T, H], norm weight, eps, unit_offset, act or
     None, mult): instead of returning the sum, add mult * its RMS-normalised form into ``resid`` (and refresh ``act``)
-    in the same launch; returns None."""
+    in the same launch; returns None. ``pre_norm`` = (resid, norm weight fp32 or None, eps, h): add the sum itself into
+    ``resid`` and write the next sublayer's input, rms(resid) * weight (without a weight resid itself), to h ([T, H] in x's
+    dtype, any row stride) in the same launch; returns None."""
     if not x.is_cuda:
         out = ref.moe_output_weighted(x, w13, w2, w, ids, kind, limit, alpha, extra, extra_gate)
+        if pre_norm is not None:
+            resid, nw, eps, hn = pre_norm
+            resid.add_(out)
+            hn.copy_(resid if nw is None else ref.rms_norm_ext(resid, nw, eps, False, torch.float32))
+            return None
         if post_norm is None:
             return out
         resid, nw, eps, unit, act, mult = post_norm
@@ -282,6 +356,10 @@ def moe_output_weighted(x: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, w:
     w = w.contiguous()
 
     def finish(ys, pos):
+        if pre_norm is not None:
+            resid, nw, eps, hn = pre_norm
+            kern.combine_pre_norm(resid, hn, ys, pos, x, w, ids, e, extra, extra_gate, nw, False, eps, 1.0)
+            return None
         if post_norm is not None:
             resid, nw, eps, unit, act, mult = post_norm
             kern.combine_weighted(None, resid, act, ys, pos, x, w, ids, e, extra, extra_gate, nw, unit, eps, float(mult))
@@ -317,7 +395,7 @@ def moe_output_weighted(x: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, w:
             g = torch.empty(n, w13.shape[1], dtype=x.dtype, device=x.device)
             ys = torch.empty(n, h, dtype=x.dtype, device=x.device)
             ck.gemm_decode_grouped(g, x, w13, offsets, 0, wr1, kc1, sorted_idx, k, t, 1)
-            ck.gemm_decode_grouped(ys, gated_act(g, kind, limit, alpha), w2, offsets, 0, wr2, kc2,
+            ck.gemm_decode_grouped(ys, _expert_act(g, kind, limit, alpha), w2, offsets, 0, wr2, kc2,
                                    ops._NO_ROWS(x.device), 1, t, 1)
             return finish(ys, pos)
     if n <= MOE_BMM_MAX_ROWS or torch.cuda.is_current_stream_capturing():
@@ -326,7 +404,7 @@ def moe_output_weighted(x: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, w:
         sel = ids.reshape(-1).long().clamp_(max=e - 1)
         xr = x.unsqueeze(1).expand(t, k, h).reshape(n, h, 1)
         g = torch.bmm(w13.index_select(0, sel), xr).squeeze(2)
-        ys = torch.bmm(w2.index_select(0, sel), gated_act(g, kind, limit, alpha).unsqueeze(2)).squeeze(2).contiguous()
+        ys = torch.bmm(w2.index_select(0, sel), _expert_act(g, kind, limit, alpha).unsqueeze(2)).squeeze(2).contiguous()
         return finish(ys, None)
     # prompt-sized steps: rows sorted by expert (identity entries sort last and run nothing), one library GEMM pair
     # per real expert over its rows
@@ -341,7 +419,7 @@ def moe_output_weighted(x: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, w:
     for ei in range(e):
         a0, a1 = off[ei], off[ei + 1]
         if a1 > a0:
-            F.linear(gated_act(F.linear(xs[a0:a1], w13[ei]), kind, limit, alpha), w2[ei], out=ys[a0:a1])
+            F.linear(_expert_act(F.linear(xs[a0:a1], w13[ei]), kind, limit, alpha), w2[ei], out=ys[a0:a1])
     return finish(ys, pos)
 
 

@@ -221,6 +221,28 @@ def softmax_topk_corrected(z: torch.Tensor, k: int, correction: Optional[torch.T
     return (w / (w.sum(-1, keepdim=True) + 1e-20)).contiguous(), ids.to(torch.int32).contiguous()
 
 
+def grouped_topk(z: torch.Tensor, k: int, count: int, keep: int, scale: float):
+    """z [T, E] fp32 logits: softmax scores over all E; the ``keep`` of ``count`` equal groups of neighbours with the
+    largest single score stay open; the k largest open scores times ``scale`` (lowest index on ties)."""
+    s = torch.softmax(z.float(), -1)
+    c = s
+    if keep < count:
+        best = s.view(s.shape[0], count, -1).amax(-1)
+        open_ = torch.zeros_like(best, dtype=torch.bool)
+        open_.scatter_(1, torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :keep], True)
+        c = s.masked_fill(~open_.repeat_interleave(s.shape[1] // count, 1), -1.0)
+    ids = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :k]
+    return (scale * torch.gather(s, 1, ids)).contiguous(), ids.to(torch.int32).contiguous()
+
+
+ACT_RELU2 = 3
+
+
+def relu2_act(z: torch.Tensor) -> torch.Tensor:
+    r = torch.relu(z.float())
+    return (r * r).to(z.dtype)
+
+
 def moe_output_weighted(x, w13, w2, w, ids, kind, limit, alpha, extra=None, extra_gate=None) -> torch.Tensor:
     t, h = x.shape
     e_real = w13.shape[0]
@@ -231,7 +253,8 @@ def moe_output_weighted(x, w13, w2, w, ids, kind, limit, alpha, extra=None, extr
             if e >= e_real:
                 y = x[rows].float()
             else:
-                a = gated_act(torch.nn.functional.linear(x[rows], w13[e]), kind, limit, alpha)
+                z = torch.nn.functional.linear(x[rows], w13[e])
+                a = relu2_act(z) if kind == ACT_RELU2 else gated_act(z, kind, limit, alpha)
                 y = torch.nn.functional.linear(a, w2[e]).float()
             out[rows] += w[rows, j, None] * y
     if extra is not None:

@@ -358,13 +358,15 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
               bias: Optional[torch.Tensor], max_q: int, heads: int, kv_heads: int, dim: int, vdim: int, window: int,
               scale: float, impl: int = 0, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
               seg: int = 0, gate: Optional[torch.Tensor] = None, out_inv_freq: Optional[torch.Tensor] = None,
-              gate_mult: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+              gate_mult: float = 1.0, out: Optional[torch.Tensor] = None, sigmoid: bool = False,
+              head_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Grouped-query attention over the cache that :func:`qkv_prep` writes. The query at position p sees the cached
     positions j <= p with p - j < window (0: all) and, with ``seg`` > 0, of its own segment: floor(j / seg) =
     floor(p / seg). Score: s = (q . k_j) * scale; with ``softcap`` > 0,
     s <- softcap * tanh(s / softcap); then - slopes[h] * (p - j) (``slopes`` [H] fp32, a linear distance penalty)
     and + bias[min(p - j, rows - 1), h]. The softmax denominator has one more term exp(sink[h]) when ``sink`` is
-    given. Returns [T, H * vdim]. ``impl``: 0 = the matrix-core kernel where it applies, 1 = the FMA kernel, 2 = the
+    given. With ``sigmoid`` there is no softmax: every visible key weighs sigmoid(s + head_bias[h]) (``head_bias`` [H] fp32,
+    optional), whatever the others weigh, and there is no sink. Returns [T, H * vdim]. ``impl``: 0 = the matrix-core kernel where it applies, 1 = the FMA kernel, 2 = the
     matrix-core kernel or an error. ``gate`` [T, H] (any row stride): head h's output is turned back by its query's position
     (``out_inv_freq`` [vdim / 2], as :func:`src.ops.conv.rot_head_gate`) and multiplied by gate_mult * sigmoid(gate[t, h]) —
     in the launch that writes it for decode steps and split keys, else in one of its own — and ``out`` may be a slice of a
@@ -374,7 +376,8 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
         if out is None:
             out = torch.empty(T, heads * vdim, dtype=q.dtype, device=q.device)
         _kern().sink_attn(out, q, cache, block_tables, cu_q, ctx_lens, positions, sink, bias, max_q, heads, kv_heads,
-                          dim, vdim, window, scale, impl, float(softcap), slopes, int(seg), gate, out_inv_freq, float(gate_mult))
+                          dim, vdim, window, scale, impl, float(softcap), slopes, int(seg), gate, out_inv_freq, float(gate_mult), bool(sigmoid),
+                          head_bias)
         return out
     bs = cache.shape[1]
     hm = _head_major(cache, kv_heads)
@@ -404,6 +407,10 @@ def sink_attn(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, 
                 sc = sc - slopes[:, None] * n[None, :].float()
             if bias is not None:
                 sc = sc + bias[n.clamp(0, bias.shape[0] - 1)].T
+            if sigmoid:
+                sc = sc if head_bias is None else sc + head_bias[:, None]
+                res[t] = torch.einsum("hj,jhv->hv", torch.sigmoid(sc).masked_fill(~ok[None, :], 0.0), vv)
+                continue
             sc = sc.masked_fill(~ok[None, :], -math.inf)
             if sink is not None:
                 sc = torch.cat([sc, sink[:, None]], 1)

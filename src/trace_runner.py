@@ -61,7 +61,7 @@ def main(argv=None) -> int:
 
     family = family_of(a.model)
     # families on the dtype-generic kernels (src/_Cmix) alone
-    generic = family in ("datatar", "fekolorn", "bapivik", "kogerax", "rerozen")
+    generic = family in ("datatar", "fekolorn", "bapivik", "kogerax", "rerozen", "malapel")
     if not generic and a.dtype == "float32":
         print(f"the {family} kernels are bfloat16 only", file=sys.stderr)
         return 3
