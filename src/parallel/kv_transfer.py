@@ -232,7 +232,7 @@ class IPCLandingZone:
     Offsets are global over the segments (segment s covers [s * seg_bytes, (s + 1) * seg_bytes)); a slot
     never spans two. Each segment stays below 2 GiB: on this ROCm (7.2, dmabuf IPC) hipIpcOpenMemHandle of
     a 2 GiB allocation never returns in the importing process, while 256 MiB..1 GiB open in < 10 ms
-    (measured, scripts/repro_ipc_kv.py). The default 4 x 1 GiB holds 64 in-flight 512-token Llama-3-8B
+    (measured). The default 4 x 1 GiB holds 64 in-flight 512-token Llama-3-8B
     prompts: a whole bench wave of 32 (with one segment, half the wave waited for the other half's
     scatter)."""
 
