@@ -172,13 +172,6 @@ def forward(config: Dict[str, Any], weights: Dict[str, torch.Tensor], tokens: Li
     return norm1p(x, w["final.norm"], eps) @ w["head"].T
 
 
-def greedy(config, weights, prompt: List[int], n: int) -> List[int]:
-    toks = list(prompt)
-    for _ in range(n):
-        toks.append(int(forward(config, weights, toks)[-1].argmax()))
-    return toks[len(prompt):]
-
-
 # --------------------------------------------------------------------------------------- test configurations
 def _mixer(heads, kv_heads, dim, vdim, rot_dims, base, scale, size=None) -> Dict[str, Any]:
     m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale}
