@@ -479,7 +479,8 @@ hipError_t launch_conv_norm(const ConvNormArgs& a, RaggedRows r0, hipStream_t s)
     return a.W <= 64 * NT ? launch_cn<16, 4>(a, r, R, tiles, s) : hipErrorInvalidValue;
   }
   if (a.W <= 4 * NT) return launch_cn<4, 1>(a, r, R, tiles, s);
-  return a.W <= 16 * NT ? launch_cn<16, 1>(a, r, R, tiles, s) : hipErrorInvalidValue;
+  if (a.W <= 16 * NT) return launch_cn<16, 1>(a, r, R, tiles, s);
+  return a.W <= 64 * NT ? launch_cn<64, 1>(a, r, R, tiles, s) : hipErrorInvalidValue;
 }
 
 hipError_t launch_rot_head_gate(const RotHeadGateArgs& a, hipStream_t s) {

@@ -441,7 +441,7 @@ def test_unequal_requests_share_steps_and_pages_are_reused(tmp_path, device, dty
     requests sitting out steps, finished requests' pages handed to later ones. Every request's logits equal those of the
     request alone (the oracle)."""
     _need(device)
-    config = CONFIGS["std"]()
+    config = CONFIGS["std" if dtype == torch.float32 else "mc"]()
     weights = weights_for(config, 5)
     lens = {"a": 70, "b": 33, "c": 1, "d": 47, "e": 64, "f": 18}
     toks = {r: tokens_for(config, n, 10 + i) for i, (r, n) in enumerate(lens.items())}
