@@ -143,6 +143,10 @@ def parse(argv=None):
                    help="instead of the default workload: Rerozen beside Fekolorn (attention next to a linear recurrence) at "
                         "equal sizes, prefill / decode throughput and its kernels alone (bench/rerozen_compare.py)")
     p.add_argument("--rerozen-args", default="", help="arguments passed on to bench/rerozen_compare.py")
+    p.add_argument("--malapel-compare", action="store_true",
+                   help="instead of the default workload: Malapel beside Datatar (the same feed-forwards over an fp32 residual) "
+                        "at equal sizes, prefill / decode throughput and its kernels alone (bench/malapel_compare.py)")
+    p.add_argument("--malapel-args", default="", help="arguments passed on to bench/malapel_compare.py")
     return p.parse_args(argv)
 
 
@@ -518,6 +522,15 @@ def main(argv=None) -> int:
         mod = importlib.util.module_from_spec(spec)
         spec.loader.exec_module(mod)
         return mod.main(shlex.split(args.rerozen_args))
+    if args.malapel_compare:  # likewise a separate measurement
+        import importlib.util
+        import shlex
+
+        spec = importlib.util.spec_from_file_location("malapel_compare",
+                                                      os.path.join(ROOT, "bench", "malapel_compare.py"))
+        mod = importlib.util.module_from_spec(spec)
+        spec.loader.exec_module(mod)
+        return mod.main(shlex.split(args.malapel_args))
     if needs_launcher(args):
         return self_launch(args, argv)
     world = int(os.environ.get("WORLD_SIZE", "1"))

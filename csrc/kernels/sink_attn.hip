@@ -216,14 +216,17 @@ template <bool F32> hipError_t launch_fma(const SinkAttnArgs& a, hipStream_t s) 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 256, vdim % 8 == 0, vdim <= 256 (the
+// bf16 on the matrix cores (v_mfma_f32_32x32x16_bf16), for dim % 16 == 0, dim <= 256, vdim % 8 == 0, vdim <= 256 and pages of a
+// power of two tokens (the
 // value columns of a staged row are padded to a multiple of 32; what the padding holds only reaches output columns that
 // do not exist).
-// Workgroup = NW waves x 32 rows of one (sequence, key/value head); NW = 1 for steps of few rows (decode). Per tile
-// of 32 keys, staged once in LDS as rows [K_g | V_g] (the next tile's global loads in flight meanwhile):
-//   S^T[key][q] = K Q^T        A = K rows from LDS, B = Q rows from LDS      (dim / 16 MFMAs)
+// Workgroup = NW waves x 32 rows of one (sequence, key/value head); NW = 1 for steps of few rows (decode). Keys are staged
+// in LDS as rows [K_g | V_g], STG at a time in two buffers in turn: one barrier per stage, the next stage's global loads in
+// flight while this one is computed. Per tile of 32 keys:
+//   S^T[key][q] = K Q^T        A = K rows from LDS, B = Q rows               (dim / 16 MFMAs; dim <= 128: Q in registers)
 //   online softmax per query column (a lane pair owns a query), fp32 scores and weights in log2 units, the bias
-//   per distance added before, the running max seeded with the sink; P is rounded to bf16 only as MFMA operand
+//   per distance added before, the running max seeded with the sink; the max moves (and O is rescaled) only when a tile
+//   exceeds it by 2^LAZY; P is rounded to bf16 only as MFMA operand
 //   O^T[d][q] += V^T P^T      A = the value columns of the same tile read transposed (ds_read_tr16_b64),
 //                              B = P^T straight from the score accumulator   (2 * vdim / 32 MFMAs)
 // Split keys (decode over long contexts): split z takes keys [jlo + z * chunk, + chunk) and writes its
@@ -231,20 +234,26 @@ template <bool F32> hipError_t launch_fma(const SinkAttnArgs& a, hipStream_t s) 
 // split 0 only.
 constexpr int MKT = 32;
 constexpr int BT_LDS_MAX = 2048;
+constexpr float LAZY = 8.0f;
+// keys per stage; whether the queries live in registers (else in LDS)
+template <int NW, int NKC> constexpr int stage_keys() { return NW == 4 && NKC <= 16 ? 64 : MKT; }
+template <int NDB, int NW, int NKC> constexpr bool q_in_regs() { return NKC <= 16 && (NW == 4 || NDB <= 4); }
 typedef __attribute__((address_space(3))) short4_t lds_short4;
 typedef __attribute__((ext_vector_type(8))) short short8_t;
 
 template <int NDB, int NW, int NKC, bool SIG>
-__global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a, int KP, int QP, int QR, int BTC,
+__global__ void __launch_bounds__(64 * NW, NW == 4 && NKC <= 16 && NDB <= 4 ? 2 : 1) sink_attn_mfma_kernel(SinkAttnArgs a, int KP, int QP, int QR, int BTC,
                                                                 float* ws_o, float* ws_ml, int nsplit, int chunk) {
-  constexpr int ROWS = 32 * NW, NT = 64 * NW;
-  constexpr int NPF = (MKT * (4 * NDB + NKC) + NT - 1) / NT;  // 16-byte chunks of a key tile per thread
+  constexpr int ROWS = 32 * NW, NT = 64 * NW, STG = stage_keys<NW, NKC>();
+  constexpr bool QREG = q_in_regs<NDB, NW, NKC>();
+  constexpr int NKK = QREG ? NKC / 2 : 1;                     // steps of 16 dims of a query held in registers
+  constexpr int NPF = (STG * (4 * NDB + NKC) + NT - 1) / NT;  // 16-byte chunks of a stage per thread
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
-  // QR query rows are staged: all ROWS of a prompt-sized step; for steps of few rows (NW = 1) only the rows there
+  // QR query rows are staged (none with QREG): all ROWS of a prompt-sized step; for steps of few rows (NW = 1) only the rows there
   // can be plus one zero row that every further query column reads, which keeps the workgroup's LDS small enough
   // for two waves per SIMD
   bf16_t* qs = reinterpret_cast<bf16_t*>(smem_raw);          // [QR][QP]
-  bf16_t* ks = qs + QR * QP;                                  // [MKT][KP] = [K_g | V_g]
+  bf16_t* ks = qs + QR * QP;                                  // two of [STG][KP] = [K_g | V_g]
   int bx = blockIdx.x, by = blockIdx.y;
   {
     // XCD k (workgroups are dealt round-robin by linear id) takes a contiguous eighth of the sequence-major tile
@@ -255,6 +264,7 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
       bx = (int)(nl % gridDim.x);
       by = (int)(nl / gridDim.x);
     }
+    bx = gridDim.x - 1 - bx;   // a sequence's last rows see the most keys: they start first
   }
   const int H = a.heads, G = a.kv_heads, QPG = H / G, D = a.dim, DV = a.vdim;
   const int s = by, g = blockIdx.z % G, z = blockIdx.z / G;
@@ -289,23 +299,36 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
     return;
   }
 
-  const int lch = D / 8;
-  for (int idx = tid; idx < QR * lch; idx += NT) {
-    const int r = idx / lch, c = idx % lch, row = row0 + r;
-    uint4 v = make_uint4(0, 0, 0, 0);
-    if (row < nrows) {
-      const int64_t t = q0 + row / QPG;
-      v = *reinterpret_cast<const uint4*>(qg + (t * H + g * QPG + row % QPG) * D + 8 * c);
+  const int nkk = D / 16;
+  bf16x8_t qf[NKK];
+  if constexpr (QREG) {
+#pragma unroll
+    for (int kk = 0; kk < NKK; ++kk) {
+      uint4 v = make_uint4(0, 0, 0, 0);
+      if (rok && kk < nkk) v = *reinterpret_cast<const uint4*>(qg + orow * D + 16 * kk + 8 * hh);
+      qf[kk] = __builtin_bit_cast(bf16x8_t, v);
     }
-    *reinterpret_cast<uint4*>(qs + r * QP + 8 * c) = v;
+  } else {
+    const int lch = D / 8;
+    for (int idx = tid; idx < QR * lch; idx += NT) {
+      const int r = idx / lch, c = idx % lch, row = row0 + r;
+      uint4 v = make_uint4(0, 0, 0, 0);
+      if (row < nrows) {
+        const int64_t t = q0 + row / QPG;
+        v = *reinterpret_cast<const uint4*>(qg + (t * H + g * QPG + row % QPG) * D + 8 * c);
+      }
+      *reinterpret_cast<uint4*>(qs + r * QP + 8 * c) = v;
+    }
   }
 
   const bool wave_live = row0 + wave * 32 < nrows;
   const int prow = rok ? (int)a.positions[q0 + myrow / QPG] : -1;
   const int jrow = first_key(a, max(prow, 0));
+  const unsigned seen = rok ? max(min(prow, jhi) - jrow + 1, 0) : 0;   // this row sees keys jrow .. jrow + seen - 1
   constexpr float LOG2E = 1.4426950408889634f;
   const float sl2 = a.scale * LOG2E;
   const bool shaped = a.softcap > 0.f || a.slopes != nullptr;
+  const bool plain = !shaped && a.bias == nullptr && sl2 > 0.f;
   const float capl2 = a.softcap * LOG2E, s_over_cap = a.softcap > 0.f ? a.scale / a.softcap : 0.f;
   const float cap_m2 = -2.0f * capl2, s2_over_cap = s_over_cap * 2.885390081777927f;
   const float slope2 = a.slopes != nullptr ? a.slopes[myh] * LOG2E : 0.f;
@@ -320,29 +343,30 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
     for (int r = 0; r < 16; ++r) o[db][r] = 0.f;
 
   const int* bt = a.block_tables + (int64_t)s * a.bt_stride;
-  const int kch = (D + DV) / 8, nkk = D / 16;
-  int* btl = reinterpret_cast<int*>(ks + MKT * KP);
+  const int kch = (D + DV) / 8;
+  bf16_t* spare = ks + 2 * STG * KP;   // [KP]: takes a stage's surplus chunks
+  int* btl = reinterpret_cast<int*>(spare + KP);
   const int b_lo = jlo / a.block_size, nbt = jhi / a.block_size - b_lo + 1;
   const bool bt_lds = nbt <= BTC;
   if (bt_lds)
     for (int u = tid; u < nbt; u += NT) btl[u] = bt[b_lo + u];
-  uint4 pf[NPF];
+  u32x4_t pf[NPF];   // (native vectors: arrays of uint4 structs go through scratch)
   // chunk idx = tid + u * NT of a tile is (key k, 16-byte piece c) = (idx / kch, idx % kch): one division per
   // thread, then steps of (NT / kch, NT % kch); a block size that is a power of two divides by shifting
   const int k_first = tid / kch, c_first = tid - k_first * kch, k_step = NT / kch, c_step = NT - k_step * kch;
-  const int bs_shift = (a.block_size & (a.block_size - 1)) == 0 ? __builtin_ctz(a.block_size) : -1;
+  const int bs_shift = __builtin_ctz(a.block_size);   // a power of two (mfma_ok)
+  const uint32_t rowb = 2 * roww, blkb = (uint32_t)G * a.block_size * rowb;
+  const char* cg = reinterpret_cast<const char*>(cache) + (int64_t)g * a.block_size * rowb;
+  // all block ids first, then all loads: no load waits for another's block id. Keys beyond the last re-read it: their
+  // scores are masked
   auto fetch = [&](int j0, bool lds) {
+    int jj[NPF], cc[NPF];
+    uint32_t blk[NPF];
     int k = k_first, c = c_first;
 #pragma unroll
     for (int u = 0; u < NPF; ++u) {
-      const int j = j0 + k;
-      pf[u] = make_uint4(0, 0, 0, 0);
-      if (k < MKT && j <= jhi) {
-        const int jb = bs_shift >= 0 ? j >> bs_shift : j / a.block_size;
-        const int64_t blk = lds ? btl[jb - b_lo] : bt[jb];
-        const int64_t rowp = ((blk * G + g) * a.block_size + (j - jb * a.block_size)) * roww;
-        pf[u] = *reinterpret_cast<const uint4*>(cache + rowp + 8 * c);
-      }
+      jj[u] = min(j0 + min(k, STG - 1), jhi);
+      cc[u] = c;
       k += k_step;
       c += c_step;
       if (c >= kch) {
@@ -350,12 +374,23 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
         ++k;
       }
     }
+    if (lds) {
+#pragma unroll
+      for (int u = 0; u < NPF; ++u) blk[u] = btl[(jj[u] >> bs_shift) - b_lo];
+    } else {
+#pragma unroll
+      for (int u = 0; u < NPF; ++u) blk[u] = bt[jj[u] >> bs_shift];
+    }
+#pragma unroll
+    for (int u = 0; u < NPF; ++u) {
+      const uint32_t in = (uint32_t)(jj[u] & (a.block_size - 1)) * rowb + 16 * cc[u];
+      pf[u] = *reinterpret_cast<const u32x4_t*>(cg + (uint64_t)blk[u] * blkb + in);
+    }
   };
   fetch(jlo, false);
   const int pitchB = KP * 2;
   const int g16 = lane >> 4, i16 = lane & 15;
-  const char* vbase = reinterpret_cast<const char*>(ks) + (4 * hh + (i16 >> 2)) * pitchB +
-                      (D + 16 * (g16 & 1) + 4 * (i16 & 3)) * 2;
+  const int voff = (4 * hh + (i16 >> 2)) * pitchB + (D + 16 * (g16 & 1) + 4 * (i16 & 3)) * 2;
   const float* bias = a.bias ? a.bias + myh : nullptr;
   // distances from bias_rows - 1 on share the table's last row: a lane whose 16 keys of a tile all lie that far
   // back adds that one value without looking anything up
@@ -366,13 +401,14 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
   const int pw_first = wave_live ? (int)a.positions[q0 + wrow_first / QPG] : 0;
   const int pw_last = wave_live ? (int)a.positions[q0 + min(wrow_last, nrows - 1) / QPG] : 0;
   const int jw_first = first_key(a, pw_first), jw_last = first_key(a, pw_last);
-  for (int j0 = jlo; j0 <= jhi; j0 += MKT) {
-    __syncthreads();  // every wave is done with the previous tile (first: the queries are being written)
+  int buf = 0;
+  for (int js = jlo; js <= jhi; js += STG, buf ^= 1) {
+    bf16_t* kst = ks + buf * STG * KP;   // last read two stages ago: every wave has passed a barrier since
     {
       int k = k_first, c = c_first;
 #pragma unroll
       for (int u = 0; u < NPF; ++u) {
-        if (k < MKT) *reinterpret_cast<uint4*>(ks + k * KP + 8 * c) = pf[u];
+        *reinterpret_cast<u32x4_t*>((k < STG ? kst + k * KP : spare) + 8 * c) = pf[u];
         k += k_step;
         c += c_step;
         if (c >= kch) {
@@ -382,128 +418,185 @@ __global__ void __launch_bounds__(64 * NW) sink_attn_mfma_kernel(SinkAttnArgs a,
       }
     }
     __syncthreads();
-    if (j0 + MKT <= jhi) fetch(j0 + MKT, bt_lds);  // in flight while this tile is computed
-    if (!wave_live || j0 > pw_last || j0 + MKT <= jw_first) continue;   // nothing of this tile is visible to the wave
-    f32x16_t sc;
+    if (js + STG <= jhi) fetch(js + STG, bt_lds);  // in flight while this stage is computed
+    for (int j0 = js; j0 < js + STG && j0 <= jhi; j0 += MKT) {
+      if (!wave_live || j0 > pw_last || j0 + MKT <= jw_first) continue;   // nothing of this tile is visible to the wave
+      const bf16_t* kt = kst + (j0 - js) * KP;
+      const char* vbase = reinterpret_cast<const char*>(kt) + voff;
+      f32x16_t sc;
 #pragma unroll
-    for (int r = 0; r < 16; ++r) sc[r] = 0.f;
-    const bf16_t* ka = ks + qcol * KP + 8 * hh;
-    const bf16_t* qb = qs + min(wave * 32 + qcol, QR - 1) * QP + 8 * hh;
-    for (int kk = 0; kk < nkk; ++kk) {
-      const bf16x8_t af = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const uint4*>(ka + 16 * kk));
-      const bf16x8_t bfr = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const uint4*>(qb + 16 * kk));
-      sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(af, bfr, sc, 0, 0, 0);
-    }
-    float mx = -INFINITY;
-    const bool interior = wave_full && j0 + MKT - 1 <= min(pw_first, jhi) && j0 >= jw_last;
-    if (shaped) {
-      // capped scores and / or a linear distance penalty: cap * tanh(s * scale / cap) - slope * n, in log2 units.
-      // tanh = 1 - 2 / (2^(2 x log2 e) + 1), so the capped score is one multiply-add of the reciprocal; the
-      // distance of score r is that of score 0 minus a constant
-      const float nf0 = (float)(prow - j0 - 4 * hh);
-      if (interior && bias == nullptr) {
+      for (int r = 0; r < 16; ++r) sc[r] = 0.f;
+      const bf16_t* ka = kt + qcol * KP + 8 * hh;
+      if constexpr (QREG) {
+        // all NKK steps without a branch between them, so that their LDS reads are in flight together: beyond dim the
+        // query's fragments are zero, and the key's first columns stand in
+        bf16x8_t kf[NKK];
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          const float nf = nf0 - (float)((r & 3) + 8 * (r >> 2));
-          float v;
-          if (a.softcap > 0.f)
-            v = fmaf(cap_m2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[r] * s2_over_cap) + 1.0f), capl2);
-          else
-            v = sc[r] * sl2;
-          v = fmaf(-slope2, nf, v);
-          sc[r] = v;
-          mx = fmaxf(mx, v);
+        for (int kk = 0; kk < NKK; ++kk)
+          kf[kk] = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const u32x4_t*>(ka + (kk < nkk ? 16 * kk : 0)));
+#pragma unroll
+        for (int kk = 0; kk < NKK; ++kk) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[kk], qf[kk], sc, 0, 0, 0);
+      } else {
+        const bf16_t* qb = qs + min(wave * 32 + qcol, QR - 1) * QP + 8 * hh;
+#pragma unroll 4
+        for (int kk = 0; kk < nkk; ++kk) {
+          const bf16x8_t af = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const uint4*>(ka + 16 * kk));
+          const bf16x8_t bfr = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const uint4*>(qb + 16 * kk));
+          sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(af, bfr, sc, 0, 0, 0);
+        }
+      }
+      float mx = -INFINITY, mul = 1.0f;   // sc * mul: scores in log2 units
+      const bool interior = wave_full && j0 + MKT - 1 <= min(pw_first, jhi) && j0 >= jw_last;
+      if (plain) {
+        mul = sl2;
+        if (!interior) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r)
+            sc[r] = (unsigned)(j0 + (r & 3) + 8 * (r >> 2) + 4 * hh - jrow) < seen ? sc[r] : -INFINITY;
+        }
+        if constexpr (!SIG) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) mx = fmaxf(mx, sc[r]);
+          mx *= sl2;
+        }
+      } else if (shaped) {
+        // capped scores and / or a linear distance penalty: cap * tanh(s * scale / cap) - slope * n, in log2 units.
+        // tanh = 1 - 2 / (2^(2 x log2 e) + 1), so the capped score is one multiply-add of the reciprocal; the
+        // distance of score r is that of score 0 minus a constant
+        const float nf0 = (float)(prow - j0 - 4 * hh);
+        if (interior && bias == nullptr) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const float nf = nf0 - (float)((r & 3) + 8 * (r >> 2));
+            float v;
+            if (a.softcap > 0.f)
+              v = fmaf(cap_m2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[r] * s2_over_cap) + 1.0f), capl2);
+            else
+              v = sc[r] * sl2;
+            v = fmaf(-slope2, nf, v);
+            sc[r] = v;
+            mx = fmaxf(mx, v);
+          }
+        } else {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const int j = j0 + (r & 3) + 8 * (r >> 2) + 4 * hh;
+            const int n = prow - j;
+            const bool valid = interior || (rok && j <= jhi && n >= 0 && j >= jrow);
+            float v = a.softcap > 0.f ? capl2 * fast_tanh(sc[r] * s_over_cap) : sc[r] * sl2;
+            v -= slope2 * (float)n;
+            if (bias != nullptr && valid) v += bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
+            v = valid ? v : -INFINITY;
+            sc[r] = v;
+            mx = fmaxf(mx, v);
+          }
+        }
+      } else if (interior) {
+        const bool far = bias == nullptr || prow - (j0 + 27 + 4 * hh) >= a.bias_rows - 1;
+        if (far) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const float v = sc[r] * sl2 + bias_far;
+            sc[r] = v;
+            mx = fmaxf(mx, v);
+          }
+        } else {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const int n = prow - (j0 + (r & 3) + 8 * (r >> 2) + 4 * hh);
+            const float v = sc[r] * sl2 + bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
+            sc[r] = v;
+            mx = fmaxf(mx, v);
+          }
         }
       } else {
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int j = j0 + (r & 3) + 8 * (r >> 2) + 4 * hh;
           const int n = prow - j;
-          const bool valid = interior || (rok && j <= jhi && n >= 0 && j >= jrow);
-          float v = a.softcap > 0.f ? capl2 * fast_tanh(sc[r] * s_over_cap) : sc[r] * sl2;
-          v -= slope2 * (float)n;
+          const bool valid = rok && j <= jhi && n >= 0 && j >= jrow;
+          float v = sc[r] * sl2;
           if (bias != nullptr && valid) v += bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
           v = valid ? v : -INFINITY;
           sc[r] = v;
           mx = fmaxf(mx, v);
         }
       }
-    } else if (interior) {
-      const bool far = bias == nullptr || prow - (j0 + 27 + 4 * hh) >= a.bias_rows - 1;
-      if (far) {
+      float alpha = 1.0f;
+      if constexpr (SIG) {
+        // sigmoid: 1 / (1 + 2^-(v + bias)); a masked score is -inf and weighs 0
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          const float v = sc[r] * sl2 + bias_far;
-          sc[r] = v;
-          mx = fmaxf(mx, v);
-        }
+        for (int r = 0; r < 16; ++r) sc[r] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(-sc[r], mul, -hb2)));
       } else {
+        mx = xor32_max(mx);
+        const float mn = mx > m + LAZY ? mx : m;
+        alpha = __builtin_amdgcn_exp2f(m - mn);   // v_exp_f32: arguments are <= 0 or -inf here
+        float sum = 0.f;
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
-          const int n = prow - (j0 + (r & 3) + 8 * (r >> 2) + 4 * hh);
-          const float v = sc[r] * sl2 + bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
-          sc[r] = v;
-          mx = fmaxf(mx, v);
+          const float pe = __builtin_amdgcn_exp2f(fmaf(sc[r], mul, -mn));
+          sc[r] = pe;
+          sum += pe;
         }
+        sum = xor32_sum(sum);
+        l = l * alpha + sum;
+        m = mn;
       }
-    } else {
-#pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        const int j = j0 + (r & 3) + 8 * (r >> 2) + 4 * hh;
-        const int n = prow - j;
-        const bool valid = rok && j <= jhi && n >= 0 && j >= jrow;
-        float v = sc[r] * sl2;
-        if (bias != nullptr && valid) v += bias[(int64_t)min(n, a.bias_rows - 1) * H] * LOG2E;
-        v = valid ? v : -INFINITY;
-        sc[r] = v;
-        mx = fmaxf(mx, v);
-      }
-    }
-    float alpha = 1.0f;
-    if constexpr (SIG) {
-      // sigmoid: 1 / (1 + 2^-(v + bias)); a masked score is -inf and weighs 0
-#pragma unroll
-      for (int r = 0; r < 16; ++r) sc[r] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-hb2 - sc[r]));
-    } else {
-      mx = xor32_max(mx);
-      const float mn = fmaxf(m, mx);
-      alpha = __builtin_amdgcn_exp2f(m - mn);   // v_exp_f32: arguments are <= 0 or -inf here
-      float sum = 0.f;
-#pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        const float pe = __builtin_amdgcn_exp2f(sc[r] - mn);
-        sc[r] = pe;
-        sum += pe;
-      }
-      sum = xor32_sum(sum);
-      l = l * alpha + sum;
-      m = mn;
-    }
-    bf16x8_t pfr[2];
-#pragma unroll
-    for (int s2 = 0; s2 < 2; ++s2) {
-      uint4 w;
-      w.x = pack2(sc[8 * s2 + 0], sc[8 * s2 + 1]);
-      w.y = pack2(sc[8 * s2 + 2], sc[8 * s2 + 3]);
-      w.z = pack2(sc[8 * s2 + 4], sc[8 * s2 + 5]);
-      w.w = pack2(sc[8 * s2 + 6], sc[8 * s2 + 7]);
-      pfr[s2] = __builtin_bit_cast(bf16x8_t, w);
-    }
-#pragma unroll
-    for (int db = 0; db < NDB; ++db) {
-      if (!SIG && alpha != 1.0f) {
-#pragma unroll
-        for (int r = 0; r < 16; ++r) o[db][r] *= alpha;
-      }
+      bf16x8_t pfr[2];
 #pragma unroll
       for (int s2 = 0; s2 < 2; ++s2) {
-        const char* a0 = vbase + (16 * s2) * pitchB + 64 * db;
-        const short4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(a0));
-        const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(a0 + 8 * pitchB));
-        const short8_t a8 = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-        o[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a8), pfr[s2], o[db], 0, 0, 0);
+        uint4 w;
+        w.x = pack2(sc[8 * s2 + 0], sc[8 * s2 + 1]);
+        w.y = pack2(sc[8 * s2 + 2], sc[8 * s2 + 3]);
+        w.z = pack2(sc[8 * s2 + 4], sc[8 * s2 + 5]);
+        w.w = pack2(sc[8 * s2 + 6], sc[8 * s2 + 7]);
+        pfr[s2] = __builtin_bit_cast(bf16x8_t, w);
+      }
+#pragma unroll
+      for (int db = 0; db < NDB; ++db) {
+        if (!SIG && alpha != 1.0f) {
+#pragma unroll
+          for (int r = 0; r < 16; ++r) o[db][r] *= alpha;
+        }
+#pragma unroll
+        for (int s2 = 0; s2 < 2; ++s2) {
+          const char* a0 = vbase + (16 * s2) * pitchB + 64 * db;
+          const short4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(a0));
+          const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(a0 + 8 * pitchB));
+          const short8_t a8 = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+          o[db] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a8), pfr[s2], o[db], 0, 0, 0);
+        }
       }
     }
+  }
+  if (NW > 1 && nsplit <= 1) {
+    // whole rows of 16-byte pieces through LDS: straight from the accumulators every store would touch 32 rows
+    const float inv = SIG ? 1.0f : (l > 0.f ? 1.0f / l : 0.f);
+    const int OP = 2 * (DV + 8);
+    char* ob = smem_raw + wave * 32 * OP;
+    __syncthreads();   // every wave is done with the keys
+#pragma unroll
+    for (int db = 0; db < NDB; ++db) {
+#pragma unroll
+      for (int q4 = 0; q4 < 4; ++q4) {
+        if (32 * db + 8 * q4 >= DV) continue;
+        uint2 w;
+        w.x = pack2(o[db][4 * q4 + 0] * inv, o[db][4 * q4 + 1] * inv);
+        w.y = pack2(o[db][4 * q4 + 2] * inv, o[db][4 * q4 + 3] * inv);
+        *reinterpret_cast<uint2*>(ob + qcol * OP + 2 * (32 * db + 8 * q4 + 4 * hh)) = w;
+      }
+    }
+    __syncthreads();
+    const int nch = DV / 8;
+    bf16_t* og = reinterpret_cast<bf16_t*>(a.out);
+    for (int idx = lane; idx < 32 * nch; idx += 64) {
+      const int r = idx / nch, c = idx - r * nch, row = row0 + wave * 32 + r;
+      if (row >= nrows) break;
+      const int t = row / QPG;
+      const uint4 w = *reinterpret_cast<const uint4*>(ob + r * OP + 16 * c);
+      *reinterpret_cast<uint4*>(og + ((int64_t)(q0 + t) * H + g * QPG + (row - t * QPG)) * DV + 8 * c) = w;
+    }
+    return;
   }
   if (!rok) return;
   if (nsplit > 1) {
@@ -779,11 +872,11 @@ template <int NDB, int NW, int NKC, bool SIG> hipError_t launch_mfma(const SinkA
   auto* fn = sink_attn_mfma_kernel<NDB, NW, NKC, SIG>;
   const int kp = a.dim + 32 * NDB + 8, qp = a.dim + 8;
   const int qpg0 = a.heads / a.kv_heads;
-  const int qr = NW == 1 ? min(32, a.max_q * qpg0 + 1) : 32 * NW;
+  const int qr = q_in_regs<NDB, NW, NKC>() ? 0 : (NW == 1 ? min(32, a.max_q * qpg0 + 1) : 32 * NW);
   const int nsp = a.ws_o != nullptr ? max(1, a.nsplit) : 1;
   // block-table entries staged per workgroup: its key range's (else they are read from global memory)
   const int btc = min(BT_LDS_MAX, (nsp > 1 ? a.chunk / a.block_size + 2 : a.bt_stride) + 1);
-  const size_t lds = sizeof(bf16_t) * ((size_t)qr * qp + (size_t)MKT * kp) + sizeof(int) * btc;
+  const size_t lds = sizeof(bf16_t) * ((size_t)qr * qp + (size_t)(2 * stage_keys<NW, NKC>() + 1) * kp) + sizeof(int) * btc;
   if (lds > 150 * 1024) return hipErrorInvalidValue;
   if (lds > 48 * 1024) {  // only then: the limit is raised per function, and a raised limit is not free
     static size_t raised = 0;
@@ -873,9 +966,10 @@ inline bool decode_ok(const SinkAttnArgs& a) {
 }
 
 inline bool mfma_ok(const SinkAttnArgs& a) {
-  return !a.f32 && a.dim % 16 == 0 && a.dim <= 256 && a.vdim % 8 == 0 && a.vdim <= 256 &&
+  return !a.f32 && (a.block_size & (a.block_size - 1)) == 0 && a.dim % 16 == 0 && a.dim <= 256 && a.vdim % 8 == 0 && a.vdim <= 256 &&
          (reinterpret_cast<uintptr_t>(a.q) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.cache) & 15) == 0 &&
-         (reinterpret_cast<uintptr_t>(a.out) & 7) == 0;
+         (reinterpret_cast<uintptr_t>(a.out) & 15) == 0 &&
+         (int64_t)a.kv_heads * a.block_size * (a.dim + a.vdim) * 2 < (1ll << 32);
 }
 
 }  // namespace
