@@ -56,40 +56,67 @@ __global__ void __launch_bounds__(NT) rms_norm_ext_kernel(void* out, int64_t ost
 
 __device__ __forceinline__ bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
+// eight fp32 weights from 8 c on, or ones
+__device__ __forceinline__ void load_w8(const float* w, int c, float* g) {
+  if (w == nullptr) {
+#pragma unroll
+    for (int q = 0; q < 8; ++q) g[q] = 1.0f;
+    return;
+  }
+  const float4 a = reinterpret_cast<const float4*>(w)[2 * c], b = reinterpret_cast<const float4*>(w)[2 * c + 1];
+  g[0] = a.x, g[1] = a.y, g[2] = a.z, g[3] = a.w, g[4] = b.x, g[5] = b.y, g[6] = b.z, g[7] = b.w;
+}
+
 // resid[t] (fp32) = rmsnorm(embed[ids[t]]) * w (fp32 weights; nullptr: the plain vectors' norm), copy[t] (optional, the
 // table's type, row stride cstride) = the same
 __global__ void __launch_bounds__(NT) embed_norm_kernel(float* resid, void* copy, int64_t cstride, const void* embed,
                                                        bool f32, const int64_t* ids, const float* w, float eps, int W) {
   __shared__ float red[NT / 64];
   const int64_t t = blockIdx.x, base = ids[t] * (int64_t)W;
-  if (!f32 && W % 8 == 0 && cstride % 8 == 0 && aligned16(embed) && aligned16(resid) && aligned16(w) && aligned16(copy)) {
-    const uint4* er = reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(embed) + base);
-    float ss = 0.f;
-    for (int c = threadIdx.x; c < W / 8; c += NT) {
-      float f[8];
-      unpack8(er[c], f);
-#pragma unroll
-      for (int q = 0; q < 8; ++q) ss += f[q] * f[q];
-    }
-    ss = block_sum<NT>(ss, red);
-    const float rs = 1.0f / sqrtf(ss / (float)W + eps);
-    float4* rr = reinterpret_cast<float4*>(resid + t * W);
-    for (int c = threadIdx.x; c < W / 8; c += NT) {
-      float f[8];
-      unpack8(er[c], f);
-#pragma unroll
-      for (int q = 0; q < 8; ++q) f[q] *= w != nullptr ? rs * w[8 * c + q] : rs;
-      rr[2 * c] = make_float4(f[0], f[1], f[2], f[3]);
-      rr[2 * c + 1] = make_float4(f[4], f[5], f[6], f[7]);
-      if (copy) reinterpret_cast<uint4*>(reinterpret_cast<bf16_t*>(copy) + t * cstride)[c] = pack8(f);
-    }
-    return;
-  }
   const float rs = row_rs(embed, base, f32, W, eps, red);
   for (int c = threadIdx.x; c < W; c += NT) {
     const float v = ldv(embed, base + c, f32) * (w != nullptr ? rs * w[c] : rs);
     resid[t * W + c] = v;
     if (copy) stv(copy, t * cstride + c, f32, v);
+  }
+}
+
+// the same for bf16 tables of a multiple of 8 columns, up to 512 CH: a wave per token, its row in registers, no barrier
+template <int CH>
+__global__ void __launch_bounds__(NT) embed_norm_wave_kernel(float* resid, bf16_t* copy, int64_t cstride, const bf16_t* embed,
+                                                            const int64_t* ids, const float* w, float eps, int T, int W) {
+  const int64_t t = (int64_t)blockIdx.x * (NT / 64) + (threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63, n8 = W / 8;
+  if (t >= T) return;
+  const u32x4_t* er = reinterpret_cast<const u32x4_t*>(embed + ids[t] * (int64_t)W);
+  u32x4_t x[CH];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int c = lane + 64 * i;
+    x[i] = c < n8 ? er[c] : u32x4_t{0, 0, 0, 0};
+  }
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    float f[8];
+    unpack8(__builtin_bit_cast(uint4, x[i]), f);
+#pragma unroll
+    for (int q = 0; q < 8; ++q) ss += f[q] * f[q];
+  }
+  const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)W + eps);
+  float4* rr = reinterpret_cast<float4*>(resid + t * W);
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int c = lane + 64 * i;
+    if (c >= n8) break;
+    float f[8], g[8];
+    unpack8(__builtin_bit_cast(uint4, x[i]), f);
+    load_w8(w, c, g);
+#pragma unroll
+    for (int q = 0; q < 8; ++q) f[q] *= rs * g[q];
+    rr[2 * c] = make_float4(f[0], f[1], f[2], f[3]);
+    rr[2 * c + 1] = make_float4(f[4], f[5], f[6], f[7]);
+    if (copy) reinterpret_cast<uint4*>(copy + t * cstride)[c] = pack8(f);
   }
 }
 
@@ -627,13 +654,14 @@ __global__ void __launch_bounds__(NT) combine_weighted_kernel(float* out, float*
     else
       __syncthreads();
     if (vec && w_f32 && astride % 8 == 0 && aligned16(w) && aligned16(act)) {
+      const float one = unit && w != nullptr ? 1.0f : 0.f;
       for (int c = threadIdx.x; c < H / 8; c += NT) {
-        float o[8];
+        const float4 u0 = *reinterpret_cast<const float4*>(acc + 8 * c), u1 = *reinterpret_cast<const float4*>(acc + 8 * c + 4);
+        const float u[8] = {u0.x, u0.y, u0.z, u0.w, u1.x, u1.y, u1.z, u1.w};
+        float o[8], g[8];
+        load_w8(reinterpret_cast<const float*>(w), c, g);
 #pragma unroll
-        for (int q = 0; q < 8; ++q) {
-          const float g = w != nullptr ? reinterpret_cast<const float*>(w)[8 * c + q] : 1.0f;
-          o[q] = acc[8 * c + q] * rs * (unit && w != nullptr ? g + 1.0f : g);
-        }
+        for (int q = 0; q < 8; ++q) o[q] = u[q] * rs * (g[q] + one);
         reinterpret_cast<uint4*>(reinterpret_cast<bf16_t*>(act) + t * astride)[c] = pack8(o);
       }
       return;
@@ -832,6 +860,14 @@ hipError_t launch_embed_norm(float* resid, void* copy, int64_t cstride, const vo
                              const float* w, float eps, int T, int W, hipStream_t s) {
   if (T == 0) return hipSuccess;
   if (W < 1 || resid == nullptr || (copy != nullptr && cstride < W)) return hipErrorInvalidValue;
+  auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (!f32 && W % 8 == 0 && W <= 4096 && cstride % 8 == 0 && a16(embed) && a16(resid) && a16(w) && a16(copy)) {
+    auto* fn = W <= 512 ? embed_norm_wave_kernel<1>
+                        : (W <= 1024 ? embed_norm_wave_kernel<2> : (W <= 2048 ? embed_norm_wave_kernel<4> : embed_norm_wave_kernel<8>));
+    hipLaunchKernelGGL(fn, dim3((T + NT / 64 - 1) / (NT / 64)), dim3(NT), 0, s, resid, reinterpret_cast<bf16_t*>(copy), cstride,
+                       reinterpret_cast<const bf16_t*>(embed), ids, w, eps, T, W);
+    return hipGetLastError();
+  }
   hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(NT), 0, s, resid, copy, cstride, embed, f32, ids, w, eps, W);
   return hipGetLastError();
 }

@@ -975,11 +975,32 @@ __global__ void __launch_bounds__(NT) qkv_prep_kernel(QkvPrepArgs a) {
       }
     }
   } else if (a.q_norm != nullptr) {   // over the whole projection (R == 1)
-    sq = block_sum<NT>(sq, red);   // (a barrier: every thread's loads are in LDS)
-    sk = block_sum<NT>(sk, red);
+    __shared__ float redk[NT / 64];
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((threadIdx.x & 63) == 0) {
+      red[threadIdx.x >> 6] = sq;
+      redk[threadIdx.x >> 6] = sk;
+    }
+    __syncthreads();   // (every thread's loads are in LDS, too)
+    sq = sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < NT / 64; ++i) {
+      sq += red[i];
+      sk += redk[i];
+    }
     const float rq = 1.0f / sqrtf(sq / (float)nq + a.eps), rk = 1.0f / sqrtf(sk / (float)nk + a.eps);
-    for (int c = threadIdx.x; c < nq; c += NT) qv[c] *= rq * a.q_norm[c];
-    for (int c = threadIdx.x; c < nk; c += NT) kv[c] *= rk * a.k_norm[c];
+    if (((nq | nk) & 3) == 0 && aligned16(a.q_norm) && aligned16(a.k_norm)) {
+      for (int c = 4 * threadIdx.x; c < nq + nk; c += 4 * NT) {   // (qv and kv are adjacent)
+        const float4 x = *reinterpret_cast<const float4*>(qv + c);
+        const float4 ww = *reinterpret_cast<const float4*>(c < nq ? a.q_norm + c : a.k_norm + (c - nq));
+        const float rs = c < nq ? rq : rk;
+        *reinterpret_cast<float4*>(qv + c) = make_float4(x.x * rs * ww.x, x.y * rs * ww.y, x.z * rs * ww.z, x.w * rs * ww.w);
+      }
+    } else {
+      for (int c = threadIdx.x; c < nq; c += NT) qv[c] *= rq * a.q_norm[c];
+      for (int c = threadIdx.x; c < nk; c += NT) kv[c] *= rk * a.k_norm[c];
+    }
   }
   __syncthreads();
   if (a.q_temp_coef != 0.f && !per_head) {
