@@ -345,7 +345,7 @@ def test_attention_edges_and_far_keys(device, kind, where, size, standout, rows)
         cases += [(torch.bfloat16, {"impl": 2}), (torch.bfloat16, {"D": 96, "V": 160, "R": 24}),
                   (torch.bfloat16, {"D": 256, "V": 256, "R": 32}), (torch.bfloat16, {"D": 176, "V": 56, "R": 32, "H": 6, "G": 1}),
                   (torch.bfloat16, {"D": 64, "V": 200, "R": 48, "impl": 2}), (torch.float32, {"D": 200, "V": 136, "R": 8}),
-                  (torch.bfloat16, {"D": 48, "V": 48, "R": 32, "H": 6, "G": 2, "impl": 2}),
+                  (torch.bfloat16, {"D": 80, "V": 40, "R": 32, "H": 9, "G": 3, "impl": 2}),
                   (torch.bfloat16, {"D": 32, "V": 8, "R": 16, "H": 9, "G": 1}), (torch.bfloat16, {"D": 24, "V": 20, "R": 8, "H": 5, "G": 5})]
     for dt, kw in cases:
         got, want = _attention_case(device, dt, kind, n_ctx, q_lo, standout, size, **kw)
